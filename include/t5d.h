@@ -45,7 +45,10 @@ enum {
 enum {
   T5D_EPI_NONE = 0,      /* C = A·W                                    */
   T5D_EPI_RESIDUAL = 1,  /* C = act(act(A·W) + residual)               */
-  T5D_EPI_GEGLU = 2      /* C[:, f] = act(act(gelu(act(a0))) * act(a1)) */
+  T5D_EPI_GEGLU = 2,     /* C[:, f] = act(act(gelu(act(a0))) * act(a1)) */
+  /* t5d_dense: a0, a1 = gate, up; g = min(a0, limit), u = clamp(a1, +-limit);
+   * C[:, f] = act(g * sigmoid(alpha g) * (u + 1)) */
+  T5D_EPI_CLAMPED_GLU = 3
 };
 
 /* Output layouts of t5d_gemm_rows. */
@@ -601,6 +604,166 @@ typedef struct {
  * nothing.  Covers the loop without state / logit callbacks. */
 int t5d_temperature_sample_step(void* stream, const t5d_model_step* model,
                                 const t5d_sample_step* sample);
+
+/* ---- decoder-only models with recurrent and windowed layers -----------------
+ * No counterpart in the reference's T5 path.  The residual stream is float32;
+ * sequences are fed in portions of any length (a whole prompt, a piece of one,
+ * one new token), each with a slot in the caches and states. */
+
+/* The tokens of one call: S portions, concatenated.  All arrays on the device. */
+typedef struct {
+  int M, S, max_len;         /* tokens, portions, longest portion */
+  const int32_t* tokens;     /* [M] */
+  const int32_t* tok_pos;    /* [M] position in its sequence */
+  const int32_t* tok_seq;    /* [M] portion it belongs to */
+  const int32_t* seq_off;    /* [S + 1] first token of each portion */
+  const int32_t* seq_start;  /* [S] position of that token */
+  const int32_t* seq_slot;   /* [S] cache / state slot; slots are distinct */
+} t5d_ragged;
+
+/* Bias-free dense layer over any number of rows.  dtype bfloat16: A [M, K] with
+ * rows lda apart, W packed (t5d_pack_weight; K % 32, N % 16), out_dtype bfloat16
+ * (dense rows of N) or float32 (the first n_store columns, rows ldc apart);
+ * float32: W row-major [K, N], dense float32 rows.  epilogue NONE or CLAMPED_GLU
+ * (W a geglu-packed gate | up pair, N both, C [M, N / 2], ldc = N / 2,
+ * n_store = N).  Up to 128 rows run on the kernels of t5d_gemm, more on those of
+ * t5d_gemm_rows. */
+int t5d_dense(void* stream, int dtype, int out_dtype, const void* A, int lda,
+              const void* W, void* C, int ldc, int n_store, int M, int K, int N,
+              int epilogue, float glu_limit, float glu_alpha);
+
+/* out[m] = table[ids[m]] + sinusoid(positions[m]), float32: entry 2i is
+ * sin(p 10000^(-2i/d)), entry 2i + 1 its cosine.  table [V, ld] of dtype, columns
+ * d .. ld - 1 zero; out [M, ld], also written to out2 if given. */
+int t5d_embed_sinusoid(void* stream, int dtype, const void* table,
+                       const int32_t* ids, const int32_t* positions, float* out,
+                       float* out2, int M, int d, int ld, int V);
+
+/* The row kernel between two dense layers of a float32 residual stream x [M, ld]:
+ *   x += rms(y) * y_norm   (y [M, ld] of y_dtype; y_norm NULL: x += y; y NULL: no)
+ *   x += add               (add [d] or NULL)
+ *   out = rms(x) * norm    as dtype, or with x0 [M, ld]: out [M, 2 ld] = x | x0
+ * rms(v) = v / sqrt(mean(v^2) + eps) over the first d columns; the others are
+ * zero.  rows (with y, add NULL): out row m comes from x row rows[m].  out NULL:
+ * only x is updated.  ld a multiple of 8, at most 16384. */
+int t5d_stream_norm(void* stream, int dtype, int y_dtype, const void* y,
+                    const float* y_norm, const float* add, float* x,
+                    const float* norm, const float* x0, const int32_t* rows,
+                    void* out, int M, int d, int ld, float eps);
+
+/* Causal attention of the new tokens over a window of their sequence.
+ * score = scale * q.k - slopes[h] * (i - j) over keys i - window < j <= i
+ * (window 0: all j <= i); softmax with exp(sink[h]) added to the denominator. */
+typedef struct {
+  int dtype, H, G, D, Dv;  /* query heads, key/value heads, key and value size */
+  int ring, window;
+  float scale, eps;
+  const void* proj;        /* [M, ld_proj]: q, k, v at these columns */
+  int ld_proj, off_q, off_k, off_v;
+  const float *q_norm, *k_norm;  /* [D] or NULL: per-head RMS norms */
+  const float *slopes, *sink;    /* [H] or NULL */
+  /* [slots, G, ring, HP], HP = t5d_window_head_pad: position p in row p % ring;
+   * ring a multiple of 64 and (window > 0) at least window - 1 + max_len.  Must
+   * hold finite values; rows outside the window are never weighed. */
+  void *key_ring, *value_ring;
+  void* q_rows;            /* scratch [M, H, HP] */
+  void* out;               /* [M, H * Dv], rows ld_out apart */
+  int ld_out;
+  void* workspace;         /* t5d_window_workspace_bytes(S, ...) or NULL */
+} t5d_window_attention;
+
+int t5d_window_head_pad(int D, int Dv);
+int64_t t5d_window_workspace_bytes(int S, int H, int D, int Dv);
+/* Appends the new keys and values to the ring and attends.  variant 0: the kernel
+ * that suits the call; 1: one token per sequence (bfloat16), 2: tiles of rows
+ * (bfloat16), 3: a wavefront per token and head (any dtype and size). */
+int t5d_window_attention_run(void* stream, const t5d_window_attention* a,
+                             const t5d_ragged* b, int variant);
+
+/* Linear recurrence with a decay per key channel (see recurrence.hip). */
+enum { T5D_DECAY_SIGMOID_POWER = 0, T5D_DECAY_EXP_SOFTPLUS = 1 };
+enum { T5D_GATE_SILU = 0, T5D_GATE_SIGMOID_LOW = 1 };
+typedef struct {
+  int dtype, H, G, D, Dv;  /* head h uses q / k head h / (H / G) */
+  int taps;                /* causal convolution + silu on q, k, v (0: none) */
+  int delta;               /* delta rule instead of u = v */
+  int decay;               /* SIGMOID_POWER: sigmoid(z + bias)^decay_power;
+                              EXP_SOFTPLUS: exp(-exp(A_log) softplus(z + bias)) */
+  int unit;                /* q, k / sqrt(sum of squares + unit_eps) */
+  int gate;                /* of the read-out: silu of projection columns, or
+                              sigmoid of low-rank columns */
+  float q_scale, decay_power, unit_eps, eps;
+  const void* proj;        /* [M, ld_proj] */
+  int ld_proj, off_q, off_k, off_v, off_beta, off_gate;
+  float* low;              /* [M, ld_low]: z at off_z (overwritten), gate */
+  int ld_low, off_z, off_low_gate;
+  const float* decay_bias; /* [H * D] */
+  const float* A_log;      /* [H] */
+  const float* conv;       /* [2 G D + H Dv, taps]: q, k, v channels */
+  const float* norm;       /* [Dv] */
+  void* conv_ring;         /* [slots, taps, 2 G D + H Dv] of dtype */
+  float* state;            /* [slots, H, D, Dv] */
+  void* out;               /* [M, H * Dv], rows ld_out apart */
+  int ld_out;
+  void* workspace;         /* t5d_recurrence_workspace_bytes(M, ...) */
+} t5d_recurrence;
+
+int64_t t5d_recurrence_workspace_bytes(int M, int H, int G, int D, int Dv);
+/* variant 0: the kernels that suit the call; 1: one token per sequence in one
+ * kernel; 2: prepare, scan token by token, finish. */
+int t5d_recurrence_run(void* stream, const t5d_recurrence* a, const t5d_ragged* b,
+                       int variant);
+
+enum { T5D_MIX_WINDOW_ATTENTION = 0, T5D_MIX_RECURRENCE = 1 };
+typedef struct {
+  int mix;
+  int proj_n, low_k, low_n, off_low, out_k, F;
+  /* proj [ld, proj_n]; low (or NULL) [low_k, low_n] applied to proj columns
+   * off_low ..; out [out_k, ld]; glu (or NULL) [ld, 2F] gate | up; down [F, ld] */
+  const void *proj, *low, *out, *glu, *down;
+  float glu_limit, glu_alpha;
+  const float *norm1, *norm1b, *norm2, *norm2b;  /* [d] */
+  void *mix_rows, *ff_rows;  /* activations [M, out_k], [M, F]; padding zero */
+  t5d_window_attention attention;  /* sizes and constants; the buffers of a */
+  t5d_recurrence recurrence;       /* call are filled in by the step */
+} t5d_hybrid_layer;
+
+/* One pass of one layer: looped layers have one entry per pass, each with its own
+ * cache.  enter: first x <- loop_in [x; x0] + enter_add. */
+typedef struct {
+  int layer, enter;
+  const float* enter_add;
+  void *cache0, *cache1;   /* key / value ring, or state / convolution ring */
+} t5d_hybrid_run;
+
+typedef struct {
+  int dtype, d, ld, V, head_n, n_layers, n_runs;
+  float eps;
+  const void *embedding;   /* [V, ld] */
+  const void *loop_in;     /* [2 ld, ld] or NULL */
+  const void *head;        /* [ld, head_n] */
+  const float* final_norm;
+  const t5d_hybrid_layer* layers;  /* HOST arrays */
+  const t5d_hybrid_run* runs;
+  /* activations of a call */
+  float *x, *x0, *low;
+  void *h, *cat, *proj, *q_rows, *y, *workspace;
+  int64_t workspace_bytes;
+  float* trace;            /* NULL or [n_runs, M, ld]: x after every run */
+  const int32_t* gate;     /* as t5d_model_step */
+} t5d_hybrid_model;
+
+/* Runs the tokens of `batch` through the model.  Logits [n_want, V] of the tokens
+ * want_rows[0 .. n_want) (NULL: every token, n_want = M; n_want 0: none). */
+int t5d_hybrid_step(void* stream, const t5d_hybrid_model* model,
+                    const t5d_ragged* batch, const int32_t* want_rows, int n_want,
+                    float* logits);
+
+/* t5d_temperature_sample_step for these models: one token per sequence
+ * (batch->tokens = cur_token, tok_pos = seq_start = cur_index). */
+int t5d_hybrid_sample_step(void* stream, const t5d_hybrid_model* model,
+                           const t5d_ragged* batch, float* logits,
+                           const t5d_sample_step* sample);
 
 /* HIP graph capture on `stream` (must not be the null stream):
  * begin, enqueue any t5d calls, end -> executable graph; launch replays it. */

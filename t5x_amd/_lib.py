@@ -11,7 +11,10 @@ from ctypes import (POINTER, Structure, c_char_p, c_float, c_int, c_int32,
                     c_int64, c_uint, c_uint8, c_void_p)
 
 F32, BF16, I8 = 0, 1, 2
-EPI_NONE, EPI_RESIDUAL, EPI_GEGLU = 0, 1, 2
+EPI_NONE, EPI_RESIDUAL, EPI_GEGLU, EPI_CLAMPED_GLU = 0, 1, 2, 3
+DECAY_SIGMOID_POWER, DECAY_EXP_SOFTPLUS = 0, 1
+GATE_SILU, GATE_SIGMOID_LOW = 0, 1
+MIX_WINDOW_ATTENTION, MIX_RECURRENCE = 0, 1
 OUT_ROWS, OUT_HEADS_KEY, OUT_HEADS_VALUE = 0, 1, 2
 LEAVE_OUT_CROSS_ATTENTION, LEAVE_OUT_SELF_ATTENTION = 1, 2
 
@@ -75,6 +78,60 @@ class SampleStep(Structure):
                ('rescale', c_int), ('topp', c_float)])
 
 
+def _fields(**groups):
+  """[(name, type)] from type='names' groups, in order."""
+  types = {'i': c_int, 'f': c_float, 'p': c_void_p, 'l': c_int64}
+  return [(n, types[k[0]]) for k, names in groups.items()
+          for n in names.split()]
+
+
+class Ragged(Structure):
+  """t5d_ragged."""
+  _fields_ = _fields(i='M S max_len', p='tokens tok_pos tok_seq seq_off '
+                     'seq_start seq_slot')
+
+
+class WindowAttention(Structure):
+  """t5d_window_attention."""
+  _fields_ = _fields(i='dtype H G D Dv ring window', f='scale eps', p='proj',
+                     i2='ld_proj off_q off_k off_v',
+                     p2='q_norm k_norm slopes sink key_ring value_ring q_rows '
+                     'out', i3='ld_out', p3='workspace')
+
+
+class Recurrence(Structure):
+  """t5d_recurrence."""
+  _fields_ = _fields(i='dtype H G D Dv taps delta decay unit gate',
+                     f='q_scale decay_power unit_eps eps', p='proj',
+                     i2='ld_proj off_q off_k off_v off_beta off_gate', p2='low',
+                     i3='ld_low off_z off_low_gate',
+                     p3='decay_bias A_log conv norm conv_ring state out',
+                     i4='ld_out', p4='workspace')
+
+
+class HybridLayer(Structure):
+  """t5d_hybrid_layer."""
+  _fields_ = _fields(i='mix proj_n low_k low_n off_low out_k F',
+                     p='proj low out glu down', f='glu_limit glu_alpha',
+                     p2='norm1 norm1b norm2 norm2b mix_rows ff_rows') + [
+                         ('attention', WindowAttention),
+                         ('recurrence', Recurrence)]
+
+
+class HybridRun(Structure):
+  """t5d_hybrid_run."""
+  _fields_ = _fields(i='layer enter', p='enter_add cache0 cache1')
+
+
+class HybridModel(Structure):
+  """t5d_hybrid_model."""
+  _fields_ = (_fields(i='dtype d ld V head_n n_layers n_runs', f='eps',
+                      p='embedding loop_in head final_norm') +
+              [('layers', POINTER(HybridLayer)), ('runs', POINTER(HybridRun))] +
+              _fields(p='x x0 low h cat proj q_rows y workspace',
+                      l='workspace_bytes', p2='trace gate'))
+
+
 _P = c_void_p
 _SIGNATURES = {
     't5d_gather_step_ids': (c_int, [_P, _P, _P, _P, c_int, c_int]),
@@ -83,6 +140,23 @@ _SIGNATURES = {
                                      POINTER(BeamStep)]),
     't5d_temperature_sample_step': (c_int, [_P, POINTER(ModelStep),
                                             POINTER(SampleStep)]),
+    't5d_dense': (c_int, [_P, c_int, c_int, _P, c_int, _P, _P] + [c_int] * 6 +
+                  [c_float] * 2),
+    't5d_embed_sinusoid': (c_int, [_P, c_int] + [_P] * 5 + [c_int] * 4),
+    't5d_stream_norm': (c_int, [_P, c_int, c_int] + [_P] * 8 + [c_int] * 3 +
+                        [c_float]),
+    't5d_window_head_pad': (c_int, [c_int, c_int]),
+    't5d_window_workspace_bytes': (c_int64, [c_int] * 4),
+    't5d_window_attention_run': (c_int, [_P, POINTER(WindowAttention),
+                                         POINTER(Ragged), c_int]),
+    't5d_recurrence_workspace_bytes': (c_int64, [c_int] * 5),
+    't5d_recurrence_run': (c_int, [_P, POINTER(Recurrence), POINTER(Ragged),
+                                   c_int]),
+    't5d_hybrid_step': (c_int, [_P, POINTER(HybridModel), POINTER(Ragged), _P,
+                                c_int, _P]),
+    't5d_hybrid_sample_step': (c_int, [_P, POINTER(HybridModel),
+                                       POINTER(Ragged), _P,
+                                       POINTER(SampleStep)]),
     't5d_graph_begin': (c_int, [_P]),
     't5d_graph_end': (c_int, [_P, POINTER(c_void_p)]),
     't5d_graph_launch': (c_int, [_P, _P]),
@@ -152,6 +226,24 @@ _SIGNATURES = {
 }
 
 _lib = None
+
+
+def ensure_built():
+  """Builds libt5d.so (make, hipcc) if it is not there: for programs that run
+  from a fresh checkout.  Compiler output goes to standard error; a lock file
+  keeps two first calls from building at once."""
+  import fcntl
+  import subprocess
+  import sys
+  if os.path.exists(LIB_PATH):
+    return
+  csrc = os.path.dirname(LIB_PATH)
+  with open(os.path.join(csrc, '.build.o'), 'w') as lock:
+    fcntl.flock(lock, fcntl.LOCK_EX)
+    if not os.path.exists(LIB_PATH):
+      jobs = os.environ.get('MAX_JOBS') or str(min(16, os.cpu_count() or 1))
+      subprocess.run(['make', '-j' + jobs, '-C', csrc], check=True,
+                     stdin=subprocess.DEVNULL, stdout=sys.stderr)
 
 
 class T5DError(RuntimeError):

@@ -21,6 +21,7 @@ Orbax, partitioned reads) is provided.
 import glob
 import gzip
 import itertools
+import json
 import os
 import re
 import zlib
@@ -167,3 +168,42 @@ def load_params(path: str, step: Optional[int] = None) -> dict:
   """The model parameters (`target`) of a checkpoint as float32 arrays, in the
   tree layout `EncoderDecoderModel.predict_batch` takes."""
   return load_t5x_checkpoint(path, step, restore_dtype=np.float32)['target']
+
+
+_SAFETENSORS_DTYPES = {
+    'F64': np.float64, 'F32': np.float32, 'F16': np.float16, 'I64': np.int64,
+    'I32': np.int32, 'I16': np.int16, 'I8': np.int8, 'U8': np.uint8,
+    'BOOL': np.bool_,
+}
+
+
+def load_safetensors(path: str) -> dict:
+  """The tensors of a safetensors file by name, as NumPy arrays (bfloat16
+  widened to float32, which is exact).  The file is an 8-byte little-endian
+  header length, that many bytes of JSON (name -> dtype, shape, data_offsets
+  into what follows) and the data."""
+  size = os.path.getsize(path)
+  with open(path, 'rb') as fp:
+    head = fp.read(8)
+    n = int.from_bytes(head, 'little')
+    if len(head) < 8 or n > size - 8:
+      raise ValueError(f'{path}: not a safetensors file')
+    header = json.loads(fp.read(n))
+    out = {}
+    for name, info in header.items():
+      if name == '__metadata__':
+        continue
+      lo, hi = info['data_offsets']
+      shape, kind = tuple(info['shape']), info['dtype']
+      dtype = np.dtype(np.uint16 if kind == 'BF16' else
+                       _SAFETENSORS_DTYPES[kind])
+      count = int(np.prod(shape, dtype=np.int64))
+      if lo < 0 or hi - lo != count * dtype.itemsize or 8 + n + hi > size:
+        raise ValueError(f'{path}: tensor {name!r} has data offsets '
+                         f'[{lo}, {hi}) for shape {list(shape)} of {kind}')
+      fp.seek(8 + n + lo)
+      flat = np.frombuffer(fp.read(hi - lo), dtype=dtype)
+      if kind == 'BF16':
+        flat = (flat.astype(np.uint32) << 16).view(np.float32)
+      out[name] = flat.reshape(shape)
+  return out

@@ -90,6 +90,13 @@ template <> struct Act<bf16_t> {
   }
 };
 
+// Load / store of one value of either activation dtype.
+template <typename T> __device__ __forceinline__ float to_f32(T v);
+template <> __device__ __forceinline__ float to_f32<float>(float v) { return v; }
+template <> __device__ __forceinline__ float to_f32<bf16_t>(bf16_t v) {
+  return bf16_to_f32(v);
+}
+
 // Unpack a 16-byte vector of activations into floats.
 __device__ __forceinline__ void unpack16(const uint4& v, float (&f)[8]) {
   f[0] = bf16lo_to_f32(v.x); f[1] = bf16hi_to_f32(v.x);
@@ -232,6 +239,15 @@ __device__ __forceinline__ float gelu_sigmoid_form(float x) {
   return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(y));
 }
 
+// Gated unit with both branches clamped: g = min(gate, limit),
+// u = clamp(up, -limit, limit) -> g * sigmoid(alpha g) * (u + 1).
+__device__ __forceinline__ float clamped_glu(float gate, float up, float limit,
+                                             float alpha) {
+  const float g = fminf(gate, limit);
+  const float u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+}
+
 inline hipStream_t as_stream(void* s) { return reinterpret_cast<hipStream_t>(s); }
 
 // Optional device-side gate.  While a fused multi-kernel entry point is
@@ -255,6 +271,10 @@ extern thread_local const int32_t* tls_gate;
 // its kernel for very wide layers, which keeps the rows resident and streams
 // only the weights.
 bool norm_gemm_is_wide(int w_dtype, int K, int N);
+// The many-row kernels behind t5d_dense (bfloat16, M of any size).
+int launch_dense_rows(hipStream_t s, const void* A, int lda, const void* W,
+                      void* C, int out_f32, int ldc, int n_store, int M, int K,
+                      int N, int epilogue, float glu_limit, float glu_alpha);
 // Embedding rows of the current tokens, read straight from the sequences:
 // ids[r] = seqs[r, *cur_index] (t5d_gather_step_ids + t5d_embed in one kernel).
 int launch_embed_from_seqs(hipStream_t s, int dtype, const void* table,

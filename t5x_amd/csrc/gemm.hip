@@ -109,10 +109,10 @@ gemm_mfma_kernel(GemmArgs g) {
         const int row = m0 + mt * 16 + arow;
         if (NJ > 0)  // rows past the edge are never stored
           aq[slot_][h][mt] = *reinterpret_cast<const uint4*>(
-              g.A + (size_t)min(row, g.M - 1) * g.K + (kt + h) * 32 + akoff);
+              g.A + (size_t)min(row, g.M - 1) * g.lda + (kt + h) * 32 + akoff);
         else if (row < g.M && kt + h < KT)
           aq[slot_][h][mt] = *reinterpret_cast<const uint4*>(
-              g.A + (size_t)row * g.K + (kt + h) * 32 + akoff);
+              g.A + (size_t)row * g.lda + (kt + h) * 32 + akoff);
         else
           aq[slot_][h][mt] = make_uint4(0, 0, 0, 0);
       }
@@ -219,7 +219,7 @@ gemm_mfma_kernel(GemmArgs g) {
     __syncthreads();
   }
 
-  const bool geglu = g.epilogue == T5D_EPI_GEGLU;
+  const bool geglu = is_gated(g.epilogue);
   auto tile_sum = [&](int ml, int nl) -> float {
     const int mt = ml >> 4, i = ml & 3, c = (ml & 15) >> 2;
     const int nn = nl >> 4, l = c * 16 + (nl & 15);
@@ -233,7 +233,7 @@ gemm_mfma_kernel(GemmArgs g) {
   auto finish = [&](int e, float r) {
     const int ml = e / TN, nl = e % TN;
     const int m = m0 + ml, n = nt0 * 16 + nl;
-    if (m >= g.M || n >= g.N) return;
+    if (m >= g.M || n >= g.n_store) return;
     if (geglu && (nl & 8)) return;
     float v = tile_sum(ml, nl);
     float vg = geglu ? tile_sum(ml, nl + 8) : 0.f;
@@ -386,7 +386,7 @@ norm_gemm_kernel(GemmArgs g) {
     for (int i = 0; i < 4; ++i) red[wave][t * 4 + i][lane] = acc[t][i];
   __syncthreads();
 
-  const bool geglu = g.epilogue == T5D_EPI_GEGLU;
+  const bool geglu = is_gated(g.epilogue);
   auto tile_sum = [&](int ml, int nl) -> float {
     const int i = ml & 3, c = (ml & 15) >> 2;
     const int nn = nl >> 4, l = c * 16 + (nl & 15);
@@ -642,8 +642,9 @@ template <int WV, bool NORMED>
 __global__ void __launch_bounds__(64 * WV)
 gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
                 const float* __restrict__ residual, float* __restrict__ C,
-                int M, int K, int N, int epilogue, const int32_t* gate,
-                const float* __restrict__ norm_scale, float eps) {
+                int M, int K, int N, int lda, int epilogue,
+                const int32_t* gate, const float* __restrict__ norm_scale,
+                float eps, float glu_limit, float glu_alpha) {
   static_assert(WV == 4 || WV == 16, "wavefronts per workgroup");
   constexpr int MB = kF32Rows;
   constexpr int RW = WV == 4 ? 4 : 8;  // partial sums held in LDS at once
@@ -652,7 +653,7 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int c = lane & 15, sub = lane >> 4;
-  const bool geglu = epilogue == T5D_EPI_GEGLU;
+  const bool geglu = is_gated(epilogue);
   const int F = N >> 1;
   const int ncols = geglu ? F : N;  // columns of work
   const int n = blockIdx.x * kF32Cols + c;
@@ -666,7 +667,7 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
   const int kq = ((K + WV - 1) / WV + 31) & ~31;
   const int kb = min(K, wave * kq), ke = min(K, kb + kq);
   int k = kb;
-  if ((K & 31) == 0 && ((uintptr_t)A & 15) == 0) {
+  if ((K & 31) == 0 && (lda & 3) == 0 && ((uintptr_t)A & 15) == 0) {
     for (; k + 32 <= ke; k += 32) {
       const int kk = k + 8 * sub;
       float w0[8], w1[8];
@@ -682,7 +683,7 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
         ax[m] = ay[m] = make_float4(0.f, 0.f, 0.f, 0.f);
         if (row < M) {
           const float4* ap =
-              reinterpret_cast<const float4*>(A + (size_t)row * K + kk);
+              reinterpret_cast<const float4*>(A + (size_t)row * lda + kk);
           ax[m] = ap[0];
           ay[m] = ap[1];
         }
@@ -720,7 +721,7 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
 #pragma unroll
     for (int m = 0; m < MB; ++m) {
       const int row = m0 + m;
-      const float a = row < M ? A[(size_t)row * K + k] : 0.f;
+      const float a = row < M ? A[(size_t)row * lda + k] : 0.f;
       if constexpr (normed) ssq[m] = fmaf(a, a, ssq[m]);
       acc0[m] = fmaf(a, w0, acc0[m]);
       acc1[m] = fmaf(a, w1, acc1[m]);
@@ -780,7 +781,10 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
     v *= inv;
     if (geglu) {
       float vg = total(MB + m, l) * inv;
-      C[(size_t)row * F + col] = gelu_tanh(v) * vg;
+      C[(size_t)row * F + col] =
+          epilogue == T5D_EPI_GEGLU
+              ? gelu_tanh(v) * vg
+              : clamped_glu(v, vg, glu_limit, glu_alpha);
     } else {
       if (epilogue == T5D_EPI_RESIDUAL) v += residual[(size_t)row * N + col];
       C[(size_t)row * N + col] = v;
@@ -987,13 +991,15 @@ bool t5d::norm_gemm_is_wide(int w_dtype, int K, int N) {
 static void launch_gemm_f32(hipStream_t s, const float* A, const float* W,
                             const float* residual, float* C, int M, int K,
                             int N, int epilogue, const float* norm_scale,
-                            float eps) {
-  const int ncols = epilogue == T5D_EPI_GEGLU ? N / 2 : N;
+                            float eps, int lda = 0, float glu_limit = 0.f,
+                            float glu_alpha = 0.f) {
+  if (lda == 0) lda = K;
+  const int ncols = is_gated(epilogue) ? N / 2 : N;
   dim3 grid((ncols + kF32Cols - 1) / kF32Cols, (M + kF32Rows - 1) / kF32Rows);
 #define T5D_F32_LAUNCH(WV_, NORMED_)                                          \
   hipLaunchKernelGGL((gemm_f32_kernel<WV_, NORMED_>), grid, dim3(64 * WV_), 0, \
-                     s, A, W, residual, C, M, K, N, epilogue, tls_gate,       \
-                     norm_scale, eps)
+                     s, A, W, residual, C, M, K, N, lda, epilogue, tls_gate,  \
+                     norm_scale, eps, glu_limit, glu_alpha)
   if (K >= 128) {
     if (norm_scale) T5D_F32_LAUNCH(16, true);
     else T5D_F32_LAUNCH(16, false);
@@ -1098,6 +1104,7 @@ extern "C" int t5d_gemm(void* stream, int dtype, int w_dtype, int out_dtype,
                           : nullptr;
     g.C = (char*)C + (size_t)m0 * n_out * out_elem;
     g.M = mc; g.K = K; g.N = N;
+    g.dense_rows();
     g.m_parts = 1;
     g.gate = tls_gate;
     g.epilogue = epilogue;
@@ -1113,6 +1120,60 @@ extern "C" int t5d_gemm(void* stream, int dtype, int w_dtype, int out_dtype,
     }
     T5D_CHECK_LAUNCH("t5d_gemm");
   }
+  return T5D_OK;
+}
+
+extern "C" int t5d_dense(void* stream, int dtype, int out_dtype, const void* A,
+                         int lda, const void* W, void* C, int ldc, int n_store,
+                         int M, int K, int N, int epilogue, float glu_limit,
+                         float glu_alpha) {
+  T5D_REQUIRE(A && W && C, T5D_EINVAL, "t5d_dense: null pointer");
+  T5D_REQUIRE(M > 0 && M < (1 << 28) && K > 0 && N > 0 && lda >= K, T5D_EINVAL,
+              "t5d_dense: M=%d K=%d N=%d lda=%d", M, K, N, lda);
+  T5D_REQUIRE(epilogue == T5D_EPI_NONE || epilogue == T5D_EPI_CLAMPED_GLU,
+              T5D_EINVAL, "t5d_dense: epilogue %d", epilogue);
+  const bool gated = is_gated(epilogue);
+  T5D_REQUIRE(gated ? N % 2 == 0 && ldc == N / 2 && n_store == N
+                    : n_store > 0 && n_store <= N && ldc >= n_store,
+              T5D_EINVAL, "t5d_dense: N=%d ldc=%d n_store=%d epilogue %d", N, ldc,
+              n_store, epilogue);
+  hipStream_t s = as_stream(stream);
+  if (dtype == T5D_F32) {
+    T5D_REQUIRE(out_dtype == T5D_F32 && n_store == N && (gated || ldc == N),
+                T5D_EINVAL,
+                "t5d_dense: float32 writes dense float32 rows (N=%d ldc=%d)", N,
+                ldc);
+    launch_gemm_f32(s, (const float*)A, (const float*)W, nullptr, (float*)C, M, K,
+                    N, epilogue, nullptr, 0.f, lda, glu_limit, glu_alpha);
+    T5D_CHECK_LAUNCH("t5d_dense(f32)");
+    return T5D_OK;
+  }
+  T5D_REQUIRE(dtype == T5D_BF16, T5D_EINVAL, "t5d_dense: dtype %d", dtype);
+  T5D_REQUIRE(out_dtype == T5D_F32
+                  ? !gated
+                  : out_dtype == T5D_BF16 && (gated || (ldc == N && n_store == N)),
+              T5D_EINVAL,
+              "t5d_dense: out_dtype %d with epilogue %d, N=%d ldc=%d n_store=%d",
+              out_dtype, epilogue, N, ldc, n_store);
+  T5D_REQUIRE(K % 32 == 0 && N % 16 == 0 && lda % 8 == 0, T5D_EINVAL,
+              "t5d_dense: K=%d N=%d must tile 32x16, lda=%d", K, N, lda);
+  T5D_REQUIRE((((uintptr_t)A | (uintptr_t)W | (uintptr_t)C) % 16) == 0, T5D_EINVAL,
+              "t5d_dense: operands must be 16-byte aligned");
+  if (M > kMaxRows)
+    return launch_dense_rows(s, A, lda, W, C, out_dtype == T5D_F32, ldc, n_store,
+                             M, K, N, epilogue, glu_limit, glu_alpha);
+  GemmPlan p;
+  if (!plan_big(M, K, N, 2, &p)) p = plan_gemm(M, K, N, 2);
+  GemmArgs g;
+  g.A = (const bf16_t*)A; g.W = W; g.scales = nullptr; g.residual = nullptr;
+  g.C = C; g.M = M; g.K = K; g.N = N; g.m_parts = 1;
+  g.gate = tls_gate; g.epilogue = epilogue; g.out_f32 = out_dtype == T5D_F32;
+  g.norm_scale = nullptr; g.eps = 0.f;
+  g.lda = lda; g.ldc = ldc; g.n_store = n_store;
+  g.glu_limit = glu_limit; g.glu_alpha = glu_alpha;
+  if (p.big) launch_gemm_big(T5D_BF16, p, g, nullptr, s);
+  else launch_mfma<bf16_t>(p, g, s);
+  T5D_CHECK_LAUNCH("t5d_dense");
   return T5D_OK;
 }
 
@@ -1171,6 +1232,7 @@ extern "C" int t5d_gemm_tiled(void* stream, int dtype, int w_dtype,
   g.scales = w_dtype == T5D_I8 ? scales : nullptr;
   g.residual = residual; g.C = C;
   g.M = M; g.K = K; g.N = N; g.m_parts = p.m_parts;
+  g.dense_rows();
   g.gate = tls_gate; g.epilogue = epilogue;
   g.out_f32 = out_dtype == T5D_F32;
   g.norm_scale = nullptr; g.eps = 0.f;
@@ -1252,6 +1314,7 @@ extern "C" int t5d_norm_gemm(void* stream, int dtype, int w_dtype,
   g.scales = w_dtype == T5D_I8 ? scales : nullptr;
   g.residual = nullptr;
   g.C = C; g.M = M; g.K = K; g.N = N;
+  g.dense_rows();
   g.m_parts = (M + 15) / 16;
   g.gate = tls_gate;
   g.epilogue = epilogue;

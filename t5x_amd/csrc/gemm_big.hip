@@ -101,10 +101,10 @@ gemm_big_kernel(GemmArgs g, int k_parts, float* __restrict__ partials) {
         const int row = m0 + mt * 16 + arow;
         if (NJ > 0)  // rows past the edge are never stored
           aq[slot_][h][mt] = *reinterpret_cast<const uint4*>(
-              g.A + (size_t)min(row, g.M - 1) * g.K + (kt + h) * 32 + akoff);
+              g.A + (size_t)min(row, g.M - 1) * g.lda + (kt + h) * 32 + akoff);
         else if (row < g.M && kt + h < kt_hi)
           aq[slot_][h][mt] = *reinterpret_cast<const uint4*>(
-              g.A + (size_t)row * g.K + (kt + h) * 32 + akoff);
+              g.A + (size_t)row * g.lda + (kt + h) * 32 + akoff);
         else
           aq[slot_][h][mt] = make_uint4(0, 0, 0, 0);
       }
@@ -187,7 +187,7 @@ gemm_big_kernel(GemmArgs g, int k_parts, float* __restrict__ partials) {
 
   // Cross-wavefront sums, CH tiles per round: (w0 + w2) + (w1 + w3).  Thread
   // (ml, nl) = (tid / 16, tid % 16) finishes element (ml, nl) of every tile.
-  const bool geglu = g.epilogue == T5D_EPI_GEGLU;
+  const bool geglu = is_gated(g.epilogue);
   const int ml = threadIdx.x >> 4, nl = threadIdx.x & 15;
   const int rl = ((ml >> 2) << 4) + nl, ri = ml & 3;
 #pragma unroll
@@ -205,7 +205,7 @@ gemm_big_kernel(GemmArgs g, int k_parts, float* __restrict__ partials) {
       if (t0 + q >= ACC) continue;
       const int mt = (t0 + q) / NT, nn = (t0 + q) % NT;
       const int m = m0 + mt * 16 + ml, n = (nt0 + nn) * 16 + nl;
-      if (m >= g.M || n >= g.N) continue;
+      if (m >= g.M || n >= g.n_store) continue;
       const int idx = q * 4 + ri;
       float v = (red[0][idx][rl] + red[2][idx][rl]) +
                 (red[1][idx][rl] + red[3][idx][rl]);

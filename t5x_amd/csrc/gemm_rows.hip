@@ -70,6 +70,10 @@ struct RowsGemmArgs {
   int epilogue;            // T5D_EPI_*
   int layout;              // T5D_OUT_*
   int E, Ep, H;            // heads layouts: m = b * E + e, n = h * 64 + d
+  int lda;                 // row stride of A
+  float* C32;              // float32 output rows instead of C (rows layout, no
+  int ldc, n_store;        // epilogue): row stride, columns stored of the N
+  float glu_limit, glu_alpha;  // T5D_EPI_CLAMPED_GLU
 };
 
 __device__ __forceinline__ uint2 pack4(float a, float b, float c, float d) {
@@ -124,8 +128,10 @@ __device__ __forceinline__ void rows_epilogue_values(
 // follow one another through the same piece without a wait in between; the
 // empty asm statements keep the compiler from moving one lane's read above
 // another lane's write (to it they are accesses of unrelated addresses).
+// CLAMPED: the gated epilogue is T5D_EPI_CLAMPED_GLU (first column of a pair:
+// gate, second: up) instead of T5D_EPI_GEGLU.
 constexpr int kRowsStageBytes = 16 * 144;
-template <int NT>
+template <int NT, bool CLAMPED>
 __device__ __forceinline__ void rows_epilogue_staged(
     const RowsGemmArgs& g, const f32x4_r (&acc)[kRowsMT][NT], int m0, int nt0,
     int n_tiles, int lane, char* stage) {
@@ -140,7 +146,32 @@ __device__ __forceinline__ void rows_epilogue_staged(
                  ? *reinterpret_cast<const float4*>(g.scales +
                                                     16 * (nt0 + nt) + 4 * gq)
                  : make_float4(1.f, 1.f, 1.f, 1.f);
-  if (g.epilogue == T5D_EPI_GEGLU) {
+  if (!CLAMPED && g.C32 != nullptr) {
+    // a lane holds 4 consecutive columns of one row: 64 bytes per row and store
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt) {
+      const int m = m0 + 16 * mt + l16;
+      if (m >= g.M) continue;
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt) {
+        if (nt0 + nt >= n_tiles) continue;
+        const int n = 16 * (nt0 + nt) + 4 * gq;
+        float* o = g.C32 + (size_t)m * g.ldc + n;
+        const float4 v = make_float4(acc[mt][nt][0] * sc[nt].x, acc[mt][nt][1] * sc[nt].y,
+                                     acc[mt][nt][2] * sc[nt].z, acc[mt][nt][3] * sc[nt].w);
+        if ((g.ldc & 3) == 0 && n + 4 <= g.n_store) {
+          *reinterpret_cast<float4*>(o) = v;
+        } else {
+          if (n < g.n_store) o[0] = v.x;
+          if (n + 1 < g.n_store) o[1] = v.y;
+          if (n + 2 < g.n_store) o[2] = v.z;
+          if (n + 3 < g.n_store) o[3] = v.w;
+        }
+      }
+    }
+    return;
+  }
+  if (CLAMPED || g.epilogue == T5D_EPI_GEGLU) {
     // tile columns 0..7 are wi_0, 8..15 the matching wi_1 columns: the lanes
     // with gq >= 2 hold the gates of the lanes with gq - 2.  32 output columns.
     // Two v_permlane32_swap hand every lane two (value, gate) pairs — the
@@ -162,12 +193,18 @@ __device__ __forceinline__ void rows_epilogue_staged(
             __float_as_uint(acc[mt][nt][3] * sc[nt].w),
             __float_as_uint(acc[mt][nt][1] * sc[nt].y), false, false);
         // [0]: the value (own in the lower half), [1]: its gate
-        const float h0 =
-            round_bf16(gelu_sigmoid_form(round_bf16(__uint_as_float(a[0])))) *
-            round_bf16(__uint_as_float(a[1]));
-        const float h1 =
-            round_bf16(gelu_sigmoid_form(round_bf16(__uint_as_float(b[0])))) *
-            round_bf16(__uint_as_float(b[1]));
+        float h0, h1;
+        if constexpr (CLAMPED) {
+          h0 = clamped_glu(__uint_as_float(a[0]), __uint_as_float(a[1]),
+                           g.glu_limit, g.glu_alpha);
+          h1 = clamped_glu(__uint_as_float(b[0]), __uint_as_float(b[1]),
+                           g.glu_limit, g.glu_alpha);
+        } else {
+          h0 = round_bf16(gelu_sigmoid_form(round_bf16(__uint_as_float(a[0])))) *
+               round_bf16(__uint_as_float(a[1]));
+          h1 = round_bf16(gelu_sigmoid_form(round_bf16(__uint_as_float(b[0])))) *
+               round_bf16(__uint_as_float(b[1]));
+        }
         *reinterpret_cast<uint32_t*>(stage + l16 * 80 + (8 * nt + col0) * 2) =
             pack_bf16x2(h0, h1);
       }
@@ -234,7 +271,7 @@ __device__ __forceinline__ void rows_epilogue_staged(
 }
 
 // SWAP: weights are the MFMA A operand (C^T is formed).
-template <typename WT, bool SWAP>
+template <typename WT, bool SWAP, bool CLAMPED = false>
 __global__ void __launch_bounds__(256, 2)
 rows_gemm_kernel(RowsGemmArgs g) {
   constexpr int TB = RowsWeightTile<WT>::kTileBytes;
@@ -270,7 +307,7 @@ rows_gemm_kernel(RowsGemmArgs g) {
   for (int i = 0; i < 4; ++i)
     arow[i] = g.A +
               (size_t)min(m_blk * kRowsBM + 16 * (wave + 4 * i) + ld_row, g.M - 1) *
-                  g.K + 8 * ld_piece;
+                  g.lda + 8 * ld_piece;
 #pragma unroll
   for (int i = 0; i < 2; ++i)
     wtile[i] = g.W + (size_t)min(n_blk * (kRowsBN / 16) + wave + 4 * i,
@@ -337,7 +374,7 @@ rows_gemm_kernel(RowsGemmArgs g) {
   if (SWAP) {
     // (the loop ends with a barrier: every wavefront is done with the tiles)
     static_assert(sizeof(s_t[0]) >= 4 * kRowsStageBytes, "stage too small");
-    rows_epilogue_staged<NT>(
+    rows_epilogue_staged<NT, CLAMPED>(
         g, acc, m0, nt0, n_tiles, lane,
         reinterpret_cast<char*>(&s_t[0][0][0]) + wave * kRowsStageBytes);
   } else {
@@ -377,7 +414,7 @@ typedef __attribute__((address_space(1))) const void* glb_ptr_t;
 // wavefronts of 128 x 128 (accumulators in the accumulation registers) lasts
 // 257 us: with one wavefront per SIMD nothing covers the operand reads from
 // LDS.
-template <bool SWAP, int NT, int WN>
+template <bool SWAP, int NT, int WN, bool CLAMPED = false>
 __global__ void __launch_bounds__(128 * WN, WN == 2 ? 2 : 1)
 rows_gemm_direct_kernel(RowsGemmArgs g) {
   constexpr int MT = kRowsMT;
@@ -427,7 +464,7 @@ rows_gemm_direct_kernel(RowsGemmArgs g) {
         g.A +
         (size_t)min(m_blk * kRowsBM + 16 * (wave + WAVES * i) + ld_row,
                     g.M - 1) *
-            g.K + 8 * ld_piece);
+            g.lda + 8 * ld_piece);
 #pragma unroll
   for (int i = 0; i < WL; ++i)
     wtile[i] = g.W + (size_t)min(n_blk * (BN / 16) +
@@ -512,7 +549,7 @@ rows_gemm_direct_kernel(RowsGemmArgs g) {
   if (SWAP) {
     static_assert(sizeof(s_t0) >= WAVES * kRowsStageBytes, "stage too small");
     __syncthreads();  // every wavefront is done with the ring
-    rows_epilogue_staged<NT>(
+    rows_epilogue_staged<NT, CLAMPED>(
         g, acc, m0, nt0, n_tiles, lane,
         reinterpret_cast<char*>(&s_t0[0][0]) + wave * kRowsStageBytes);
   } else {
@@ -550,6 +587,67 @@ extern "C" int t5d_gemm_rows_tile(int w_dtype, int64_t M, int K, int N) {
   if (c192 < best) { best = c192; pick = 3; }
   if (c128 < 0.97 * best) pick = 1;
   return pick;
+}
+
+// Picks the workgroup tile (tile 0) and launches checked arguments.
+static int launch_rows(hipStream_t s, int w_dtype, const RowsGemmArgs& g,
+                       int tile) {
+  const int m_blocks = (g.M + kRowsBM - 1) / kRowsBM;
+  const int n_blocks = (g.N + kRowsBN - 1) / kRowsBN;
+  dim3 grid((unsigned)m_blocks * n_blocks), block(256);
+  const bool swap = g.layout != T5D_OUT_HEADS_VALUE;
+  const int pick = tile ? tile : t5d_gemm_rows_tile(w_dtype, g.M, g.K, g.N);
+  const int wgs192 = m_blocks * ((g.N + 191) / 192),
+            wgs256 = m_blocks * ((g.N + 255) / 256);
+  if (g.epilogue == T5D_EPI_CLAMPED_GLU) {  // bfloat16 weights, rows layout
+    if (g.K >= 64 && pick == 3)
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, 3, 4, true>),
+                         dim3((unsigned)wgs192), dim3(512), 0, s, g);
+    else if (g.K >= 64 && pick == 2)
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 4, true>),
+                         dim3((unsigned)wgs256), dim3(512), 0, s, g);
+    else if (g.K >= 64)
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2, true>), grid,
+                         block, 0, s, g);
+    else
+      hipLaunchKernelGGL((rows_gemm_kernel<bf16_t, true, true>), grid, block, 0,
+                         s, g);
+  } else if (w_dtype == T5D_BF16 && g.K >= 64 && pick == 3) {
+    dim3 wgrid((unsigned)wgs192), wblock(512);
+    if (swap)
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, 3, 4>), wgrid, wblock,
+                         0, s, g);
+    else
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<false, 3, 4>), wgrid, wblock,
+                         0, s, g);
+  } else if (w_dtype == T5D_BF16 && g.K >= 64 && pick == 2) {
+    dim3 wgrid((unsigned)wgs256), wblock(512);
+    if (swap)
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 4>), wgrid,
+                         wblock, 0, s, g);
+    else
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<false, kRowsNT, 4>), wgrid,
+                         wblock, 0, s, g);
+  } else if (w_dtype == T5D_BF16 && g.K >= 64) {
+    if (swap)
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2>), grid,
+                         block, 0, s, g);
+    else
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<false, kRowsNT, 2>), grid,
+                         block, 0, s, g);
+  } else if (w_dtype == T5D_BF16) {
+    if (swap)
+      hipLaunchKernelGGL((rows_gemm_kernel<bf16_t, true>), grid, block, 0, s, g);
+    else
+      hipLaunchKernelGGL((rows_gemm_kernel<bf16_t, false>), grid, block, 0, s, g);
+  } else {
+    if (swap)
+      hipLaunchKernelGGL((rows_gemm_kernel<int8_t, true>), grid, block, 0, s, g);
+    else
+      hipLaunchKernelGGL((rows_gemm_kernel<int8_t, false>), grid, block, 0, s, g);
+  }
+  T5D_CHECK_LAUNCH("t5d_gemm_rows");
+  return T5D_OK;
 }
 
 extern "C" int t5d_gemm_rows(void* stream, int w_dtype, const void* A,
@@ -604,48 +702,24 @@ extern "C" int t5d_gemm_rows_tiled(void* stream, int w_dtype, const void* A,
   g.M = (int)M; g.K = K; g.N = N;
   g.epilogue = epilogue; g.layout = out_layout;
   g.E = E; g.Ep = Ep; g.H = H;
-  const int m_blocks = ((int)M + kRowsBM - 1) / kRowsBM;
-  const int n_blocks = (N + kRowsBN - 1) / kRowsBN;
-  dim3 grid((unsigned)m_blocks * n_blocks), block(256);
-  hipStream_t s = as_stream(stream);
-  const bool swap = out_layout != T5D_OUT_HEADS_VALUE;
-  const int pick = tile ? tile : t5d_gemm_rows_tile(w_dtype, M, K, N);
-  const int wgs192 = m_blocks * ((N + 191) / 192),
-            wgs256 = m_blocks * ((N + 255) / 256);
-  if (w_dtype == T5D_BF16 && K >= 64 && pick == 3) {
-    dim3 wgrid((unsigned)wgs192), wblock(512);
-    if (swap)
-      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, 3, 4>), wgrid, wblock,
-                         0, s, g);
-    else
-      hipLaunchKernelGGL((rows_gemm_direct_kernel<false, 3, 4>), wgrid, wblock,
-                         0, s, g);
-  } else if (w_dtype == T5D_BF16 && K >= 64 && pick == 2) {
-    dim3 wgrid((unsigned)wgs256), wblock(512);
-    if (swap)
-      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 4>), wgrid,
-                         wblock, 0, s, g);
-    else
-      hipLaunchKernelGGL((rows_gemm_direct_kernel<false, kRowsNT, 4>), wgrid,
-                         wblock, 0, s, g);
-  } else if (w_dtype == T5D_BF16 && K >= 64) {
-    if (swap)
-      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2>), grid,
-                         block, 0, s, g);
-    else
-      hipLaunchKernelGGL((rows_gemm_direct_kernel<false, kRowsNT, 2>), grid,
-                         block, 0, s, g);
-  } else if (w_dtype == T5D_BF16) {
-    if (swap)
-      hipLaunchKernelGGL((rows_gemm_kernel<bf16_t, true>), grid, block, 0, s, g);
-    else
-      hipLaunchKernelGGL((rows_gemm_kernel<bf16_t, false>), grid, block, 0, s, g);
-  } else {
-    if (swap)
-      hipLaunchKernelGGL((rows_gemm_kernel<int8_t, true>), grid, block, 0, s, g);
-    else
-      hipLaunchKernelGGL((rows_gemm_kernel<int8_t, false>), grid, block, 0, s, g);
-  }
-  T5D_CHECK_LAUNCH("t5d_gemm_rows");
-  return T5D_OK;
+  g.lda = K; g.C32 = nullptr; g.ldc = g.n_store = N;
+  g.glu_limit = g.glu_alpha = 0.f;
+  return launch_rows(as_stream(stream), w_dtype, g, tile);
+}
+
+int t5d::launch_dense_rows(hipStream_t s, const void* A, int lda,
+                           const void* W, void* C, int out_f32, int ldc,
+                           int n_store, int M, int K, int N, int epilogue,
+                           float glu_limit, float glu_alpha) {
+  RowsGemmArgs g;
+  g.A = (const bf16_t*)A; g.W = (const char*)W;
+  g.scales = nullptr; g.residual = nullptr;
+  g.C = out_f32 ? nullptr : (bf16_t*)C;
+  g.C32 = out_f32 ? (float*)C : nullptr;
+  g.M = M; g.K = K; g.N = N;
+  g.epilogue = epilogue; g.layout = T5D_OUT_ROWS;
+  g.E = g.Ep = g.H = 0;
+  g.lda = lda; g.ldc = ldc; g.n_store = n_store;
+  g.glu_limit = glu_limit; g.glu_alpha = glu_alpha;
+  return launch_rows(s, T5D_BF16, g, 0);
 }

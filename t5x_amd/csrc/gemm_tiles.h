@@ -71,21 +71,38 @@ struct GemmArgs {
   int out_f32;
   const bf16_t* norm_scale;  // norm_gemm_kernel: [K] layer-norm scale
   float eps;
+  // Row strides of A and of a C that is not gated, and how many of the N columns
+  // are stored (gemm_mfma_kernel and gemm_big_kernel; norm_gemm_kernel takes
+  // dense rows).
+  int lda, ldc, n_store;
+  float glu_limit, glu_alpha;  // T5D_EPI_CLAMPED_GLU
+  // rows of K (N) elements, every column stored
+  void dense_rows() { lda = K; ldc = N; n_store = N; glu_limit = glu_alpha = 0.f; }
 };
+
+// Epilogues that pair two weight columns into one output column.
+__host__ __device__ __forceinline__ bool is_gated(int epilogue) {
+  return epilogue == T5D_EPI_GEGLU || epilogue == T5D_EPI_CLAMPED_GLU;
+}
 
 // Apply scale + epilogue to one finished column (pair) of row m; `res` is the
 // residual element (fetched early by the caller).
 __device__ __forceinline__ void store_result(const GemmArgs& g, int m, int n,
                                              float v, float v_gate, float res) {
-  if (g.epilogue == T5D_EPI_GEGLU) {
+  if (is_gated(g.epilogue)) {
     const int f = (n >> 4) * 8 + (n & 7);
     const int F = g.N >> 1;
+    if (g.epilogue == T5D_EPI_CLAMPED_GLU) {
+      reinterpret_cast<bf16_t*>(g.C)[(size_t)m * F + f] =
+          f32_to_bf16(clamped_glu(v, v_gate, g.glu_limit, g.glu_alpha));
+      return;
+    }
     float a0 = round_bf16(v), a1 = round_bf16(v_gate);
     float h = round_bf16(round_bf16(gelu_sigmoid_form(a0)) * a1);
     reinterpret_cast<bf16_t*>(g.C)[(size_t)m * F + f] = f32_to_bf16(h);
     return;
   }
-  const size_t o = (size_t)m * g.N + n;
+  const size_t o = (size_t)m * g.ldc + n;
   if (g.out_f32) {
     reinterpret_cast<float*>(g.C)[o] = v;
     return;

@@ -43,6 +43,22 @@ int check_model(const t5d_model_step* m) {
   return T5D_OK;
 }
 
+int check_sample(const char* name, const t5d_sample_step* s) {
+  T5D_REQUIRE(s && s->sequences && s->cur_index && s->cur_token && s->ended &&
+                  s->log_prob && s->max_decode_len && s->initial_eos_count &&
+                  s->temperature && s->step_count && s->tokens &&
+                  s->token_logprobs && s->all_ended && s->keep_going,
+              T5D_EINVAL, "%s: null buffer", name);
+  T5D_REQUIRE(s->S > 2 && s->topk >= 0 && s->topp >= 0.f &&
+                  (s->gumbel == nullptr || s->noise_ring > 0),
+              T5D_EINVAL,
+              "%s: S=%d topk=%d topp=%f ring=%d", name, s->S, s->topk,
+              (double)s->topp, s->noise_ring);
+  T5D_REQUIRE(!(s->topk > 0 && s->topp > 0.f), T5D_EINVAL,
+              "At most one of `topp` or `topk` may be non-zero.");
+  return T5D_OK;
+}
+
 }  // namespace
 
 namespace {
@@ -228,28 +244,31 @@ extern "C" int t5d_temperature_sample_step(void* stream,
                                            const t5d_model_step* m,
                                            const t5d_sample_step* s) {
   T5D_TRY(check_model(m));
-  T5D_REQUIRE(s && s->sequences && s->cur_index && s->cur_token && s->ended &&
-                  s->log_prob && s->max_decode_len && s->initial_eos_count &&
-                  s->temperature && s->step_count && s->tokens &&
-                  s->token_logprobs && s->all_ended && s->keep_going,
-              T5D_EINVAL, "t5d_temperature_sample_step: null buffer");
+  T5D_TRY(check_sample("t5d_temperature_sample_step", s));
   T5D_REQUIRE(m->gate == s->keep_going, T5D_EINVAL,
               "t5d_temperature_sample_step: the model gate must be the loop "
               "flag");
   T5D_REQUIRE(m->pending_src == nullptr, T5D_EINVAL,
               "t5d_temperature_sample_step: sampling rows are never reordered");
-  T5D_REQUIRE(s->S > 2 && s->topk >= 0 && s->topp >= 0.f &&
-                  (s->gumbel == nullptr || s->noise_ring > 0),
-              T5D_EINVAL,
-              "t5d_temperature_sample_step: S=%d topk=%d topp=%f ring=%d", s->S,
-              s->topk, (double)s->topp, s->noise_ring);
-  T5D_REQUIRE(!(s->topk > 0 && s->topp > 0.f), T5D_EINVAL,
-              "At most one of `topp` or `topk` may be non-zero.");
   T5D_TRY(decoder_step_impl(stream, m, s->cur_token, nullptr, nullptr, 0,
                             false));
   GateScope gate(s->keep_going);
   return launch_sample_step(as_stream(stream), m->logits, s, m->R, m->V,
                             m->cache_index, m->NL);
+}
+
+extern "C" int t5d_hybrid_sample_step(void* stream, const t5d_hybrid_model* m,
+                                      const t5d_ragged* b, float* logits,
+                                      const t5d_sample_step* s) {
+  T5D_REQUIRE(m && b && logits, T5D_EINVAL, "t5d_hybrid_sample_step: null buffer");
+  T5D_REQUIRE(m->gate == (s ? s->keep_going : nullptr), T5D_EINVAL,
+              "t5d_hybrid_sample_step: the model gate must be the loop flag");
+  T5D_TRY(check_sample("t5d_hybrid_sample_step", s));
+  T5D_REQUIRE(b->M == b->S && b->max_len == 1, T5D_EINVAL,
+              "t5d_hybrid_sample_step: one token per sequence");
+  T5D_TRY(t5d_hybrid_step(stream, m, b, nullptr, b->M, logits));
+  GateScope gate(s->keep_going);
+  return launch_sample_step(as_stream(stream), logits, s, b->M, m->V, nullptr, 0);
 }
 
 extern "C" int t5d_measure_leave_out(int mask) {

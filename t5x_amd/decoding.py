@@ -315,14 +315,18 @@ def _sample_setup(inputs, cache, tokens_to_logits, num_decodes, cache_offset,
   # A step function that can run whole iterations on the device exposes
   # `fused_sample_step(...)`; it then owns the caches of all rows (the incoming
   # cache must be the untouched zero cache, which is then not even expanded).
+  # (`fused_takes_cache`: it copies the expanded cache instead, and continues
+  # from whatever a prefill has left there.)
+  takes_cache = getattr(tokens_to_logits, 'fused_takes_cache', False)
   use_fused = (getattr(tokens_to_logits, 'fused_sample_step', None) is not None
-               and getattr(cache, 'fresh', False) and initial_index is None and
+               and (takes_cache or (getattr(cache, 'fresh', False) and
+                                    initial_index is None)) and
                cache_offset == getattr(tokens_to_logits, 'cache_offset', 0) and
                state_callback_fn is None and logit_callback_fn is None)
   if not use_fused:
     _check_cache_room(cache, inputs.shape[1],
                       expect_empty=initial_index is None)
-  if use_fused:
+  if use_fused and not takes_cache:
     expanded_inputs = (flat_batch_beam_expand(inputs, num_decodes)
                        if num_decodes > 1 else inputs)
     expanded_cache = cache
@@ -590,7 +594,9 @@ class SampleLoop(_InFlight):
     self.step = 0
     self.fused = None
     if use_fused:
+      takes_cache = getattr(tokens_to_logits, 'fused_takes_cache', False)
       self.fused = tokens_to_logits.fused_sample_step(
+          **({'cache': cache} if takes_cache else {}),
           sequences=self.sequences, cur_index=self.cur_index,
           cur_token=self.cur_token, ended=self.ended, log_prob=self.log_prob,
           max_decode_len=self.mdl, initial_eos_count=self.eos0,

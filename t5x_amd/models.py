@@ -60,17 +60,14 @@ class StepFunction:
         max_decode_length=self.max_decode_length)
 
 
-class EncoderDecoderModel:
-  """t5x/models.py:364-758, inference methods only."""
+class BatchPredictor:
+  """What the models share: a decode function, batches predicted one by one or
+  several in flight.  A subclass defines predict_batch_with_aux and
+  begin_predict_batch_with_aux."""
 
-  def __init__(self, module, input_vocabulary: Any = None,
-               output_vocabulary: Any = None, optimizer_def: Any = None,
-               decode_fn: Callable = decoding.beam_search,
-               default_decoder_params: Optional[DecoderParams] = None,
-               **unused_training_kwargs):
-    del optimizer_def, unused_training_kwargs
+  def _init_decoding(self, module, output_vocabulary, decode_fn,
+                     default_decoder_params):
     self.module = module
-    self._input_vocabulary = input_vocabulary or Vocabulary()
     self._output_vocabulary = output_vocabulary or Vocabulary()
     self._decode_fn = decode_fn
     self._default_decoder_params = default_decoder_params or DecoderParams()
@@ -82,6 +79,94 @@ class EncoderDecoderModel:
   @property
   def output_vocabulary(self):
     return self._output_vocabulary
+
+  def predict_batch(self, params, batch, rng=None):
+    """t5x/models.py:177-193."""
+    return self.predict_batch_with_aux(params=params, batch=batch, rng=rng)[0]
+
+  def begin_predict_batch(self, params, batch, rng=None, in_flight=False):
+    """predict_batch set up and started but not waited for -> Prediction."""
+    return self.begin_predict_batch_with_aux(params, batch, rng,
+                                             in_flight=in_flight).first()
+
+  # the methods a caller may hold instead of which begin_predict_batch can be
+  # called: a subclass that overrides one of them without overriding the
+  # begin variant must be called through its override (infer._begin_of)
+  begin_predict_batch.stands_for = ('predict_batch', 'predict_batch_with_aux')
+
+  def predict_batches(self, params, batches, rngs=None,
+                      in_flight: Optional[int] = None, **kwargs):
+    """predict_batch_with_aux over an iterable of batches, yielding each
+    batch's result in order, with up to `in_flight` decodes running on the
+    device at once (each on its own streams): the device spends most of a
+    decode step of one batch waiting on dependent launches, which the other
+    batches' steps fill.  Every batch's result is what predict_batch_with_aux
+    returns for it alone.  `rngs`: one per batch, or None.  in_flight None:
+    batches_in_flight() of the first batch.  With decode functions other than
+    beam_search / temperature_sample the batches run one after the other."""
+    rngs = iter(rngs) if rngs is not None else None
+    batches = iter(batches)
+    try:
+      first = next(batches)
+    except StopIteration:
+      return
+    if in_flight is None:
+      in_flight = self.batches_in_flight(first, kwargs.get('num_decodes'))
+
+    def begin(batch):
+      rng = next(rngs) if rngs is not None else None
+      return self.begin_predict_batch_with_aux(
+          params, batch, rng, in_flight=in_flight > 1, **kwargs)
+
+    yield from infer.map_in_flight(
+        begin, itertools.chain([first], batches), in_flight)
+
+  def _begin_decode(self, inputs, cache, tokens_to_logits, num_decodes, rng,
+                    decoder_params, cache_offset, return_all_decodes,
+                    initial_index=None):
+    """Starts the decode function (t5x/models.py:716-758) -> Prediction."""
+    if decoder_params is None:
+      decoder_params = {}
+    if initial_index is not None:
+      decoder_params['initial_index'] = initial_index
+    if rng is not None:
+      if decoder_params.get('decode_rng') is not None:
+        raise ValueError(
+            f'Got RNG both from the `rng` argument ({rng}) and'
+            " `decoder_params['decode_rng']`"
+            f' ({decoder_params["decode_rng"]}). Please specify one or the'
+            ' other.')
+      decoder_params['decode_rng'] = rng
+    if 'eos_id' not in decoder_params:
+      decoder_params['eos_id'] = self.output_vocabulary.eos_id or 1
+    decode_kwargs = dict(
+        inputs=inputs, cache=cache, tokens_to_logits=tokens_to_logits,
+        num_decodes=num_decodes, cache_offset=cache_offset, **decoder_params)
+    begin, bound = _begin_of(self._decode_fn)
+    if begin is None:  # some other decode function: it runs here and now
+      decode = decoding.Decode(_Ran(self._decode_fn(**decode_kwargs)))
+    else:
+      decode = begin(**bound, **decode_kwargs)
+      decode.start()
+    return Prediction(decode, return_all_decodes)
+
+
+class EncoderDecoderModel(BatchPredictor):
+  """t5x/models.py:364-758, inference methods only."""
+
+  def __init__(self, module, input_vocabulary: Any = None,
+               output_vocabulary: Any = None, optimizer_def: Any = None,
+               decode_fn: Callable = decoding.beam_search,
+               default_decoder_params: Optional[DecoderParams] = None,
+               **unused_training_kwargs):
+    del optimizer_def, unused_training_kwargs
+    self._input_vocabulary = input_vocabulary or Vocabulary()
+    self._init_decoding(module, output_vocabulary, decode_fn,
+                        default_decoder_params)
+
+  # defined here so that a subclass overriding predict_batch_with_aux alone is
+  # told apart (stands_for)
+  begin_predict_batch = BatchPredictor.begin_predict_batch
 
   def _compute_logits_from_slice(self, decoding_state, params, encoded_inputs,
                                  raw_inputs, max_decode_length):
@@ -120,10 +205,6 @@ class EncoderDecoderModel:
       raise NotImplementedError('module.decode has no `prefill` argument')
     return cache, None
 
-  def predict_batch(self, params, batch, rng=None):
-    """t5x/models.py:177-193."""
-    return self.predict_batch_with_aux(params=params, batch=batch, rng=rng)[0]
-
   def predict_batch_with_aux(
       self, params, batch, rng=None,
       decoder_params: Optional[MutableMapping[str, Any]] = None,
@@ -133,43 +214,6 @@ class EncoderDecoderModel:
     return self.begin_predict_batch_with_aux(
         params, batch, rng, decoder_params, return_all_decodes, num_decodes,
         prompt_with_targets).result()
-
-  def begin_predict_batch(self, params, batch, rng=None, in_flight=False):
-    """predict_batch set up and started but not waited for -> Prediction."""
-    return self.begin_predict_batch_with_aux(params, batch, rng,
-                                             in_flight=in_flight).first()
-
-  # the methods a caller may hold instead of which begin_predict_batch can be
-  # called: a subclass that overrides one of them without overriding the
-  # begin variant must be called through its override (infer._begin_of)
-  begin_predict_batch.stands_for = ('predict_batch', 'predict_batch_with_aux')
-
-  def predict_batches(self, params, batches, rngs=None,
-                      in_flight: Optional[int] = None, **kwargs):
-    """predict_batch_with_aux over an iterable of batches, yielding each
-    batch's result in order, with up to `in_flight` decodes running on the
-    device at once (each on its own streams): the device spends most of a
-    decode step of one batch waiting on dependent launches, which the other
-    batches' steps fill.  Every batch's result is what predict_batch_with_aux
-    returns for it alone.  `rngs`: one per batch, or None.  in_flight None:
-    batches_in_flight() of the first batch.  With decode functions other than
-    beam_search / temperature_sample the batches run one after the other."""
-    rngs = iter(rngs) if rngs is not None else None
-    batches = iter(batches)
-    try:
-      first = next(batches)
-    except StopIteration:
-      return
-    if in_flight is None:
-      in_flight = self.batches_in_flight(first, kwargs.get('num_decodes'))
-
-    def begin(batch):
-      rng = next(rngs) if rngs is not None else None
-      return self.begin_predict_batch_with_aux(
-          params, batch, rng, in_flight=in_flight > 1, **kwargs)
-
-    yield from infer.map_in_flight(
-        begin, itertools.chain([first], batches), in_flight)
 
   def batches_in_flight(self, batch, num_decodes=None) -> int:
     """How many batches shaped like `batch` to keep decoding at once: as many
@@ -233,36 +277,139 @@ class EncoderDecoderModel:
         self, params, expand(encoded_inputs), expand(encoder_input_tokens),
         decoder_input_tokens.shape[1], in_flight=in_flight)
 
-    if decoder_params is None:
-      decoder_params = {}
-    if initial_index is not None:
-      decoder_params['initial_index'] = initial_index
-    if rng is not None:
-      if decoder_params.get('decode_rng') is not None:
-        raise ValueError(
-            f'Got RNG both from the `rng` argument ({rng}) and'
-            " `decoder_params['decode_rng']`"
-            f' ({decoder_params["decode_rng"]}). Please specify one or the'
-            ' other.')
-      decoder_params['decode_rng'] = rng
-
     scanned = hasattr(self.module, 'scan_layers') and self.module.scan_layers
-    if 'eos_id' not in decoder_params:
-      decoder_params['eos_id'] = self.output_vocabulary.eos_id or 1
-    decode_kwargs = dict(
-        inputs=decoder_prompt_inputs, cache=cache,
-        tokens_to_logits=tokens_ids_to_logits, num_decodes=num_decodes,
-        cache_offset=1 if scanned else 0, **decoder_params)
-    begin, bound = _begin_of(self._decode_fn)
-    if begin is None:  # some other decode function: it runs here and now
-      decode = decoding.Decode(_Ran(self._decode_fn(**decode_kwargs)))
-    else:
-      decode = begin(**bound, **decode_kwargs)
-      decode.start()
-    return Prediction(decode, return_all_decodes)
+    return self._begin_decode(decoder_prompt_inputs, cache, tokens_to_logits,
+                              num_decodes, rng, decoder_params,
+                              1 if scanned else 0, return_all_decodes,
+                              initial_index)
 
 
 EncoderDecoderModel.begin_predict_batch_with_aux.stands_for = (
+    'predict_batch_with_aux',)
+
+
+class PrefilledStepFunction:
+  """`tokens_ids_to_logits` over a cache that already holds the prompts: one new
+  token per row.  A fused loop copies the (expanded) cache it is handed."""
+
+  cache_offset = 0
+  fused_takes_cache = True
+
+  def __init__(self, module, params):
+    self.module, self.params = module, params
+
+  def fused_sample_step(self, **kw):
+    return self.module.make_fused_sample_step(self.params, **kw)
+
+  def __call__(self, decoding_state):
+    logits = self.module.decode_step(self.params, decoding_state.cache,
+                                     decoding_state.cur_token)
+    return logits, decoding_state.cache
+
+
+class DecoderOnlyModel(BatchPredictor):
+  """Decoder-only language models (t5x/models.py, DecoderOnlyModel; inference
+  methods): the prompt is prefilled in one pass, then the decode function
+  continues it."""
+
+  def __init__(self, module, vocabulary: Any = None,
+               output_vocabulary: Any = None,
+               decode_fn: Callable = decoding.temperature_sample,
+               default_decoder_params: Optional[DecoderParams] = None,
+               **unused_training_kwargs):
+    del unused_training_kwargs
+    self._init_decoding(module, output_vocabulary or vocabulary, decode_fn,
+                        default_decoder_params)
+
+  # defined here so that a subclass overriding predict_batch_with_aux alone is
+  # told apart (stands_for)
+  begin_predict_batch = BatchPredictor.begin_predict_batch
+
+  def predict_batch_with_aux(
+      self, params, batch, rng=None,
+      decoder_params: Optional[MutableMapping[str, Any]] = None,
+      return_all_decodes: bool = None, num_decodes: int = None):
+    """batch: decoder_input_tokens [B, L], the prompt of every row at its start,
+    and decoder_causal_attention [B, L], one where the row holds a prompt token.
+    Returns (decodes [B, L], {'scores'}): column i of a row is the token at
+    position i + 1, the prompt's own from its second token on, then what was
+    generated."""
+    return self.begin_predict_batch_with_aux(
+        params, batch, rng, decoder_params, return_all_decodes,
+        num_decodes).result()
+
+  def batches_in_flight(self, batch, num_decodes=None) -> int:
+    """How many batches shaped like `batch` to keep decoding at once."""
+    if _begin_of(self._decode_fn)[0] is None:
+      return 1
+    if num_decodes is None:
+      num_decodes = self._default_decoder_params.num_decodes
+    B, L = np.shape(batch['decoder_input_tokens'])[:2]
+    return self.module.batches_in_flight(B, num_decodes, L)
+
+  def begin_predict_batch_with_aux(
+      self, params, batch, rng=None,
+      decoder_params: Optional[MutableMapping[str, Any]] = None,
+      return_all_decodes: bool = None, num_decodes: int = None,
+      in_flight: bool = False):
+    """predict_batch_with_aux up to and including the start of its decode loop
+    -> Prediction."""
+    del in_flight
+    if return_all_decodes is None:
+      return_all_decodes = self._default_decoder_params.return_all_decodes
+    if num_decodes is None:
+      num_decodes = self._default_decoder_params.num_decodes
+    host = lambda x: np.asarray(x.cpu() if isinstance(x, torch.Tensor) else x)
+    tokens = host(batch['decoder_input_tokens']).astype(np.int32)
+    prompt = host(batch['decoder_causal_attention']) != 0
+    lengths = prompt.sum(axis=1).astype(np.int32)
+    B, L = tokens.shape
+    if (lengths < 1).any() or not (prompt == (np.arange(L)[None, :] <
+                                              lengths[:, None])).all():
+      raise ValueError('decoder_causal_attention must mark a prefix of at least '
+                       'one token in every row')
+    inputs = tokens * prompt
+    # The last prompt token is the first one the decode loop feeds.
+    initial_index = lengths - 1
+    cache = self.module.init_cache(B, L + 2,
+                                   portion=max(1, int(initial_index.max())))
+    self.module.prefill(params, cache, inputs, initial_index)
+    return self._begin_decode(
+        inputs, cache, PrefilledStepFunction(self.module, params), num_decodes,
+        rng, decoder_params, 0, return_all_decodes, initial_index)
+
+  def generate(self, params, prompts, max_tokens: int, batch_size: int = 16,
+               num_decodes: int = 1, seed: int = 0):
+    """Continues lists of token ids by up to `max_tokens` tokens each, yielding
+    the new tokens of each prompt in order (cut after the first end token)."""
+    prompts = [list(p) for p in prompts]
+    eos = self.output_vocabulary.eos_id
+
+    def batches():
+      for at in range(0, len(prompts), batch_size):
+        part = prompts[at:at + batch_size]
+        L = max(len(p) for p in part) + max_tokens
+        tokens = np.zeros((len(part), L), np.int32)
+        mask = np.zeros((len(part), L), np.int32)
+        for r, p in enumerate(part):
+          tokens[r, :len(p)] = p
+          mask[r, :len(p)] = 1
+        yield {'decoder_input_tokens': tokens, 'decoder_causal_attention': mask}
+
+    rngs = itertools.count(seed)
+    done = 0
+    for decodes, _ in self.predict_batches(params, batches(), rngs,
+                                           num_decodes=num_decodes):
+      for row in infer._to_numpy(decodes):
+        n = len(prompts[done])
+        new = row[n - 1:n - 1 + max_tokens].tolist()
+        if eos in new:
+          new = new[:new.index(eos) + 1]
+        yield new
+        done += 1
+
+
+DecoderOnlyModel.begin_predict_batch_with_aux.stands_for = (
     'predict_batch_with_aux',)
 
 

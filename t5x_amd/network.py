@@ -308,7 +308,112 @@ def _plain_caches(kv, layout, n):
   return kv[0], kv[1]
 
 
-class Transformer:
+class DecodeContexts:
+  """What a module that drives decode loops on the device keeps between them:
+  pools of decode contexts (caches, state, captured graphs) and the streams they
+  run on.  A module has `device` (None: the GPU) and `_beam_ctx = {}`."""
+
+  # How many decode streams the device runs side by side.  None: the
+  # environment variable T5X_AMD_STREAMS_SIDE_BY_SIDE if set, else measured
+  # once per device and process (streams_side_by_side).  A fixed value makes
+  # the number of batch lanes and of batches in flight, hence what is
+  # captured and held, the same in every run; results never depend on it.
+  side_by_side = None
+
+  def _dev(self):
+    if self.device is None:
+      if not torch.cuda.is_available():
+        raise RuntimeError('t5x_amd needs a GPU (no CPU fallback)')
+      self.device = torch.device('cuda')
+    return self.device
+
+  # Decode contexts of one (weights, shapes, options) key that are kept for
+  # re-binding: more than one only when several decodes are in flight at once.
+  MAX_CONTEXTS_PER_KEY = 4
+
+  def _decode_context(self, key, w, owner, make, rebind):
+    """A decode context for `owner` (the loop object that will drive it): a
+    kept one of this key that no live, unfinished loop owns any more, re-bound,
+    or a new one.  Contexts are kept in small pools per key, so that a caller
+    who keeps several decodes in flight (each on its own stream) pays for
+    their allocation and graph capture once.  make(slot) builds a context for
+    pool slot `slot`, whose stream is decode_stream(slot)."""
+    pool = self._beam_ctx.get(key)
+    if pool and pool[0].w is not w:  # an id reused by other weights
+      del self._beam_ctx[key]
+      pool = None
+    if pool is None:
+      if len(self._beam_ctx) >= 2:  # a context holds the caches: keep few
+        self._beam_ctx.pop(next(iter(self._beam_ctx)))
+      pool = self._beam_ctx[key] = []
+    for ctx in pool:
+      if ctx.is_free():
+        rebind(ctx)
+        ctx.claim(owner)
+        return ctx
+    ctx = make(len(pool))
+    ctx.claim(owner)
+    if len(pool) < self.MAX_CONTEXTS_PER_KEY:
+      pool.append(ctx)
+    return ctx
+
+  def streams_side_by_side(self) -> int:
+    """How many decode streams the device runs side by side.  One hardware
+    queue of the process serves the default stream, the others are dealt to
+    the streams in turn, and queues beyond the fourth share command
+    processors (3 decodes in flight pay with the runtime's default of 4
+    queues, 4 with GPU_MAX_HW_QUEUES=8 or more, a fifth never).  Which queue a
+    stream got cannot be asked, so it is measured once per device when the
+    decode streams are made: the first n streams count when n short busy
+    kernels, one per stream, take about as long as one."""
+    import os
+    fixed = self.side_by_side
+    if fixed is None and os.environ.get('T5X_AMD_STREAMS_SIDE_BY_SIDE'):
+      fixed = int(os.environ['T5X_AMD_STREAMS_SIDE_BY_SIDE'])
+    if fixed is not None:
+      return max(1, min(int(fixed), self.MAX_CONTEXTS_PER_KEY))
+    self.decode_stream(0, measure=True)
+    key = self._stream_key()
+    measured = _DECODE_STREAMS_SIDE_BY_SIDE.get(key)
+    if measured is not None:
+      return measured
+    try:
+      queues = int(os.environ.get('GPU_MAX_HW_QUEUES', '4'))
+    except ValueError:
+      queues = 4
+    return 4 if queues >= 8 else 3
+
+  def _stream_key(self):
+    key = torch.device(self._dev()).index
+    return torch.cuda.current_device() if key is None else key
+
+  def decode_stream(self, slot, measure=False):
+    """The stream of the decode contexts in pool slot `slot` (with batch
+    lanes: of lane l of the context in slot s, at s * lanes + l).  The device
+    runs streams side by side only when they sit on different hardware
+    queues, of which a process has few (4 by default) and which streams are
+    given in turn as they are first used; so the decode streams of a device
+    are made once per process, together, and each is used once right away:
+    consecutive slots then sit on different queues whatever streams the
+    caller, or another model on the same device, makes later."""
+    dev, key = self._dev(), self._stream_key()
+    streams = _DECODE_STREAMS.get(key)
+    if streams is None:
+      streams = [torch.cuda.Stream(device=dev)
+                 for _ in range(self.MAX_CONTEXTS_PER_KEY)]
+      touch = torch.zeros((16,), dtype=torch.int32, device=dev)
+      torch.cuda.current_stream().synchronize()
+      for stream in streams:
+        with torch.cuda.stream(stream):
+          touch.zero_()
+        stream.synchronize()
+      _DECODE_STREAMS[key] = streams
+    if measure and key not in _DECODE_STREAMS_SIDE_BY_SIDE:
+      _DECODE_STREAMS_SIDE_BY_SIDE[key] = _measure_side_by_side(streams)
+    return streams[slot % len(streams)]
+
+
+class Transformer(DecodeContexts):
   """network.Transformer with `apply(variables, *args, method=..., **kwargs)`.
 
   `variables['params']` is the reference parameter tree (NumPy or torch
@@ -324,13 +429,6 @@ class Transformer:
   # decode on its own, 1 when several batches are in flight (those fill the
   # device better than lanes do, and streams that run side by side are few).
   decode_lanes = None
-
-  # How many decode streams the device runs side by side.  None: the
-  # environment variable T5X_AMD_STREAMS_SIDE_BY_SIDE if set, else measured
-  # once per device and process (streams_side_by_side).  A fixed value makes
-  # the number of batch lanes and of batches in flight, hence what is
-  # captured and held, the same in every run; results never depend on it.
-  side_by_side = None
 
   def __init__(self, config: T5Config, device=None, scan_layers: bool = False):
     """scan_layers: hand out and accept the cache in the layout of a scanned
@@ -357,13 +455,6 @@ class Transformer:
     self._beam_ctx = {}
 
   # -- plumbing ---------------------------------------------------------------
-  def _dev(self):
-    if self.device is None:
-      if not torch.cuda.is_available():
-        raise RuntimeError('t5x_amd needs a GPU (no CPU fallback)')
-      self.device = torch.device('cuda')
-    return self.device
-
   def decoder_weights(self, params) -> DecoderWeights:
     key = id(params)
     if key not in self._weights:
@@ -673,66 +764,6 @@ class Transformer:
                                         enc_tokens, lanes=lanes, slot=slot),
         rebind=lambda ctx: ctx.rebind(loop, encoded, enc_tokens))
 
-  # Decode contexts of one (weights, shapes, options) key that are kept for
-  # re-binding: more than one only when several decodes are in flight at once.
-  MAX_CONTEXTS_PER_KEY = 4
-
-  def _decode_context(self, key, w, owner, make, rebind):
-    """A decode context for `owner` (the loop object that will drive it): a
-    kept one of this key that no live, unfinished loop owns any more, re-bound,
-    or a new one.  Contexts are kept in small pools per key, so that a caller
-    who keeps several decodes in flight (each on its own stream) pays for
-    their allocation and graph capture once.  make(slot) builds a context for
-    pool slot `slot`, whose stream is decode_stream(slot)."""
-    pool = self._beam_ctx.get(key)
-    if pool and pool[0].w is not w:  # an id reused by other weights
-      del self._beam_ctx[key]
-      pool = None
-    if pool is None:
-      if len(self._beam_ctx) >= 2:  # a context holds the caches: keep few
-        self._beam_ctx.pop(next(iter(self._beam_ctx)))
-      pool = self._beam_ctx[key] = []
-    for ctx in pool:
-      if ctx.is_free():
-        rebind(ctx)
-        ctx.claim(owner)
-        return ctx
-    ctx = make(len(pool))
-    ctx.claim(owner)
-    if len(pool) < self.MAX_CONTEXTS_PER_KEY:
-      pool.append(ctx)
-    return ctx
-
-  def streams_side_by_side(self) -> int:
-    """How many decode streams the device runs side by side.  One hardware
-    queue of the process serves the default stream, the others are dealt to
-    the streams in turn, and queues beyond the fourth share command
-    processors (3 decodes in flight pay with the runtime's default of 4
-    queues, 4 with GPU_MAX_HW_QUEUES=8 or more, a fifth never).  Which queue a
-    stream got cannot be asked, so it is measured once per device when the
-    decode streams are made: the first n streams count when n short busy
-    kernels, one per stream, take about as long as one."""
-    import os
-    fixed = self.side_by_side
-    if fixed is None and os.environ.get('T5X_AMD_STREAMS_SIDE_BY_SIDE'):
-      fixed = int(os.environ['T5X_AMD_STREAMS_SIDE_BY_SIDE'])
-    if fixed is not None:
-      return max(1, min(int(fixed), self.MAX_CONTEXTS_PER_KEY))
-    self.decode_stream(0, measure=True)
-    key = self._stream_key()
-    measured = _DECODE_STREAMS_SIDE_BY_SIDE.get(key)
-    if measured is not None:
-      return measured
-    try:
-      queues = int(os.environ.get('GPU_MAX_HW_QUEUES', '4'))
-    except ValueError:
-      queues = 4
-    return 4 if queues >= 8 else 3
-
-  def _stream_key(self):
-    key = torch.device(self._dev()).index
-    return torch.cuda.current_device() if key is None else key
-
   def decode_context_bytes(self, batch_size, num_decodes, enc_len,
                            decode_len) -> int:
     """What one decode in flight keeps on the device besides the shared
@@ -754,31 +785,6 @@ class Transformer:
                                      decode_len)
     free, _ = torch.cuda.mem_get_info(self._dev())
     return max(1, min(n, int(free // 2 // max(1, need))))
-
-  def decode_stream(self, slot, measure=False):
-    """The stream of the decode contexts in pool slot `slot` (with batch
-    lanes: of lane l of the context in slot s, at s * lanes + l).  The device
-    runs streams side by side only when they sit on different hardware
-    queues, of which a process has few (4 by default) and which streams are
-    given in turn as they are first used; so the decode streams of a device
-    are made once per process, together, and each is used once right away:
-    consecutive slots then sit on different queues whatever streams the
-    caller, or another model on the same device, makes later."""
-    dev, key = self._dev(), self._stream_key()
-    streams = _DECODE_STREAMS.get(key)
-    if streams is None:
-      streams = [torch.cuda.Stream(device=dev)
-                 for _ in range(self.MAX_CONTEXTS_PER_KEY)]
-      touch = torch.zeros((16,), dtype=torch.int32, device=dev)
-      torch.cuda.current_stream().synchronize()
-      for stream in streams:
-        with torch.cuda.stream(stream):
-          touch.zero_()
-        stream.synchronize()
-      _DECODE_STREAMS[key] = streams
-    if measure and key not in _DECODE_STREAMS_SIDE_BY_SIDE:
-      _DECODE_STREAMS_SIDE_BY_SIDE[key] = _measure_side_by_side(streams)
-    return streams[slot % len(streams)]
 
   # -- fused sampling: one graph replay per loop iteration --------------------------
   def make_fused_sample_step(self, params, encoded, enc_tokens, owner=None,
@@ -854,31 +860,22 @@ class _OwnedContext:
     return int(self._flag_host[ticket])
 
 
-class FusedSampleStep(_OwnedContext):
+class SampleStepGraph(_OwnedContext):
   """Whole temperature_sample iterations as replays of one captured HIP graph
   (decoder step on the current tokens, token choice, bookkeeping, loop flag).
-  Owns the self-attention caches of its rows as one block
-  [layers, 2, rows, H, 64, L].  The host refills a ring of Gumbel noise for
-  the next `ring` steps, enqueues that many replays, and only then reads the
-  flag back; replays enqueued after the last row ended change nothing."""
+  The host refills a ring of Gumbel noise for the next `ring` steps, enqueues
+  that many replays, and only then reads the flag back; replays enqueued after
+  the last row ended change nothing.  A subclass owns the caches and enqueues an
+  iteration (`_enqueue`)."""
 
-  def __init__(self, module, params, encoded, enc_tokens, *, sequences,
-               cur_index, cur_token, ended, log_prob, max_decode_len,
-               initial_eos_count, temperature, all_ended, eos_id, topk, topp,
-               rescale, noise_source=None, ring=8, slot=0):
-    from t5x_amd import _lib
+  def _init_state(self, module, vocab, slot, *, sequences, cur_index, cur_token,
+                  ended, log_prob, max_decode_len, initial_eos_count,
+                  temperature, all_ended, eos_id, topk, topp, rescale,
+                  noise_source=None, ring=8):
+    from t5x_amd import _lib, ops
     self._lib = _lib
-    cfg, dev = module.config, module._dev()
-    self.module, self.device = module, dev
-    w = module.decoder_weights(params)
-    if isinstance(encoded, BeamShared):
-      beams, enc, enc_tok = encoded.beams, encoded.x, enc_tokens.x
-    else:
-      beams, enc, enc_tok = 1, encoded, enc_tokens
-    enc_tok = torch.as_tensor(np.asarray(enc_tok), device=dev) if not isinstance(
-        enc_tok, torch.Tensor) else enc_tok.to(dev)
-    cross = module._cross_kv(w, enc, enc_tok, beams)
-    self.w, self.cross = w, cross
+    self.module, self.device = module, module._dev()
+    dev = self.device
     # The state the captured graph addresses; a later call is re-bound onto it
     # and reads its results (sequences, log_prob) from here.
     self.sequences, self.cur_index, self.cur_token = (sequences, cur_index,
@@ -888,17 +885,6 @@ class FusedSampleStep(_OwnedContext):
                                                    initial_eos_count)
     self.temperature = temperature
     R, S = sequences.shape
-    act = w.act_dtype
-    # bfloat16: the caches are kept in a layout of the loop's own
-    # (decode_cache_layout); cache_tree() converts back.
-    self.cache_layout, self.L = decode_cache_layout(act, 1, S - 2)
-    L = self.L
-    nl = cfg.num_decoder_layers
-    self.kv = torch.zeros((nl, 2, R, cfg.num_heads, cfg.head_dim,
-                           L + (32 if self.cache_layout == 3 else 0)),
-                          dtype=act, device=dev)
-    self.cache_index = torch.zeros((nl,), dtype=torch.int32, device=dev)
-    self.bufs = _StepBuffers(cfg, R, dev, act)
     self.keep_going = torch.ones((), dtype=torch.int32, device=dev)
     self.step_count = torch.zeros((), dtype=torch.int32, device=dev)
     self.tokens = torch.empty((R,), dtype=torch.int32, device=dev)
@@ -906,18 +892,13 @@ class FusedSampleStep(_OwnedContext):
     self.all_ended = all_ended
     self.noise_source, self.ring = noise_source, int(ring)
     # A row ends at the latest in the iteration that writes its last position,
-    # so no more than max(max_decode_len) iterations ever run (and no noise is
-    # asked for beyond them).
-    self.max_steps = int(max_decode_len.max().item())
+    # so no more than max(max_decode_len - cur_index) iterations ever run (and
+    # no noise is asked for beyond them).
+    self.max_steps = self._longest_row()
     self.noise = None
     if noise_source is not None:
-      self.noise = torch.empty((self.ring, R, cfg.vocab_size),
-                               dtype=torch.float32, device=dev)
-    layer_caches = [(self.kv[i, 0], self.kv[i, 1]) for i in range(nl)]
-    self.model = module._model_step(w, cross, self.bufs, layer_caches,
-                                    self.cache_index, R, beams, L,
-                                    gate=self.keep_going,
-                                    cache_layout=self.cache_layout)
+      self.noise = torch.empty((self.ring, R, vocab), dtype=torch.float32,
+                               device=dev)
     P = _lib.ptr
     st = _lib.SampleStep()
     st.sequences, st.cur_index, st.cur_token = (P(sequences), P(cur_index),
@@ -929,7 +910,6 @@ class FusedSampleStep(_OwnedContext):
     st.noise_ring = self.ring
     st.step_count, st.tokens, st.token_logprobs = (
         P(self.step_count), P(self.tokens), P(self.tok_lp))
-    from t5x_amd import ops
     self.sample_ws = ops.sample_tokens_workspace(R, dev)
     st.workspace = P(self.sample_ws)
     st.all_ended, st.keep_going = P(all_ended), P(self.keep_going)
@@ -941,42 +921,26 @@ class FusedSampleStep(_OwnedContext):
     self.stream = module.decode_stream(slot)
     self.graph = None
     self.step = 0
-    self._capture()
 
   _STATE = ('sequences', 'cur_index', 'cur_token', 'ended', 'log_prob',
             'max_decode_len', 'initial_eos_count', 'temperature')
 
-  def rebind(self, encoded, enc_tokens, *, noise_source=None, **state):
-    """Starts another call of the same shape and options on this context: the
-    new state is copied into the buffers the graph addresses, the new encoder
-    output is projected into the same cross K/V buffers, caches and counters
-    restart."""
-    module, dev = self.module, self.device
-    cur = torch.cuda.current_stream()
-    cur.wait_stream(self.stream)
-    if isinstance(encoded, BeamShared):
-      beams, enc, enc_tok = encoded.beams, encoded.x, enc_tokens.x
-    else:
-      beams, enc, enc_tok = 1, encoded, enc_tokens
-    enc_tok = torch.as_tensor(np.asarray(enc_tok), device=dev) if not isinstance(
-        enc_tok, torch.Tensor) else enc_tok.to(dev)
-    cross = module._cross_kv(self.w, enc, enc_tok, beams, out=self.cross)
-    assert cross is self.cross
+  def _longest_row(self):
+    return max(1, int((self.max_decode_len - self.cur_index).max().item()))
+
+  def _rebind_state(self, noise_source, state):
+    """The new call's state into the buffers the graph addresses."""
     for name in self._STATE:
       getattr(self, name).copy_(state[name])
     self.all_ended.zero_()
     self.keep_going.fill_(1)
     self.step_count.zero_()
-    self.kv.zero_()
-    self.cache_index.zero_()
     self.noise_source = noise_source
-    self.max_steps = int(self.max_decode_len.max().item())
+    self.max_steps = self._longest_row()
     self.step = 0
-    self.stream.wait_stream(cur)
 
   def _enqueue(self):
-    self._lib.call('t5d_temperature_sample_step', self.stream.cuda_stream,
-                   self.model, self.sample)
+    raise NotImplementedError
 
   def _record(self):
     lib = self._lib
@@ -1073,6 +1037,74 @@ class FusedSampleStep(_OwnedContext):
     self.finish()
     return int(self.step_count.item())
 
+  def __del__(self):
+    try:
+      if self.graph is not None:
+        self._lib.call('t5d_graph_destroy', self.graph)
+    except Exception:  # pylint: disable=broad-except
+      pass
+
+
+class FusedSampleStep(SampleStepGraph):
+  """SampleStepGraph of the encoder-decoder: owns the self-attention caches of
+  its rows as one block [layers, 2, rows, H, 64, L]."""
+
+  def __init__(self, module, params, encoded, enc_tokens, *, slot=0, **state):
+    cfg, dev = module.config, module._dev()
+    w = module.decoder_weights(params)
+    if isinstance(encoded, BeamShared):
+      beams, enc, enc_tok = encoded.beams, encoded.x, enc_tokens.x
+    else:
+      beams, enc, enc_tok = 1, encoded, enc_tokens
+    enc_tok = torch.as_tensor(np.asarray(enc_tok), device=dev) if not isinstance(
+        enc_tok, torch.Tensor) else enc_tok.to(dev)
+    cross = module._cross_kv(w, enc, enc_tok, beams)
+    self.w, self.cross = w, cross
+    self._init_state(module, cfg.vocab_size, slot, **state)
+    R, S = self.sequences.shape
+    act = w.act_dtype
+    # bfloat16: the caches are kept in a layout of the loop's own
+    # (decode_cache_layout); cache_tree() converts back.
+    self.cache_layout, self.L = decode_cache_layout(act, 1, S - 2)
+    L = self.L
+    nl = cfg.num_decoder_layers
+    self.kv = torch.zeros((nl, 2, R, cfg.num_heads, cfg.head_dim,
+                           L + (32 if self.cache_layout == 3 else 0)),
+                          dtype=act, device=dev)
+    self.cache_index = torch.zeros((nl,), dtype=torch.int32, device=dev)
+    self.bufs = _StepBuffers(cfg, R, dev, act)
+    layer_caches = [(self.kv[i, 0], self.kv[i, 1]) for i in range(nl)]
+    self.model = module._model_step(w, cross, self.bufs, layer_caches,
+                                    self.cache_index, R, beams, L,
+                                    gate=self.keep_going,
+                                    cache_layout=self.cache_layout)
+    self._capture()
+
+  def rebind(self, encoded, enc_tokens, *, noise_source=None, **state):
+    """Starts another call of the same shape and options on this context: the
+    new state is copied into the buffers the graph addresses, the new encoder
+    output is projected into the same cross K/V buffers, caches and counters
+    restart."""
+    module, dev = self.module, self.device
+    cur = torch.cuda.current_stream()
+    cur.wait_stream(self.stream)
+    if isinstance(encoded, BeamShared):
+      beams, enc, enc_tok = encoded.beams, encoded.x, enc_tokens.x
+    else:
+      beams, enc, enc_tok = 1, encoded, enc_tokens
+    enc_tok = torch.as_tensor(np.asarray(enc_tok), device=dev) if not isinstance(
+        enc_tok, torch.Tensor) else enc_tok.to(dev)
+    cross = module._cross_kv(self.w, enc, enc_tok, beams, out=self.cross)
+    assert cross is self.cross
+    self._rebind_state(noise_source, state)
+    self.kv.zero_()
+    self.cache_index.zero_()
+    self.stream.wait_stream(cur)
+
+  def _enqueue(self):
+    self._lib.call('t5d_temperature_sample_step', self.stream.cuda_stream,
+                   self.model, self.sample)
+
   def cache_tree(self):
     """The caches in the reference's tree layout."""
     self.stream.synchronize()
@@ -1084,13 +1116,6 @@ class FusedSampleStep(_OwnedContext):
     return cache_tree(torch.stack([k for k, _ in plain]),
                       torch.stack([v for _, v in plain]),
                       self.cache_index, self.module.scan_layers)
-
-  def __del__(self):
-    try:
-      if self.graph is not None:
-        self._lib.call('t5d_graph_destroy', self.graph)
-    except Exception:  # pylint: disable=broad-except
-      pass
 
 
 class _BeamLane:
