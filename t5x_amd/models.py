@@ -278,10 +278,9 @@ class EncoderDecoderModel(BatchPredictor):
         decoder_input_tokens.shape[1], in_flight=in_flight)
 
     scanned = hasattr(self.module, 'scan_layers') and self.module.scan_layers
-    return self._begin_decode(decoder_prompt_inputs, cache, tokens_to_logits,
-                              num_decodes, rng, decoder_params,
-                              1 if scanned else 0, return_all_decodes,
-                              initial_index)
+    return self._begin_decode(
+        decoder_prompt_inputs, cache, tokens_ids_to_logits, num_decodes, rng,
+        decoder_params, 1 if scanned else 0, return_all_decodes, initial_index)
 
 
 EncoderDecoderModel.begin_predict_batch_with_aux.stands_for = (
@@ -371,8 +370,9 @@ class DecoderOnlyModel(BatchPredictor):
     inputs = tokens * prompt
     # The last prompt token is the first one the decode loop feeds.
     initial_index = lengths - 1
-    cache = self.module.init_cache(B, L + 2,
-                                   portion=max(1, int(initial_index.max())))
+    # (beam_search counts its steps from there: up to L positions more.)
+    longest = max(1, int(initial_index.max()))
+    cache = self.module.init_cache(B, longest + L + 2, portion=longest)
     self.module.prefill(params, cache, inputs, initial_index)
     return self._begin_decode(
         inputs, cache, PrefilledStepFunction(self.module, params), num_decodes,

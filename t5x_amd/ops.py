@@ -10,13 +10,15 @@ import ctypes
 import torch
 
 from t5x_amd import _lib
-from t5x_amd._lib import BF16, EPI_GEGLU, EPI_NONE, EPI_RESIDUAL, F32, I8
+from t5x_amd._lib import (BF16, EPI_CLAMPED_GLU, EPI_GEGLU, EPI_NONE,
+                          EPI_RESIDUAL, F32, I8)
 
 __all__ = [
     'PackedWeight', 'pack_weight', 'embed', 'rmsnorm', 'gemm',
     'self_attention_step', 'cross_attention_step', 'add_i32',
     'cache_gather_beams', 'gather_beams', 'top_k', 'beam_topk', 'BeamBuffers',
-    'beam_update', 'beam_cond', 'sample_tokens', 'sample_update',
+    'beam_update', 'beam_cond', 'sample_tokens', 'sample_update', 'dense',
+    'embed_sinusoid', 'stream_norm', 'window_attention', 'recurrence',
 ]
 
 
@@ -765,3 +767,101 @@ def sample_update(tokens, token_logprobs, sequences, cur_index, cur_token,
             log_prob.data_ptr(), max_decode_len.data_ptr(),
             initial_eos_count.data_ptr(), all_ended.data_ptr(), R, S,
             int(eos_id))
+
+
+# ------------------------------------------------------------------------------
+# Decoder-only models with a float32 residual stream
+# ------------------------------------------------------------------------------
+
+
+def dense(a, w: PackedWeight, out=None, out_dtype=None, n_store=None,
+          glu=None):
+  """a @ W over any number of rows (t5d_dense).  a [M, >= K] with unit column
+  stride; n_store: only the first columns (float32 output of bfloat16 rows);
+  glu (limit, alpha): W is a gate | up pair and the clamped gated unit is
+  applied."""
+  if not a.is_cuda or a.dim() != 2 or a.stride(1) != 1 or a.shape[1] != w.K:
+    raise ValueError(f'a is {tuple(a.shape)}; kernel K={w.K}')
+  M = a.shape[0]
+  out_dtype = out_dtype or a.dtype
+  if glu is not None:
+    n_store, cols, epi = w.N, w.N // 2, EPI_CLAMPED_GLU
+  else:
+    n_store = cols = n_store or w.N
+    epi = EPI_NONE
+  if out is None:
+    out = torch.empty((M, cols), dtype=out_dtype, device=a.device)
+  _chk(out, 'out', out_dtype, 2)
+  if tuple(out.shape) != (M, cols):
+    raise ValueError(f'out shape {tuple(out.shape)} != {(M, cols)}')
+  limit, alpha = glu or (0.0, 0.0)
+  _lib.call('t5d_dense', _s(), _lib.dtype_code(a.dtype),
+            _lib.dtype_code(out_dtype), a.data_ptr(), a.stride(0),
+            w.data.data_ptr(), out.data_ptr(), cols, n_store, M, w.K, w.N, epi,
+            float(limit), float(alpha))
+  return out
+
+
+def embed_sinusoid(table, ids, positions, width):
+  """float32 [M, ld]: table rows (columns beyond `width` zero) plus the
+  sinusoidal vector of their positions."""
+  _chk(table, 'table', ndim=2)
+  _chk(ids, 'ids', torch.int32, 1)
+  _chk(positions, 'positions', torch.int32, 1)
+  V, ld = table.shape
+  if positions.shape != ids.shape or not 0 < width <= ld:
+    raise ValueError('ids / positions / width mismatch')
+  out = torch.empty((ids.shape[0], ld), dtype=torch.float32,
+                    device=table.device)
+  _lib.call('t5d_embed_sinusoid', _s(), _lib.dtype_code(table.dtype),
+            table.data_ptr(), ids.data_ptr(), positions.data_ptr(),
+            out.data_ptr(), None, ids.shape[0], int(width), ld, V)
+  return out
+
+
+def stream_norm(x, width, dtype, y=None, y_norm=None, add=None, norm=None,
+                x0=None, rows=None, eps=1e-6):
+  """The row kernel between two dense layers of a float32 stream x [M, ld]
+  (t5d_stream_norm): updates x in place and returns the normed rows (with norm)
+  or x | x0 (with x0) as dtype, or None."""
+  _chk(x, 'x', torch.float32, 2)
+  M, ld = x.shape
+  for t, name in ((y_norm, 'y_norm'), (add, 'add'), (norm, 'norm')):
+    if t is not None:
+      _chk(t, name, torch.float32, 1)
+      if t.shape[0] != width:
+        raise ValueError(f'{name} must have {width} entries')
+  if y is not None:
+    _chk(y, 'y', ndim=2)
+    if y.shape != x.shape:
+      raise ValueError('y must have the shape of x')
+  if x0 is not None:
+    _chk(x0, 'x0', torch.float32, 2)
+    if x0.shape != x.shape:
+      raise ValueError('x0 must have the shape of x')
+  out = None
+  n = M
+  if rows is not None:
+    _chk(rows, 'rows', torch.int32, 1)
+    n = rows.shape[0]
+  if norm is not None or x0 is not None:
+    out = torch.empty((n, ld if x0 is None else 2 * ld), dtype=dtype,
+                      device=x.device)
+  P = _lib.ptr
+  _lib.call('t5d_stream_norm', _s(), _lib.dtype_code(dtype),
+            _lib.dtype_code(y.dtype if y is not None else dtype), P(y),
+            P(y_norm), P(add), x.data_ptr(), P(norm), P(x0), P(rows), P(out), n,
+            int(width), ld, float(eps))
+  return out
+
+
+def window_attention(desc, ragged, variant=0):
+  """t5d_window_attention_run over filled-in descriptions (_lib.WindowAttention,
+  _lib.Ragged)."""
+  _lib.call('t5d_window_attention_run', _s(), desc, ragged, int(variant))
+
+
+def recurrence(desc, ragged, variant=0):
+  """t5d_recurrence_run over filled-in descriptions (_lib.Recurrence,
+  _lib.Ragged)."""
+  _lib.call('t5d_recurrence_run', _s(), desc, ragged, int(variant))
