@@ -30,12 +30,12 @@ def softplus(z):
 
 def sinusoid(positions, width):
   """[T, width]: sine in the even entries, cosine in the odd ones."""
-  i = np.arange(width // 2)
+  i = np.arange((width + 1) // 2)
   angle = np.asarray(positions, np.float64)[:, None] * np.power(
       10000.0, -2.0 * i / width)[None, :]
   out = np.zeros((len(positions), width))
-  out[:, 0:2 * len(i):2] = np.sin(angle)
-  out[:, 1:2 * len(i):2] = np.cos(angle)
+  out[:, 0::2] = np.sin(angle)
+  out[:, 1::2] = np.cos(angle)[:, :width // 2]
   return out
 
 

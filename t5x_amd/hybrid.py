@@ -485,6 +485,8 @@ class StepRows:
   def __init__(self, tokens, positions):
     R, dev = tokens.numel(), tokens.device
     self.rows = torch.arange(R + 1, dtype=torch.int32, device=dev)
+    if not (tokens.is_contiguous() and positions.is_contiguous()):
+      raise ValueError('tokens and positions must be contiguous')
     self.tokens, self.positions = tokens, positions
     r = self.ragged = _lib.Ragged()
     r.M = r.S = R
@@ -707,7 +709,7 @@ class HybridDecoder(network.DecodeContexts):
     """One new token per row (device ids [R]), at position cache_index, which
     advances -> logits [R, vocab]."""
     w = self.decoder_weights(params)
-    ids = ids.reshape(-1).to(torch.int32)
+    ids = ids.reshape(-1).to(torch.int32).contiguous()
     R, index = ids.numel(), cache['cache_index']
     if index.numel() != R:  # rows expanded into beams
       index = index.reshape(-1, 1).expand(-1, R // index.numel())
