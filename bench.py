@@ -46,6 +46,10 @@ CONFIGS = {
 }
 DEFAULT_CONFIG = 'base-beam4'
 
+# --stage hybrid: name -> (width, feed-forward); heads of 128
+HYBRID_SIZES = {'base': (768, 2048), 'large': (1024, 2816), 'xl': (2048, 5120)}
+MFMA_F32_PEAK_TFLOPS = 157.3
+
 
 def parse_args():
   ap = argparse.ArgumentParser()
@@ -66,7 +70,7 @@ def parse_args():
   ap.add_argument('--lanes', type=int, default=None,
                   help='batch slices stepped concurrently (default: library)')
   ap.add_argument('--stage', default='decode',
-                  choices=['decode', 'encoder', 'dense', 'memory'],
+                  choices=['decode', 'encoder', 'dense', 'memory', 'hybrid'],
                   help="'encoder': the once-per-batch stage before the decode "
                        'loop (encoder forward + cross K/V projection); a step '
                        "is one batch.  'dense': the decoder's dense layers on "
@@ -77,7 +81,17 @@ def parse_args():
                        'and the next reads (an XCD\'s own L2, the memory-side '
                        'cache, HBM), for plain streaming kernels and for the '
                        'logits between the vocabulary projection and the '
-                       'selection kernel')
+                       "selection kernel.  'hybrid': prefill and decode "
+                       'throughput of a decoder-only hybrid model (--hybrid-'
+                       'size), its mixer kernels on their own, and beside them '
+                       'a T5.1.1 encoder and decoder of the same width and '
+                       'depth')
+  ap.add_argument('--hybrid-size', default='large',
+                  choices=sorted(HYBRID_SIZES),
+                  help='width and feed-forward of --stage hybrid')
+  ap.add_argument('--hybrid-batch', type=int, default=None,
+                  help='prompts prefilled together with --stage hybrid '
+                       '(default 4)')
   ap.add_argument('--in-flight', type=int, default=None,
                   help='also measure this many whole decodes of different '
                        'batches running on the device at once (default for '
@@ -988,6 +1002,237 @@ def main_encoder(args):
   print(json.dumps(out))
 
 
+class HybridStage:
+  """A decoder-only model of 8 layers of a real model's proportions (two thirds
+  recurrent, a quarter windowed attention, a feed-forward everywhere), random
+  weights, and the T5.1.1 encoder / decoder of the same width, feed-forward and
+  depth."""
+
+  LAYERS = 8
+  WINDOW = 1024
+  VOCAB = 32128
+
+  def __init__(self, size, batch, prompt, rows, seed):
+    import torch
+    from t5x_amd import hybrid, network
+    self.torch, self.hybrid, self.network = torch, hybrid, network
+    W, F = HYBRID_SIZES[size]
+    self.W, self.F, self.B, self.T, self.R = W, F, batch, prompt, rows
+    H = W // 128
+    mixers = {
+        'channel_delta': {'heads': H, 'kv_heads': H, 'dim': 128, 'vdim': 128,
+                          'conv': 4},
+        'gla': {'heads': H, 'dim': 128, 'vdim': 128, 'tau': 16.0},
+        'attention': {'heads': H, 'kv_heads': max(1, H // 4), 'dim': 128,
+                      'vdim': 128, 'mask': {'size': self.WINDOW},
+                      'scale': 128 ** -0.5}}
+    order = ['channel_delta', 'gla', 'channel_delta', 'attention']
+    mlp = {'kind': 'dense', 'ff': F, 'limit': 7.0}
+    self.config = {
+        'architecture': 'Mokivik', 'width': W, 'vocab': self.VOCAB,
+        'norm': {'eps': 1e-6},
+        'layers': [{'type': t, 'mixer': mixers[t], 'mlp': mlp}
+                   for t in (order * 2)[:self.LAYERS]]}
+    self.H = H
+    self.cfg = hybrid.HybridConfig.from_dict(self.config, 'bfloat16')
+    self.module = hybrid.HybridDecoder(self.cfg)
+    self.module.max_portion = self.T   # a prompt is one portion
+    self.module.max_tokens = self.B * self.T
+    self.params = hybrid.init_params(self.cfg, seed)
+    self.w = self.module.decoder_weights(self.params)
+    self.rs = np.random.Generator(np.random.PCG64(seed))
+
+  def prompts(self, n, length):
+    return self.rs.integers(1, self.VOCAB, size=(n, length)).astype(np.int32)
+
+  def timed(self, fn, n):
+    torch = self.torch
+    fn()
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    for _ in range(n):
+      fn()
+    torch.cuda.synchronize()
+    return (time.perf_counter() - t0) / n
+
+  def prefill(self, n):
+    """Seconds of one prefill of B prompts of T tokens, one logits row each."""
+    cache = self.module.init_cache(self.B, self.T, portion=self.T)
+    tok = self.prompts(self.B, self.T)
+    portions = [(r, 0, tok[r]) for r in range(self.B)]
+    want = [[self.T - 1]] * self.B
+    return self.timed(lambda: self.module.advance(self.params, cache, portions,
+                                                  want), n)
+
+  def decode(self, n):
+    """Seconds of one replayed decode iteration of R rows at position T."""
+    torch = self.torch
+    R, T = self.R, self.T
+    cache = self.module.init_cache(R, T + n + 40, portion=64)
+    cache['cache_index'].fill_(T)
+    seqs = torch.zeros((R, T + n + 40), dtype=torch.int32, device='cuda')
+    seqs[:, :T + 1] = 5
+    i32 = lambda v: torch.full((R,), v, dtype=torch.int32, device='cuda')
+    ctx = self.hybrid.HybridSampleStep(
+        self.module, self.params, cache, sequences=seqs, cur_index=i32(T),
+        cur_token=i32(5), ended=torch.zeros((R,), dtype=torch.uint8,
+                                            device='cuda'),
+        log_prob=torch.zeros((R,), device='cuda'),
+        max_decode_len=i32(T + n + 38), initial_eos_count=i32(0),
+        temperature=torch.zeros((R,), device='cuda'),
+        all_ended=torch.zeros((), dtype=torch.int32, device='cuda'),
+        eos_id=-1, topk=0, topp=0.0, rescale=True)
+    ctx.launch_graph(ctx.graph, 8)
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    ctx.launch_graph(ctx.graph, n)
+    torch.cuda.synchronize()
+    return (time.perf_counter() - t0) / n
+
+  def t5(self, n_enc, n_dec, enc_len=512):
+    """The same of a T5.1.1 encoder over as many tokens, and of its decoder with
+    as many rows (cross-attention over 512 positions included)."""
+    torch, network = self.torch, self.network
+    cfg = network.T5Config(
+        emb_dim=self.W, num_heads=self.W // 64, num_encoder_layers=self.LAYERS,
+        num_decoder_layers=self.LAYERS, mlp_dim=self.F)
+    params = network.init_params(cfg, 1)
+    module = network.Transformer(cfg)
+    B = self.B * self.T // enc_len
+    tok = torch.as_tensor(self.prompts(B, enc_len), device='cuda')
+    enc = self.timed(lambda: module.apply({'params': params}, tok,
+                                          method=module.encode), n_enc)
+    R, L = self.R, 256
+    tok = torch.as_tensor(self.prompts(R, enc_len), device='cuda')
+    encoded = module.apply({'params': params}, tok, method=module.encode)
+    i32 = lambda v: torch.full((R,), v, dtype=torch.int32, device='cuda')
+    ctx = network.FusedSampleStep(
+        module, params, encoded, tok,
+        sequences=torch.zeros((R, L + 2), dtype=torch.int32, device='cuda'),
+        cur_index=i32(0), cur_token=i32(5),
+        ended=torch.zeros((R,), dtype=torch.uint8, device='cuda'),
+        log_prob=torch.zeros((R,), device='cuda'), max_decode_len=i32(L),
+        initial_eos_count=i32(0),
+        temperature=torch.zeros((R,), device='cuda'),
+        all_ended=torch.zeros((), dtype=torch.int32, device='cuda'),
+        eos_id=-1, topk=0, topp=0.0, rescale=True)
+    launch = lambda k: ctx.launch_graph(ctx.graph, k)
+    first = (L - n_dec) // 2
+    launch(first)
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    launch(n_dec)
+    torch.cuda.synchronize()
+    return enc, (time.perf_counter() - t0) / n_dec
+
+  # -- kernels on their own ----------------------------------------------------
+  def kernels(self):
+    """Each mixer's kernels at the prefill and the decode shape, by HIP events."""
+    from t5x_amd import _lib, ops
+    torch, H, W = self.torch, self.H, self.W
+    G, D = max(1, H // 4), 128
+    out = []
+    for mode in ('prefill', 'decode'):
+      S, n = (self.B, self.T) if mode == 'prefill' else (self.R, 1)
+      start = 0 if mode == 'prefill' else self.T
+      portions = self.hybrid.Portions(
+          [(s, start, np.zeros(n, np.int32)) for s in range(S)], [], 'cuda')
+      bufs = self.hybrid._Buffers(self.w, S * n, S, 'cuda')
+      cache = self.module.init_cache(S, self.T + 64, portion=n)
+      bufs.proj.normal_()
+      M = S * n
+      for i in (3, 0, 1):
+        kind = self.cfg.layers[i].mixer.type
+        layer, leaf = bufs.layers[i], cache['decoder'][f'run_{i}']
+        if kind == 'attention':
+          a = layer.attention
+          a.dtype, a.proj, a.ld_proj = _lib.BF16, bufs.proj.data_ptr(), layer.proj_n
+          a.key_ring, a.value_ring = (leaf[k].data_ptr() for k in
+                                      ('key_ring', 'value_ring'))
+          a.ring = leaf['key_ring'].shape[2]
+          a.q_rows, a.out, a.ld_out = (bufs.q_rows.data_ptr(), layer.mix_rows,
+                                       layer.out_k)
+          a.workspace = bufs.workspace.data_ptr()
+          sec = time_kernel(torch, lambda: ops.window_attention(
+              a, portions.ragged), 10)
+          seen = self.WINDOW
+          if mode == 'prefill':
+            i_ = np.arange(self.T)
+            pairs = float(S * H * np.minimum(i_ + 1, seen).sum())
+            work, unit, peak = 4.0 * D * pairs, 'TFLOP/s', MFMA_BF16_PEAK_TFLOPS
+          else:
+            work, unit, peak = S * G * seen * 2 * D * 2.0, 'GB/s', HBM_PEAK_GBPS
+        else:
+          r = layer.recurrence
+          bufs.low.normal_()
+          r.dtype, r.proj, r.ld_proj = _lib.BF16, bufs.proj.data_ptr(), layer.proj_n
+          r.low, r.ld_low = bufs.low.data_ptr(), layer.low_n
+          r.state = leaf['state'].data_ptr()
+          r.conv_ring = _lib.ptr(leaf.get('conv_ring'))
+          r.out, r.ld_out = layer.mix_rows, layer.out_k
+          r.workspace = bufs.workspace.data_ptr()
+          r.workspace_bytes = bufs.workspace.numel()
+          sec = time_kernel(torch, lambda: ops.recurrence(
+              r, portions.ragged), 10)
+          ops_per = 7.0 if r.delta else 5.0
+          if mode == 'prefill':
+            work, unit, peak = (ops_per * D * D * H * M, 'TFLOP/s',
+                                MFMA_F32_PEAK_TFLOPS)
+          else:
+            work, unit, peak = 2.0 * S * H * D * D * 4, 'GB/s', HBM_PEAK_GBPS
+        rate = work / sec / (1e12 if unit == 'TFLOP/s' else 1e9)
+        out.append({'kernel': f'{kind} ({mode})', 'us': round(sec * 1e6, 2),
+                    'achieved': round(rate, 1), 'peak': peak, 'unit': unit,
+                    'frac': round(rate / peak, 4)})
+    return out
+
+
+def main_hybrid(args):
+  """Prefill and decode of a decoder-only hybrid model beside T5.1.1 of equal
+  width and depth.  A step is one prefill of the batch; `value` is its rate."""
+  size = args.hybrid_size
+  batch = args.hybrid_batch or 4
+  w = HybridStage(size, batch, 4096, 64, args.seed)
+  steps = min(args.steps, 10)
+  kernels = w.kernels()
+  prefill, decode = w.prefill(steps), w.decode(64)
+  t5_enc, t5_dec = w.t5(steps, 64)
+  M = w.B * w.T
+  best = max((k for k in kernels if 'prefill' in k['kernel']),
+             key=lambda k: k['us'])
+  out = {
+      'metric': f'prefilled tokens/sec, hybrid decoder-only model ({size}) on 1 '
+                'GPU',
+      'value': round(M / prefill, 1), 'unit': 'tokens/s', 'n_gpus': 1,
+      'steps': steps, 'warmup': 1, 'ms_per_step': round(prefill * 1e3, 4),
+      'higher_is_better': True, 'scaling': 'weak', 'vs_baseline': None,
+      'dtype': 'bf16', 'data': 'synthetic',
+      'config': {
+          'workload': f'{w.LAYERS} layers of width {w.W}, feed-forward {w.F}: 4 '
+                      'channel-decay delta rule, 2 gated linear attention, 2 '
+                      f'attention over {w.WINDOW} keys, heads of 128; {w.B} '
+                      f'prompts of {w.T} tokens; decode of {w.R} rows at '
+                      f'position {w.T}',
+          'name': size, 'stage': 'hybrid',
+          'decode': {'rows': w.R, 'ms_per_step': round(decode * 1e3, 4),
+                     'tokens_per_s': round(w.R / decode, 1)},
+          't5_same_width': {
+              'what': f'T5.1.1 encoder of {w.LAYERS} layers over {M} tokens (rows '
+                      f'of 512) and decoder of {w.LAYERS} layers with {w.R} '
+                      'rows (positions around 128 of 256, 512 encoder '
+                      'positions)',
+              'encoder_tokens_per_s': round(M / t5_enc, 1),
+              'decode_ms_per_step': round(t5_dec * 1e3, 4),
+              'decode_tokens_per_s': round(w.R / t5_dec, 1)},
+          'kernels': kernels},
+      'roofline': {'kernel': best['kernel'], 'bound': 'mfma',
+                   'achieved': best['achieved'], 'peak': best['peak'],
+                   'unit': best['unit'], 'frac': best['frac'],
+                   'traffic': None, 'avg_launch_us': best['us']},
+  }
+  print(json.dumps(out))
+
+
 def main():
   args = parse_args()
   if args.gpus != 1:
@@ -1006,6 +1251,8 @@ def main():
     return main_encoder(args)
   if args.stage == 'dense':
     return main_dense(args)
+  if args.stage == 'hybrid':
+    return main_hybrid(args)
   if args.stage == 'memory':
     return main_memory(args)
   w = Workload(args.config, args.seed, args.lanes)

@@ -705,12 +705,15 @@ typedef struct {
   float* state;            /* [slots, H, D, Dv] */
   void* out;               /* [M, H * Dv], rows ld_out apart */
   int ld_out;
-  void* workspace;         /* t5d_recurrence_workspace_bytes(M, ...) */
+  void* workspace;         /* t5d_recurrence_workspace_bytes(...), 16-aligned */
+  int64_t workspace_bytes;
 } t5d_recurrence;
 
-int64_t t5d_recurrence_workspace_bytes(int M, int H, int G, int D, int Dv);
+/* Scratch for S portions of M tokens in all.  S 0: without the part for chunks
+ * (portions then run token by token). */
+int64_t t5d_recurrence_workspace_bytes(int M, int S, int H, int G, int D, int Dv);
 /* variant 0: the kernels that suit the call; 1: one token per sequence in one
- * kernel; 2: prepare, scan token by token, finish. */
+ * kernel; 2: portions token by token; 3: portions in chunks of 16 tokens. */
 int t5d_recurrence_run(void* stream, const t5d_recurrence* a, const t5d_ragged* b,
                        int variant);
 

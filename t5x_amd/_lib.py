@@ -106,7 +106,7 @@ class Recurrence(Structure):
                      i2='ld_proj off_q off_k off_v off_beta off_gate', p2='low',
                      i3='ld_low off_z off_low_gate',
                      p3='decay_bias A_log conv norm conv_ring state out',
-                     i4='ld_out', p4='workspace')
+                     i4='ld_out', p4='workspace', l='workspace_bytes')
 
 
 class HybridLayer(Structure):
@@ -149,7 +149,7 @@ _SIGNATURES = {
     't5d_window_workspace_bytes': (c_int64, [c_int] * 4),
     't5d_window_attention_run': (c_int, [_P, POINTER(WindowAttention),
                                          POINTER(Ragged), c_int]),
-    't5d_recurrence_workspace_bytes': (c_int64, [c_int] * 5),
+    't5d_recurrence_workspace_bytes': (c_int64, [c_int] * 6),
     't5d_recurrence_run': (c_int, [_P, POINTER(Recurrence), POINTER(Ragged),
                                    c_int]),
     't5d_hybrid_step': (c_int, [_P, POINTER(HybridModel), POINTER(Ragged), _P,

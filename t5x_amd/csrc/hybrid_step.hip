@@ -66,9 +66,8 @@ int mixer(void* stream, const t5d_hybrid_model* m, const t5d_hybrid_layer& l,
   a.low = m->low; a.ld_low = l.low_n;
   a.state = (float*)run.cache0; a.conv_ring = run.cache1;
   a.out = l.mix_rows; a.ld_out = l.out_k;
-  a.workspace =
-      m->workspace_bytes >= t5d_recurrence_workspace_bytes(b->M, a.H, a.G, a.D, a.Dv)
-          ? m->workspace : nullptr;
+  a.workspace = m->workspace;
+  a.workspace_bytes = m->workspace_bytes;
   return t5d_recurrence_run(stream, &a, b, 0);
 }
 

@@ -10,10 +10,22 @@
 // live in the slot too, a ring by position), optional unit norms of q and k, the
 // decay from a low-rank projection, and the norm and gate of the read-out.
 //
-// A portion runs as prepare (a wavefront per token and head vector), scan and
-// finish; a step of one token per sequence is one kernel per (sequence, head)
+// A portion runs as prepare (a wavefront per token and head vector), the
+// recurrence and finish.  Long portions are cut into chunks of 16 tokens.  With
+// P_t the product of the decays of a chunk up to token t, the state S0 before it
+// and X the solution of (I + diag(beta) A) X = diag(beta) R, A[t][s] = sum_d k_t
+// (P_t / P_s) k_s for s < t, and B the same with q_t for s <= t,
+//   Wk = X(k P), Us = X(v):       u = Us - Wk S0          (no delta rule: u = v)
+//   Qs = q P - B Wk, Os = B Us:   o = Os + Qs S0
+//   S  = diag(P_16) S0 + Kh^T u,  Kh_t = k_t P_16 / P_t
+// Everything but the products with S0 and the state is independent of the other
+// chunks: one kernel forms it for all chunks at once (quotients of decays as
+// running products, which are at most 1), a second walks the chunks with three
+// matrix products each, in float32 on the matrix cores.  Short portions go token
+// by token; a step of one token per sequence is one kernel per (sequence, head)
 // that reads and writes the state once.
 #include "common.h"
+#include "gemm_tiles.h"
 
 namespace t5d {
 
@@ -22,6 +34,8 @@ struct RecArgs {
   t5d_ragged b;
   // float32 scratch of a portion
   float *wq, *wk, *wv, *wbeta, *wo;
+  float* wchunk;  // chunked portions: the chunks' operands (ChunkLayout)
+  int chunks;     // of the longest portion: the chunk kernel's grid
   int C;  // channels of the convolution
   const int32_t* gate;
 };
@@ -223,6 +237,315 @@ recurrence_scan_kernel(RecArgs g, const TQ* q_rows, const TQ* k_rows,
   }
 }
 
+// ---- chunks ---------------------------------------------------------------------------
+constexpr int kChunk = 16;
+
+// A sequence's first chunk in the scratch memory: the sequences before it have
+// at most this many chunks together.
+__host__ __device__ __forceinline__ size_t chunk_base(int64_t first_token, int seq) {
+  return (size_t)(first_token / kChunk + seq);
+}
+
+// What the chunk kernel leaves per (chunk, head), in floats, in the
+// operand order of v_mfma_f32_16x16x4_f32: lane (x, g) of 16 x 4 holds element
+// (row x, k g) of the left operand, (k g, column x) of the right one, and rows
+// 4 g + i of column x of the result.  Step i of a product takes k = 4 g + i from
+// lane (x, g), so that a result tile is the right operand of the next product as
+// it stands; a left operand is then one float4 per lane and tile:
+//   wk, qs [tile of 16 channels][lane]: channels 16 tile + 4 g + i of token x
+//   kh     [tile][lane]: tokens 4 g + i, channel 16 tile + x
+//   us, os [tile of 16 columns][lane]: tokens 4 g + i, column 16 tile + x
+//   pc     [channel]: the chunk's whole decay
+struct ChunkLayout {
+  int dp, vp;
+  __host__ __device__ ChunkLayout(int dp_, int vp_) : dp(dp_), vp(vp_) {}
+  __host__ __device__ size_t wk() const { return 0; }
+  __host__ __device__ size_t qs() const { return (size_t)kChunk * dp; }
+  __host__ __device__ size_t kh() const { return (size_t)2 * kChunk * dp; }
+  __host__ __device__ size_t us() const { return (size_t)3 * kChunk * dp; }
+  __host__ __device__ size_t os() const { return us() + (size_t)kChunk * vp; }
+  __host__ __device__ size_t pc() const { return os() + (size_t)kChunk * vp; }
+  __host__ __device__ size_t size() const { return pc() + dp; }
+};
+
+template <int DP, bool DELTA, typename TQ>
+__global__ void __launch_bounds__(256)
+recurrence_chunk_kernel(RecArgs g, const TQ* q_rows, const TQ* k_rows,
+                        const TQ* v_rows, int ldq, int ldk, int ldv,
+                        float q_scale) {
+  constexpr int LS = DP + 4, C = kChunk;
+  __shared__ __align__(16) float s_k[C * LS];
+  __shared__ __align__(16) float s_q[C * LS];
+  __shared__ __align__(16) float s_g[C * LS];
+  __shared__ __align__(16) float s_a[C][C];
+  __shared__ __align__(16) float s_b[C][C];
+  __shared__ float s_beta[C];
+  T5D_GATED(g.gate);
+  const t5d_recurrence& a = g.a;
+  const int chunk = blockIdx.x, h = blockIdx.y, seq = blockIdx.z;
+  const int hg = h / (a.H / a.G);
+  const int off = g.b.seq_off[seq];
+  const int n = min(C, g.b.seq_off[seq + 1] - off - chunk * C);
+  if (n <= 0) return;
+  const int m0 = off + chunk * C;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const TQ* q = q_rows + (size_t)m0 * ldq + (size_t)hg * a.D;
+  const TQ* k = k_rows + (size_t)m0 * ldk + (size_t)hg * a.D;
+  const TQ* v = v_rows + (size_t)m0 * ldv + (size_t)h * a.Dv;
+  const float* lg = a.low + (size_t)m0 * a.ld_low + a.off_z + (size_t)h * a.D;
+  // tokens past the end: no key, no query, no decay
+#pragma unroll
+  for (int i = 0; i < C * DP / 256; ++i) {
+    const int e = tid + 256 * i, t = e / DP, d = e % DP;
+    const bool ok = t < n && d < a.D;
+    s_k[t * LS + d] = ok ? to_f32<TQ>(k[(size_t)t * ldk + d]) : 0.f;
+    s_q[t * LS + d] = ok ? to_f32<TQ>(q[(size_t)t * ldq + d]) * q_scale : 0.f;
+    s_g[t * LS + d] = ok ? expf(lg[(size_t)t * a.ld_low + d]) : 1.f;
+  }
+  if (tid < C) s_beta[tid] = DELTA && tid < n ? g.wbeta[(size_t)(m0 + tid) * a.H + h] : 0.f;
+  s_a[tid >> 4][tid & 15] = 0.f;
+  s_b[tid >> 4][tid & 15] = 0.f;
+  __syncthreads();
+  {
+    // 32 lanes per source token s, which walk t = s .. 15 with k_s decayed on
+    // the way; source j then source 15 - j, 17 steps for everyone.
+    constexpr int E = (DP + 127) / 128;
+    const int j = tid >> 5, c0 = 4 * (tid & 31);
+#pragma unroll
+    for (int pass = 0; pass < 2; ++pass) {
+      const int s = pass == 0 ? j : C - 1 - j;
+      float4 x[E];
+#pragma unroll
+      for (int e = 0; e < E; ++e)
+        x[e] = c0 + 128 * e < DP
+                   ? *reinterpret_cast<const float4*>(s_k + s * LS + c0 + 128 * e)
+                   : make_float4(0.f, 0.f, 0.f, 0.f);
+      for (int t = s; t < C; ++t) {
+        float ka = 0.f, qa = 0.f;
+#pragma unroll
+        for (int e = 0; e < E; ++e) {
+          if (c0 + 128 * e >= DP) continue;
+          const int o = t * LS + c0 + 128 * e;
+          if (t > s) {
+            const float4 w = *reinterpret_cast<const float4*>(s_g + o);
+            x[e].x *= w.x; x[e].y *= w.y; x[e].z *= w.z; x[e].w *= w.w;
+          }
+          const float4 y = *reinterpret_cast<const float4*>(s_q + o);
+          qa = fmaf(x[e].x, y.x, qa); qa = fmaf(x[e].y, y.y, qa);
+          qa = fmaf(x[e].z, y.z, qa); qa = fmaf(x[e].w, y.w, qa);
+          if (DELTA) {
+            const float4 z = *reinterpret_cast<const float4*>(s_k + o);
+            ka = fmaf(x[e].x, z.x, ka); ka = fmaf(x[e].y, z.y, ka);
+            ka = fmaf(x[e].z, z.z, ka); ka = fmaf(x[e].w, z.w, ka);
+          }
+        }
+        auto over32 = [](float f) {
+          f = lanes16_sum(f);
+          const auto w = __builtin_amdgcn_permlane16_swap(
+              __float_as_uint(f), __float_as_uint(f), false, false);
+          return __uint_as_float(w[0]) + __uint_as_float(w[1]);
+        };
+        qa = over32(qa);
+        if (DELTA) ka = over32(ka);
+        if ((tid & 31) == 0) {
+          s_b[t][s] = qa;
+          if (DELTA && t > s) s_a[t][s] = ka;
+        }
+      }
+    }
+  }
+  __syncthreads();
+
+  const int vp = (a.Dv + 15) / 16 * 16;
+  const ChunkLayout lay(DP, vp);
+  float* w = g.wchunk + ((chunk_base(off, seq) + chunk) * a.H + h) * lay.size();
+  // A thread per channel, then per value column: the triangular solve and the
+  // products with B down the column.
+  for (int c = tid; c < DP + vp; c += 256) {
+    const bool channel = c < DP;
+    const int vc = c - DP;
+    float x[C], upto[C];  // solution; decay up to and with token t
+    float run = 1.f;
+#pragma unroll
+    for (int t = 0; t < C; ++t) {
+      float rhs;
+      if (channel) {
+        run *= s_g[t * LS + c];
+        upto[t] = run;
+        rhs = s_k[t * LS + c] * run;
+      } else {
+        rhs = t < n && vc < a.Dv ? to_f32<TQ>(v[(size_t)t * ldv + vc]) : 0.f;
+      }
+      if (DELTA) {
+#pragma unroll
+        for (int s = 0; s < t; ++s) rhs = fmaf(-s_a[t][s], x[s], rhs);
+        rhs *= s_beta[t];
+      }
+      x[t] = rhs;
+    }
+    if (channel) {
+      // this thread's column of the three arrays is read by no other thread
+      float back = 1.f;
+      w[lay.pc() + c] = run;
+#pragma unroll
+      for (int t = C - 1; t >= 0; --t) {
+        float y = s_q[t * LS + c] * upto[t];
+        if (DELTA) {
+#pragma unroll
+          for (int s = 0; s <= t; ++s) y = fmaf(-s_b[t][s], x[s], y);
+        }
+        const float gt = s_g[t * LS + c];
+        s_g[t * LS + c] = s_k[t * LS + c] * back;
+        back *= gt;
+        s_q[t * LS + c] = y;
+        if (DELTA) s_k[t * LS + c] = x[t];
+      }
+    } else {
+      float4* us = reinterpret_cast<float4*>(w + lay.us()) + (vc >> 4) * 64 + (vc & 15);
+      float4* os = reinterpret_cast<float4*>(w + lay.os()) + (vc >> 4) * 64 + (vc & 15);
+      float y[C];
+#pragma unroll
+      for (int t = 0; t < C; ++t) {
+        y[t] = 0.f;
+#pragma unroll
+        for (int s = 0; s <= t; ++s) y[t] = fmaf(s_b[t][s], x[s], y[t]);
+      }
+#pragma unroll
+      for (int q4 = 0; q4 < 4; ++q4) {
+        us[16 * q4] = make_float4(x[4 * q4], x[4 * q4 + 1], x[4 * q4 + 2], x[4 * q4 + 3]);
+        os[16 * q4] = make_float4(y[4 * q4], y[4 * q4 + 1], y[4 * q4 + 2], y[4 * q4 + 3]);
+      }
+    }
+  }
+  __syncthreads();
+  for (int f = tid; f < DP * 4; f += 256) {
+    const int tile = f >> 6, l = f & 63, x = l & 15, g4 = l >> 4;
+    const int o = x * LS + 16 * tile + 4 * g4;
+    if (DELTA)
+      reinterpret_cast<float4*>(w + lay.wk())[f] =
+          *reinterpret_cast<const float4*>(s_k + o);
+    reinterpret_cast<float4*>(w + lay.qs())[f] =
+        *reinterpret_cast<const float4*>(s_q + o);
+    const float* kh = s_g + 4 * g4 * LS + 16 * tile + x;
+    reinterpret_cast<float4*>(w + lay.kh())[f] =
+        make_float4(kh[0], kh[LS], kh[2 * LS], kh[3 * LS]);
+  }
+  (void)lane;
+}
+
+// Walks the chunks of one (sequence, head) for 16 value columns.  Each of 4
+// wavefronts holds NTW tiles of 16 channels x 16 columns of the state.
+template <int NTW, bool DELTA>
+__global__ void __launch_bounds__(256)
+recurrence_chain_kernel(RecArgs g) {
+  constexpr int DP = 64 * NTW;
+  __shared__ float4 s_u[2][4][64];
+  __shared__ float4 s_o[2][4][64];
+  T5D_GATED(g.gate);
+  const t5d_recurrence& a = g.a;
+  const int vt = blockIdx.x, h = blockIdx.y, seq = blockIdx.z;
+  const int off = g.b.seq_off[seq], len = g.b.seq_off[seq + 1] - off;
+  if (len <= 0) return;
+  const int start = g.b.seq_start[seq], slot = g.b.seq_slot[seq];
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int x = lane & 15, g4 = lane >> 4;
+  const int vp = (int)gridDim.x * 16, col = 16 * vt + x;
+  const bool col_ok = col < a.Dv;
+  const ChunkLayout lay(DP, vp);
+  const int nc = (len + kChunk - 1) / kChunk;
+  const size_t stride = (size_t)a.H * lay.size();
+  const float* base = g.wchunk + (chunk_base(off, seq) * a.H + h) * lay.size();
+
+  float* state = a.state + ((size_t)slot * a.H + h) * a.D * a.Dv + col;
+  f32x4_v st[NTW];
+#pragma unroll
+  for (int t = 0; t < NTW; ++t)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = 16 * (wave * NTW + t) + 4 * g4 + i;
+      st[t][i] = start > 0 && col_ok && d < a.D ? state[(size_t)d * a.Dv] : 0.f;
+    }
+  float* out = g.wo + ((size_t)off * a.H + h) * a.Dv + col;
+
+  struct Operands {
+    float4 wk[NTW], qs[NTW], kh[NTW], pc[NTW], us, os;
+  };
+  auto load = [&](Operands& o, int c) {
+    const float* w = base + (size_t)c * stride;
+#pragma unroll
+    for (int t = 0; t < NTW; ++t) {
+      const int tile = wave * NTW + t;
+      if (DELTA)
+        o.wk[t] = reinterpret_cast<const float4*>(w + lay.wk())[tile * 64 + lane];
+      o.qs[t] = reinterpret_cast<const float4*>(w + lay.qs())[tile * 64 + lane];
+      o.kh[t] = reinterpret_cast<const float4*>(w + lay.kh())[tile * 64 + lane];
+      o.pc[t] = reinterpret_cast<const float4*>(w + lay.pc())[tile * 4 + g4];
+    }
+    o.us = reinterpret_cast<const float4*>(w + lay.us())[vt * 64 + lane];
+    // (only the row this wavefront stores is used)
+    o.os.x = (w + lay.os())[(vt * 64 + lane) * 4 + wave];
+  };
+  auto step = [&](const Operands& o, int c) {
+    const int buf = c & 1;
+    f32x4_v u = (f32x4_v){0.f, 0.f, 0.f, 0.f}, r = u;
+#pragma unroll
+    for (int t = 0; t < NTW; ++t) {
+      const float qs[4] = {o.qs[t].x, o.qs[t].y, o.qs[t].z, o.qs[t].w};
+      const float wk[4] = {o.wk[t].x, o.wk[t].y, o.wk[t].z, o.wk[t].w};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        if (DELTA)
+          u = __builtin_amdgcn_mfma_f32_16x16x4f32(wk[i], st[t][i], u, 0, 0, 0);
+        r = __builtin_amdgcn_mfma_f32_16x16x4f32(qs[i], st[t][i], r, 0, 0, 0);
+      }
+    }
+    if (DELTA) s_u[buf][wave][lane] = make_float4(u[0], u[1], u[2], u[3]);
+    s_o[buf][wave][lane] = make_float4(r[0], r[1], r[2], r[3]);
+    __syncthreads();
+    float uu[4] = {o.us.x, o.us.y, o.us.z, o.us.w};
+    if (DELTA) {
+#pragma unroll
+      for (int p = 0; p < 4; ++p) {
+        const float4 q = s_u[buf][p][lane];
+        uu[0] -= q.x; uu[1] -= q.y; uu[2] -= q.z; uu[3] -= q.w;
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < NTW; ++t) {
+      const float kh[4] = {o.kh[t].x, o.kh[t].y, o.kh[t].z, o.kh[t].w};
+      st[t][0] *= o.pc[t].x; st[t][1] *= o.pc[t].y;
+      st[t][2] *= o.pc[t].z; st[t][3] *= o.pc[t].w;
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        st[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(kh[i], uu[i], st[t], 0, 0, 0);
+    }
+    // the read-out of tokens 4 g + wave
+    float y = o.os.x;
+#pragma unroll
+    for (int p = 0; p < 4; ++p)
+      y += reinterpret_cast<const float*>(&s_o[buf][p][lane])[wave];
+    const int tok = kChunk * c + 4 * g4 + wave;
+    if (tok < len && col_ok) out[(size_t)tok * a.H * a.Dv] = y;
+  };
+  Operands o0, o1;
+  load(o0, 0);
+  for (int c = 0; c < nc; c += 2) {
+    load(o1, min(c + 1, nc - 1));
+    step(o0, c);
+    if (c + 1 >= nc) break;
+    load(o0, min(c + 2, nc - 1));
+    step(o1, c + 1);
+  }
+#pragma unroll
+  for (int t = 0; t < NTW; ++t)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = 16 * (wave * NTW + t) + 4 * g4 + i;
+      if (col_ok && d < a.D) state[(size_t)d * a.Dv] = st[t][i];
+    }
+}
+
 // The convolution's last inputs of a portion, written once nothing of the portion
 // reads the ring any more.
 template <typename T>
@@ -418,6 +741,37 @@ static void launch_scan(hipStream_t s, const RecArgs& g, const TQ* q, const TQ* 
 #undef T5D_SC
 }
 
+template <bool DELTA, typename TQ>
+static void launch_chunks(hipStream_t s, const RecArgs& g, const TQ* q,
+                          const TQ* k, const TQ* v, int ldq, int ldk, int ldv,
+                          float q_scale) {
+  const dim3 grid(g.chunks, g.a.H, g.b.S), block(256);
+  const dim3 cgrid((g.a.Dv + 15) / 16, g.a.H, g.b.S);
+#define T5D_CH(E_)                                                              \
+  do {                                                                          \
+    hipLaunchKernelGGL((recurrence_chunk_kernel<64 * E_, DELTA, TQ>), grid,     \
+                       block, 0, s, g, q, k, v, ldq, ldk, ldv, q_scale);        \
+    hipLaunchKernelGGL((recurrence_chain_kernel<E_, DELTA>), cgrid, block, 0, s, \
+                       g);                                                      \
+  } while (0)
+  if (g.a.D <= 64) T5D_CH(1);
+  else if (g.a.D <= 128) T5D_CH(2);
+  else if (g.a.D <= 256) T5D_CH(4);
+  else T5D_CH(8);
+#undef T5D_CH
+}
+
+// The recurrence of a portion: chunks, or token by token (g.wchunk null).
+template <bool DELTA, typename TQ>
+static void launch_recurrence(hipStream_t s, const RecArgs& g, const TQ* q,
+                              const TQ* k, const TQ* v, int ldq, int ldk, int ldv,
+                              float q_scale) {
+  if (g.wchunk != nullptr)
+    launch_chunks<DELTA, TQ>(s, g, q, k, v, ldq, ldk, ldv, q_scale);
+  else
+    launch_scan<DELTA, TQ>(s, g, q, k, v, ldq, ldk, ldv, q_scale);
+}
+
 template <typename T>
 static int run_portions(hipStream_t s, const RecArgs& g) {
   const t5d_recurrence& a = g.a;
@@ -429,16 +783,16 @@ static int run_portions(hipStream_t s, const RecArgs& g) {
   if (qkv) {
     const int gd = a.G * a.D, hv = a.H * a.Dv;
     if (a.delta)
-      launch_scan<true, float>(s, g, g.wq, g.wk, g.wv, gd, gd, hv, 1.f);
+      launch_recurrence<true, float>(s, g, g.wq, g.wk, g.wv, gd, gd, hv, 1.f);
     else
-      launch_scan<false, float>(s, g, g.wq, g.wk, g.wv, gd, gd, hv, 1.f);
+      launch_recurrence<false, float>(s, g, g.wq, g.wk, g.wv, gd, gd, hv, 1.f);
   } else {
     const T* p = reinterpret_cast<const T*>(a.proj);
     if (a.delta)
-      launch_scan<true, T>(s, g, p + a.off_q, p + a.off_k, p + a.off_v, a.ld_proj,
+      launch_recurrence<true, T>(s, g, p + a.off_q, p + a.off_k, p + a.off_v, a.ld_proj,
                            a.ld_proj, a.ld_proj, a.q_scale);
     else
-      launch_scan<false, T>(s, g, p + a.off_q, p + a.off_k, p + a.off_v, a.ld_proj,
+      launch_recurrence<false, T>(s, g, p + a.off_q, p + a.off_k, p + a.off_v, a.ld_proj,
                             a.ld_proj, a.ld_proj, a.q_scale);
   }
   T5D_CHECK_LAUNCH("recurrence (scan)");
@@ -456,15 +810,31 @@ static int run_portions(hipStream_t s, const RecArgs& g) {
 
 static int64_t round4(int64_t n) { return (n + 3) / 4 * 4; }
 
+// Floats of scratch of the un-chunked kernels.
+static int64_t portion_floats(int64_t M, int H, int G, int D, int Dv) {
+  return 2 * round4(M * G * D) + 2 * round4(M * H * Dv) + round4(M * H);
+}
+
+static int channel_pad(int D) {
+  return D <= 64 ? 64 : D <= 128 ? 128 : D <= 256 ? 256 : 512;
+}
+static int64_t chunk_floats(int64_t M, int S, int H, int D, int Dv) {
+  const ChunkLayout lay(channel_pad(D), (Dv + 15) / 16 * 16);
+  return (int64_t)chunk_base(M, S) * H * (int64_t)lay.size();
+}
+
+// Portions from here on run in chunks.
+constexpr int kChunkFrom = 24;
+
 }  // namespace t5d
 
 using namespace t5d;
 
-extern "C" int64_t t5d_recurrence_workspace_bytes(int M, int H, int G, int D,
+extern "C" int64_t t5d_recurrence_workspace_bytes(int M, int S, int H, int G, int D,
                                                   int Dv) {
-  if (M <= 0 || H <= 0 || G <= 0 || D <= 0 || Dv <= 0) return -1;
-  return 4 * (2 * round4((int64_t)M * G * D) + 2 * round4((int64_t)M * H * Dv) +
-              round4((int64_t)M * H));
+  if (M <= 0 || S < 0 || H <= 0 || G <= 0 || D <= 0 || Dv <= 0) return -1;
+  return 4 * (portion_floats(M, H, G, D, Dv) +
+              (S > 0 ? chunk_floats(M, S, H, D, Dv) : 0));
 }
 
 extern "C" int t5d_recurrence_run(void* stream, const t5d_recurrence* a,
@@ -487,7 +857,7 @@ extern "C" int t5d_recurrence_run(void* stream, const t5d_recurrence* a,
                   b->max_len <= b->M,
               T5D_EINVAL, "t5d_recurrence_run: M=%d S=%d max_len=%d", b->M, b->S,
               b->max_len);
-  T5D_REQUIRE(variant >= 0 && variant <= 2, T5D_EINVAL,
+  T5D_REQUIRE(variant >= 0 && variant <= 3, T5D_EINVAL,
               "t5d_recurrence_run: variant %d", variant);
   RecArgs g;
   g.a = *a; g.b = *b; g.gate = tls_gate;
@@ -499,7 +869,8 @@ extern "C" int t5d_recurrence_run(void* stream, const t5d_recurrence* a,
               "t5d_recurrence_run: variant 1 does not cover this call");
   hipStream_t s = as_stream(stream);
   if (variant == 1 || (variant == 0 && can_step)) {
-    g.wq = g.wk = g.wv = g.wbeta = g.wo = nullptr;
+    g.wq = g.wk = g.wv = g.wbeta = g.wo = g.wchunk = nullptr;
+    g.chunks = 0;
     const bool bf16 = a->dtype == T5D_BF16;
     if (a->delta) {
       if (bf16) launch_step<true, bf16_t>(s, g);
@@ -518,5 +889,15 @@ extern "C" int t5d_recurrence_run(void* stream, const t5d_recurrence* a,
                 hv = round4((int64_t)b->M * a->H * a->Dv);
   g.wq = w; g.wk = w + qk; g.wv = w + 2 * qk; g.wo = w + 2 * qk + hv;
   g.wbeta = w + 2 * qk + 2 * hv;
+  const int64_t plain = portion_floats(b->M, a->H, a->G, a->D, a->Dv);
+  g.chunks = (b->max_len + kChunk - 1) / kChunk;
+  const bool fits =
+      a->workspace_bytes >=
+      4 * (plain + chunk_floats(b->M, b->S, a->H, a->D, a->Dv));
+  T5D_REQUIRE(a->workspace_bytes >= 4 * plain && (variant != 3 || fits), T5D_EINVAL,
+              "t5d_recurrence_run: a workspace of %lld bytes",
+              (long long)a->workspace_bytes);
+  g.wchunk = variant == 3 || (variant == 0 && fits && b->max_len >= kChunkFrom)
+                 ? w + plain : nullptr;
   return a->dtype == T5D_BF16 ? run_portions<bf16_t>(s, g) : run_portions<float>(s, g);
 }

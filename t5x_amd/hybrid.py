@@ -443,8 +443,10 @@ class _Buffers:
         ws = max(ws, lib.t5d_window_workspace_bytes(seqs, m.heads, m.dim,
                                                     m.vdim))
       else:
+        # (one token per sequence: no scratch for chunks)
         ws = max(ws, lib.t5d_recurrence_workspace_bytes(
-            tokens, m.heads, m.kv_heads, m.dim, m.vdim))
+            tokens, seqs if tokens > seqs else 0, m.heads, m.kv_heads, m.dim,
+            m.vdim))
     self.q_rows = rows(q_cols) if q_cols else None
     self.workspace = torch.empty((ws,), dtype=torch.uint8, device=device)
 
@@ -560,16 +562,13 @@ class HybridDecoder(network.DecodeContexts):
   def _buffers(self, w, tokens, seqs):
     """Shared activation buffers of at least this size (calls on one stream)."""
     b = self._bufs
-    if b is None or b[0] is not w or b[1].tokens < tokens or b[1].seqs < seqs:
-      grow = lambda n: 1 << (n - 1).bit_length()
-      old = b[1] if b is not None and b[0] is w else None
-      self._bufs = None
-      tokens, seqs = grow(tokens), grow(seqs)
-      if old is not None:
-        tokens, seqs = max(tokens, old.tokens), max(seqs, old.seqs)
-      del old, b
+    have = (b[1].tokens, b[1].seqs) if b is not None and b[0] is w else (0, 0)
+    if tokens > have[0] or seqs > have[1]:
+      grow = lambda n, h: max(1 << (n - 1).bit_length(), h)
+      self._bufs = self._step = b = None
+      seqs = grow(seqs, have[1])
+      tokens = max(grow(tokens, have[0]), 2 * seqs)
       b = self._bufs = (w, _Buffers(w, tokens, seqs, self._dev()))
-      self._step = None
     return b[1]
 
   def _model(self, w: HybridWeights, bufs: _Buffers, cache, gate=None):

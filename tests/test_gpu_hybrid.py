@@ -408,12 +408,12 @@ class Recurrence:
     M = len(proj)
     out = torch.full((M, H * Dv + 6), 3.0, dtype=self.dt, device='cuda')
     ws = torch.empty(
-        (_lib.load().t5d_recurrence_workspace_bytes(M, H, G, D, Dv),),
-        dtype=torch.uint8, device='cuda')
+        (_lib.load().t5d_recurrence_workspace_bytes(
+            M, len(portions), H, G, D, Dv),), dtype=torch.uint8, device='cuda')
     r = self.r
     r.proj, r.low, r.out, r.ld_out = (proj.data_ptr(), low.data_ptr(),
                                       out.data_ptr(), H * Dv + 6)
-    r.workspace = ws.data_ptr()
+    r.workspace, r.workspace_bytes = ws.data_ptr(), ws.numel()
     ops.recurrence(r, x.ragged, variant)
     got = host(out)
     assert (got[:, H * Dv:] == 3.0).all()
@@ -472,12 +472,14 @@ def test_recurrence_portions_and_steps(dt, strong, delta, H, G, D, Dv, taps):
   seq = r.sequence(T)
   want = r.oracle(seq)
   assert rel(r.run([(1, 0, T)], [seq]), want) < r.tol
-  for cuts in ([1, 2, 3, 5, 8, 24, 25, 41, 57], [16, 32, 64], [2, 4, 6, 70]):
-    got, at = [], 0
-    for end in cuts + [T]:
-      got.append(r.run([(0, at, end)], [seq], variant=2))
-      at = end
-    assert rel(np.concatenate(got), want) < r.tol, cuts
+  for variant in (2, 3):  # token by token, in chunks
+    assert rel(r.run([(1, 0, T)], [seq], variant), want) < r.tol, variant
+    for cuts in ([1, 2, 3, 5, 8, 24, 25, 41, 57], [16, 32, 64], [2, 4, 6, 70]):
+      got, at = [], 0
+      for end in cuts + [T]:
+        got.append(r.run([(0, at, end)], [seq], variant))
+        at = end
+      assert rel(np.concatenate(got), want) < r.tol, (variant, cuts)
   got = [r.run([(1, 0, 40)], [seq])]
   got += [r.run([(1, t, t + 1)], [seq]) for t in range(40, T)]
   assert rel(np.concatenate(got), want) < r.tol
