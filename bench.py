@@ -1022,7 +1022,7 @@ class HybridStage:
     mixers = {
         'channel_delta': {'heads': H, 'kv_heads': H, 'dim': 128, 'vdim': 128,
                           'conv': 4},
-        'gla': {'heads': H, 'dim': 128, 'vdim': 128, 'tau': 16.0},
+        'gla': {'heads': H, 'dim': 128, 'vdim': 128, 'tau': 12.0},
         'attention': {'heads': H, 'kv_heads': max(1, H // 4), 'dim': 128,
                       'vdim': 128, 'mask': {'size': self.WINDOW},
                       'scale': 128 ** -0.5}}

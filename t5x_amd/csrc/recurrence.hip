@@ -10,8 +10,8 @@
 // live in the slot too, a ring by position), optional unit norms of q and k, the
 // decay from a low-rank projection, and the norm and gate of the read-out.
 //
-// A portion runs as prepare (a wavefront per token and head vector), the
-// recurrence and finish.  Long portions are cut into chunks of 16 tokens.  With
+// Short portions run as prepare (a wavefront per token and head vector), a scan
+// token by token, and finish.  Long ones are cut into chunks of 16 tokens.  With
 // P_t the product of the decays of a chunk up to token t, the state S0 before it
 // and X the solution of (I + diag(beta) A) X = diag(beta) R, A[t][s] = sum_d k_t
 // (P_t / P_s) k_s for s < t, and B the same with q_t for s <= t,
@@ -19,11 +19,11 @@
 //   Qs = q P - B Wk, Os = B Us:   o = Os + Qs S0
 //   S  = diag(P_16) S0 + Kh^T u,  Kh_t = k_t P_16 / P_t
 // Everything but the products with S0 and the state is independent of the other
-// chunks: one kernel forms it for all chunks at once (quotients of decays as
-// running products, which are at most 1), a second walks the chunks with three
-// matrix products each, in float32 on the matrix cores.  Short portions go token
-// by token; a step of one token per sequence is one kernel per (sequence, head)
-// that reads and writes the state once.
+// chunks: one kernel forms it for all chunks at once, from the projections on
+// (quotients of decays as running products, which are at most 1), a second walks
+// the chunks with three matrix products each, in float32 on the matrix cores.
+// A step of one token per sequence is one kernel per (sequence, head) that reads
+// and writes the state once.
 #include "common.h"
 #include "gemm_tiles.h"
 
@@ -40,7 +40,12 @@ struct RecArgs {
   const int32_t* gate;
 };
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float exp_f(float z) {
+  return __builtin_amdgcn_exp2f(z * 1.4426950408889634f);
+}
+__device__ __forceinline__ float sigmoid_f(float z) {
+  return 1.0f / (1.0f + exp_f(-z));
+}
 __device__ __forceinline__ float softplus_f(float z) {
   return z > 20.f ? z : log1pf(expf(z));
 }
@@ -73,7 +78,7 @@ __device__ __forceinline__ float conv_channel(const RecArgs& g, int m, int first
                         : to_f32<T>(ring[(size_t)((pos - j) % a.taps) * g.C]);
     s = fmaf(v, w[a.taps - 1 - j], s);
   }
-  return s / (1.0f + expf(-s));
+  return s * sigmoid_f(s);
 }
 
 // ---- prepare ----------------------------------------------------------------------
@@ -268,11 +273,53 @@ struct ChunkLayout {
   __host__ __device__ size_t size() const { return pc() + dp; }
 };
 
-template <int DP, bool DELTA, typename TQ>
-__global__ void __launch_bounds__(256)
-recurrence_chunk_kernel(RecArgs g, const TQ* q_rows, const TQ* k_rows,
-                        const TQ* v_rows, int ldq, int ldk, int ldv,
-                        float q_scale) {
+// 16 tokens of one projection column, through the convolution and silu if there
+// is one (TM: at least its taps).  i0: the chunk's first token within the portion.
+template <int TM, typename T>
+__device__ __forceinline__ void chunk_column(const RecArgs& g, int m0, int n, int i0,
+                                             int pos0, int slot, int col, int cc,
+                                             float (&y)[kChunk]) {
+  const t5d_recurrence& a = g.a;
+  const T* p = reinterpret_cast<const T*>(a.proj) + (size_t)m0 * a.ld_proj + col;
+  float x[kChunk];
+#pragma unroll
+  for (int t = 0; t < kChunk; ++t)
+    x[t] = t < n ? to_f32<T>(p[(size_t)t * a.ld_proj]) : 0.f;
+  if constexpr (TM == 0) {
+#pragma unroll
+    for (int t = 0; t < kChunk; ++t) y[t] = x[t];
+    return;
+  }
+  constexpr int N = TM > 0 ? TM : 1;
+  float w[N], before[N];  // before[j]: the value j tokens before the chunk
+  const T* ring = reinterpret_cast<const T*>(a.conv_ring) +
+                  (size_t)slot * a.taps * g.C + cc;
+#pragma unroll
+  for (int j = 0; j < N; ++j) {
+    w[j] = j < a.taps ? a.conv[(size_t)cc * a.taps + a.taps - 1 - j] : 0.f;
+    before[j] = 0.f;
+    if (j > 0 && j < a.taps) {
+      if (i0 >= j)
+        before[j] = to_f32<T>(p[-(ptrdiff_t)j * a.ld_proj]);
+      else if (pos0 >= j)
+        before[j] = to_f32<T>(ring[(size_t)((pos0 - j) % a.taps) * g.C]);
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < kChunk; ++t) {
+    float s = 0.f;
+#pragma unroll
+    for (int j = 0; j < N; ++j)
+      s = fmaf(w[j], t >= j ? x[t >= j ? t - j : 0] : before[t >= j ? 0 : j - t], s);
+    y[t] = s * sigmoid_f(s);
+  }
+}
+
+constexpr int kChunkTaps = 8;  // longest convolution of the chunk kernel
+
+template <int DP, bool DELTA, typename T>
+__global__ void __launch_bounds__(256, DP <= 128 ? 4 : DP <= 256 ? 2 : 1)
+recurrence_chunk_kernel(RecArgs g) {
   constexpr int LS = DP + 4, C = kChunk;
   __shared__ __align__(16) float s_k[C * LS];
   __shared__ __align__(16) float s_q[C * LS];
@@ -280,6 +327,7 @@ recurrence_chunk_kernel(RecArgs g, const TQ* q_rows, const TQ* k_rows,
   __shared__ __align__(16) float s_a[C][C];
   __shared__ __align__(16) float s_b[C][C];
   __shared__ float s_beta[C];
+  extern __shared__ float s_v[];  // [C][vp]
   T5D_GATED(g.gate);
   const t5d_recurrence& a = g.a;
   const int chunk = blockIdx.x, h = blockIdx.y, seq = blockIdx.z;
@@ -288,23 +336,82 @@ recurrence_chunk_kernel(RecArgs g, const TQ* q_rows, const TQ* k_rows,
   const int n = min(C, g.b.seq_off[seq + 1] - off - chunk * C);
   if (n <= 0) return;
   const int m0 = off + chunk * C;
-  const int tid = threadIdx.x, lane = tid & 63;
-  const TQ* q = q_rows + (size_t)m0 * ldq + (size_t)hg * a.D;
-  const TQ* k = k_rows + (size_t)m0 * ldk + (size_t)hg * a.D;
-  const TQ* v = v_rows + (size_t)m0 * ldv + (size_t)h * a.Dv;
-  const float* lg = a.low + (size_t)m0 * a.ld_low + a.off_z + (size_t)h * a.D;
-  // tokens past the end: no key, no query, no decay
+  const int tid = threadIdx.x;
+  const int vp = (a.Dv + 15) / 16 * 16;
+  const int slot = g.b.seq_slot[seq], pos0 = g.b.seq_start[seq] + chunk * C;
+  // Columns of q, k, v and the decay; tokens past the end have no key, no query,
+  // no value and no decay.
+  for (int u = tid; u < 3 * DP + vp; u += 256) {
+    const int kind = u < DP ? 0 : u < 2 * DP ? 1 : u < 2 * DP + vp ? 2 : 3;
+    const int c = kind == 3 ? u - 2 * DP - vp : u - kind * DP;
+    float y[C];
+    if (c >= (kind == 2 ? a.Dv : a.D)) {
 #pragma unroll
-  for (int i = 0; i < C * DP / 256; ++i) {
-    const int e = tid + 256 * i, t = e / DP, d = e % DP;
-    const bool ok = t < n && d < a.D;
-    s_k[t * LS + d] = ok ? to_f32<TQ>(k[(size_t)t * ldk + d]) : 0.f;
-    s_q[t * LS + d] = ok ? to_f32<TQ>(q[(size_t)t * ldq + d]) * q_scale : 0.f;
-    s_g[t * LS + d] = ok ? expf(lg[(size_t)t * a.ld_low + d]) : 1.f;
+      for (int t = 0; t < C; ++t) y[t] = kind == 3 ? 1.f : 0.f;
+    } else if (kind == 3) {
+      const float* z = a.low + (size_t)m0 * a.ld_low + a.off_z + (size_t)h * a.D + c;
+#pragma unroll
+      for (int t = 0; t < C; ++t) y[t] = t < n ? z[(size_t)t * a.ld_low] : 0.f;
+#pragma unroll
+      for (int t = 0; t < C; ++t)
+        y[t] = t < n ? exp_f(log_decay(a, y[t], h, c)) : 1.f;
+    } else {
+      const int col = kind == 0 ? a.off_q + hg * a.D + c
+                      : kind == 1 ? a.off_k + hg * a.D + c : a.off_v + h * a.Dv + c;
+      const int cc = kind == 0 ? hg * a.D + c
+                     : kind == 1 ? (a.G + hg) * a.D + c
+                                 : 2 * a.G * a.D + h * a.Dv + c;
+      if (a.taps == 0)
+        chunk_column<0, T>(g, m0, n, chunk * C, pos0, slot, col, cc, y);
+      else if (a.taps <= 4)
+        chunk_column<4, T>(g, m0, n, chunk * C, pos0, slot, col, cc, y);
+      else
+        chunk_column<kChunkTaps, T>(g, m0, n, chunk * C, pos0, slot, col, cc, y);
+#pragma unroll
+      for (int t = 0; t < C; ++t)  // the convolution reaches past the end
+        if (t >= n) y[t] = 0.f;
+    }
+    float* dst = kind == 0 ? s_q : kind == 1 ? s_k : kind == 2 ? s_v : s_g;
+    const int stride = kind == 2 ? vp : LS;
+#pragma unroll
+    for (int t = 0; t < C; ++t) dst[t * stride + c] = y[t];
   }
-  if (tid < C) s_beta[tid] = DELTA && tid < n ? g.wbeta[(size_t)(m0 + tid) * a.H + h] : 0.f;
+  if (tid < C)
+    s_beta[tid] =
+        DELTA && tid < n
+            ? sigmoid_f(to_f32<T>(reinterpret_cast<const T*>(
+                  a.proj)[(size_t)(m0 + tid) * a.ld_proj + a.off_beta + h]))
+            : 0.f;
   s_a[tid >> 4][tid & 15] = 0.f;
   s_b[tid >> 4][tid & 15] = 0.f;
+  __syncthreads();
+  {
+    // unit norms and the query's factor: 8 lanes per row of q, then of k
+    const bool query = tid < 128;
+    float* row = (query ? s_q : s_k) + ((tid >> 3) & 15) * LS + 4 * (tid & 7);
+    float f = query ? a.q_scale : 1.f;
+    if (a.unit) {
+      float ss = 0.f;
+#pragma unroll
+      for (int e = 0; e < DP / 32; ++e) {
+        const float4 x = *reinterpret_cast<const float4*>(row + 32 * e);
+        ss = fmaf(x.x, x.x, ss); ss = fmaf(x.y, x.y, ss);
+        ss = fmaf(x.z, x.z, ss); ss = fmaf(x.w, x.w, ss);
+      }
+      ss += dpp_move<kDppXor1>(ss);
+      ss += dpp_move<kDppXor2>(ss);
+      ss += dpp_move<kDppHalfMirror>(ss);
+      f /= sqrtf(ss + a.unit_eps);
+    }
+    if (a.unit || query) {
+#pragma unroll
+      for (int e = 0; e < DP / 32; ++e) {
+        float4 x = *reinterpret_cast<const float4*>(row + 32 * e);
+        x.x *= f; x.y *= f; x.z *= f; x.w *= f;
+        *reinterpret_cast<float4*>(row + 32 * e) = x;
+      }
+    }
+  }
   __syncthreads();
   {
     // 32 lanes per source token s, which walk t = s .. 15 with k_s decayed on
@@ -356,7 +463,6 @@ recurrence_chunk_kernel(RecArgs g, const TQ* q_rows, const TQ* k_rows,
   }
   __syncthreads();
 
-  const int vp = (a.Dv + 15) / 16 * 16;
   const ChunkLayout lay(DP, vp);
   float* w = g.wchunk + ((chunk_base(off, seq) + chunk) * a.H + h) * lay.size();
   // A thread per channel, then per value column: the triangular solve and the
@@ -364,41 +470,48 @@ recurrence_chunk_kernel(RecArgs g, const TQ* q_rows, const TQ* k_rows,
   for (int c = tid; c < DP + vp; c += 256) {
     const bool channel = c < DP;
     const int vc = c - DP;
-    float x[C], upto[C];  // solution; decay up to and with token t
-    float run = 1.f;
+    // (a zero the compiler cannot see through: it would otherwise read all of A
+    // and B into registers ahead of this loop)
+    int z = 0;
+    asm volatile("" : "+s"(z));
+    float x[C], run = 1.f;
+    float* sq = s_q + c;
+    float* sk = s_k + c;
+    float* sg = s_g + c;  // of a channel: read and written by this thread alone
 #pragma unroll
     for (int t = 0; t < C; ++t) {
+      __builtin_amdgcn_sched_barrier(0);
       float rhs;
       if (channel) {
-        run *= s_g[t * LS + c];
-        upto[t] = run;
-        rhs = s_k[t * LS + c] * run;
+        run *= sg[t * LS];
+        rhs = sk[t * LS] * run;
       } else {
-        rhs = t < n && vc < a.Dv ? to_f32<TQ>(v[(size_t)t * ldv + vc]) : 0.f;
+        rhs = s_v[t * vp + vc];
       }
       if (DELTA) {
 #pragma unroll
-        for (int s = 0; s < t; ++s) rhs = fmaf(-s_a[t][s], x[s], rhs);
+        for (int s = 0; s < t; ++s) rhs = fmaf(-s_a[t + z][s], x[s], rhs);
         rhs *= s_beta[t];
       }
       x[t] = rhs;
-    }
-    if (channel) {
-      // this thread's column of the three arrays is read by no other thread
-      float back = 1.f;
-      w[lay.pc() + c] = run;
-#pragma unroll
-      for (int t = C - 1; t >= 0; --t) {
-        float y = s_q[t * LS + c] * upto[t];
+      if (channel) {
+        float y = sq[t * LS] * run;
         if (DELTA) {
 #pragma unroll
-          for (int s = 0; s <= t; ++s) y = fmaf(-s_b[t][s], x[s], y);
+          for (int s = 0; s <= t; ++s) y = fmaf(-s_b[t + z][s], x[s], y);
         }
-        const float gt = s_g[t * LS + c];
-        s_g[t * LS + c] = s_k[t * LS + c] * back;
+        sq[t * LS] = y;
+      }
+    }
+    if (channel) {
+      w[lay.pc() + c] = run;
+      float back = 1.f;
+#pragma unroll
+      for (int t = C - 1; t >= 0; --t) {
+        const float gt = sg[t * LS];
+        sg[t * LS] = sk[t * LS] * back;
         back *= gt;
-        s_q[t * LS + c] = y;
-        if (DELTA) s_k[t * LS + c] = x[t];
+        if (DELTA) sk[t * LS] = x[t];
       }
     } else {
       float4* us = reinterpret_cast<float4*>(w + lay.us()) + (vc >> 4) * 64 + (vc & 15);
@@ -406,9 +519,10 @@ recurrence_chunk_kernel(RecArgs g, const TQ* q_rows, const TQ* k_rows,
       float y[C];
 #pragma unroll
       for (int t = 0; t < C; ++t) {
+        __builtin_amdgcn_sched_barrier(0);
         y[t] = 0.f;
 #pragma unroll
-        for (int s = 0; s <= t; ++s) y[t] = fmaf(s_b[t][s], x[s], y[t]);
+        for (int s = 0; s <= t; ++s) y[t] = fmaf(s_b[t + z][s], x[s], y[t]);
       }
 #pragma unroll
       for (int q4 = 0; q4 < 4; ++q4) {
@@ -430,7 +544,6 @@ recurrence_chunk_kernel(RecArgs g, const TQ* q_rows, const TQ* k_rows,
     reinterpret_cast<float4*>(w + lay.kh())[f] =
         make_float4(kh[0], kh[LS], kh[2 * LS], kh[3 * LS]);
   }
-  (void)lane;
 }
 
 // Walks the chunks of one (sequence, head) for 16 value columns.  Each of 4
@@ -443,14 +556,19 @@ recurrence_chain_kernel(RecArgs g) {
   __shared__ float4 s_o[2][4][64];
   T5D_GATED(g.gate);
   const t5d_recurrence& a = g.a;
-  const int vt = blockIdx.x, h = blockIdx.y, seq = blockIdx.z;
+  // The workgroups of one (sequence, head) read the same operands: consecutive
+  // block ids go round-robin over the 8 XCDs, so theirs are 8 apart.
+  const int vp = (a.Dv + 15) / 16 * 16, vts = vp / 16;
+  const int pair = (blockIdx.x & 7) + 8 * ((blockIdx.x >> 3) / vts);
+  if (pair >= a.H * g.b.S) return;
+  const int vt = (blockIdx.x >> 3) % vts, h = pair % a.H, seq = pair / a.H;
   const int off = g.b.seq_off[seq], len = g.b.seq_off[seq + 1] - off;
   if (len <= 0) return;
   const int start = g.b.seq_start[seq], slot = g.b.seq_slot[seq];
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int x = lane & 15, g4 = lane >> 4;
-  const int vp = (int)gridDim.x * 16, col = 16 * vt + x;
+  const int col = 16 * vt + x;
   const bool col_ok = col < a.Dv;
   const ChunkLayout lay(DP, vp);
   const int nc = (len + kChunk - 1) / kChunk;
@@ -489,27 +607,33 @@ recurrence_chain_kernel(RecArgs g) {
   auto step = [&](const Operands& o, int c) {
     const int buf = c & 1;
     f32x4_v u = (f32x4_v){0.f, 0.f, 0.f, 0.f}, r = u;
+    if (DELTA) {
+#pragma unroll
+      for (int t = 0; t < NTW; ++t) {
+        const float wk[4] = {o.wk[t].x, o.wk[t].y, o.wk[t].z, o.wk[t].w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          u = __builtin_amdgcn_mfma_f32_16x16x4f32(wk[i], st[t][i], u, 0, 0, 0);
+      }
+    }
 #pragma unroll
     for (int t = 0; t < NTW; ++t) {
       const float qs[4] = {o.qs[t].x, o.qs[t].y, o.qs[t].z, o.qs[t].w};
-      const float wk[4] = {o.wk[t].x, o.wk[t].y, o.wk[t].z, o.wk[t].w};
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        if (DELTA)
-          u = __builtin_amdgcn_mfma_f32_16x16x4f32(wk[i], st[t][i], u, 0, 0, 0);
+      for (int i = 0; i < 4; ++i)
         r = __builtin_amdgcn_mfma_f32_16x16x4f32(qs[i], st[t][i], r, 0, 0, 0);
-      }
     }
     if (DELTA) s_u[buf][wave][lane] = make_float4(u[0], u[1], u[2], u[3]);
     s_o[buf][wave][lane] = make_float4(r[0], r[1], r[2], r[3]);
     __syncthreads();
     float uu[4] = {o.us.x, o.us.y, o.us.z, o.us.w};
     if (DELTA) {
-#pragma unroll
-      for (int p = 0; p < 4; ++p) {
-        const float4 q = s_u[buf][p][lane];
-        uu[0] -= q.x; uu[1] -= q.y; uu[2] -= q.z; uu[3] -= q.w;
-      }
+      const float4 p0 = s_u[buf][0][lane], p1 = s_u[buf][1][lane];
+      const float4 p2 = s_u[buf][2][lane], p3 = s_u[buf][3][lane];
+      uu[0] -= (p0.x + p1.x) + (p2.x + p3.x);
+      uu[1] -= (p0.y + p1.y) + (p2.y + p3.y);
+      uu[2] -= (p0.z + p1.z) + (p2.z + p3.z);
+      uu[3] -= (p0.w + p1.w) + (p2.w + p3.w);
     }
 #pragma unroll
     for (int t = 0; t < NTW; ++t) {
@@ -528,14 +652,18 @@ recurrence_chain_kernel(RecArgs g) {
     const int tok = kChunk * c + 4 * g4 + wave;
     if (tok < len && col_ok) out[(size_t)tok * a.H * a.Dv] = y;
   };
-  Operands o0, o1;
-  load(o0, 0);
-  for (int c = 0; c < nc; c += 2) {
-    load(o1, min(c + 1, nc - 1));
-    step(o0, c);
-    if (c + 1 >= nc) break;
-    load(o0, min(c + 2, nc - 1));
-    step(o1, c + 1);
+  // The operands of the next chunks are on their way while one is multiplied.
+  constexpr int DEPTH = NTW <= 4 ? 4 : 2;
+  Operands o[DEPTH];
+#pragma unroll
+  for (int i = 0; i + 1 < DEPTH; ++i) load(o[i], min(i, nc - 1));
+  for (int c0 = 0; c0 < nc; c0 += DEPTH) {
+#pragma unroll
+    for (int i = 0; i < DEPTH; ++i) {
+      if (c0 + i >= nc) break;
+      load(o[(i + DEPTH - 1) % DEPTH], min(c0 + i + DEPTH - 1, nc - 1));
+      step(o[i], c0 + i);
+    }
   }
 #pragma unroll
   for (int t = 0; t < NTW; ++t)
@@ -579,12 +707,54 @@ __device__ __forceinline__ float out_gate(const t5d_recurrence& a, int m, int h,
   return z * sigmoid_f(z);
 }
 
-template <typename T>
+// A wavefront per (token, head); with VEC 4 columns per lane, two heads of up to
+// 128 columns per wavefront.
+template <typename T, bool VEC>
 __global__ void __launch_bounds__(256)
 recurrence_finish_kernel(RecArgs g) {
   T5D_GATED(g.gate);
   const t5d_recurrence& a = g.a;
   const int lane = threadIdx.x & 63;
+  if constexpr (VEC) {
+    const int64_t unit = (int64_t)blockIdx.x * 8 + (threadIdx.x >> 5);
+    const bool on = unit < (int64_t)g.b.M * a.H;
+    const int m = on ? unit / a.H : 0, h = on ? unit % a.H : 0;
+    const int c = 4 * (lane & 31);
+    const bool ok = on && c < a.Dv;
+    float4 o = make_float4(0.f, 0.f, 0.f, 0.f), z = o;
+    if (ok) {
+      o = *reinterpret_cast<const float4*>(g.wo + (size_t)unit * a.Dv + c);
+      if (a.gate == T5D_GATE_SIGMOID_LOW) {
+        z = *reinterpret_cast<const float4*>(a.low + (size_t)m * a.ld_low +
+                                             a.off_low_gate + (size_t)h * a.Dv + c);
+      } else {
+        const T* p = reinterpret_cast<const T*>(a.proj) + (size_t)m * a.ld_proj +
+                     a.off_gate + (size_t)h * a.Dv + c;
+        z = make_float4(to_f32<T>(p[0]), to_f32<T>(p[1]), to_f32<T>(p[2]),
+                        to_f32<T>(p[3]));
+      }
+    }
+    float ss = lanes16_sum(o.x * o.x + o.y * o.y + o.z * o.z + o.w * o.w);
+    const auto w = __builtin_amdgcn_permlane16_swap(
+        __float_as_uint(ss), __float_as_uint(ss), false, false);
+    ss = __uint_as_float(w[0]) + __uint_as_float(w[1]);
+    if (!ok) return;
+    const float inv = 1.0f / sqrtf(ss / (float)a.Dv + a.eps);
+    const bool silu = a.gate != T5D_GATE_SIGMOID_LOW;
+    auto put = [&](float v, float zz, float nw) {
+      return v * inv * nw * (silu ? zz * sigmoid_f(zz) : sigmoid_f(zz));
+    };
+    const float y0 = put(o.x, z.x, a.norm[c]), y1 = put(o.y, z.y, a.norm[c + 1]);
+    const float y2 = put(o.z, z.z, a.norm[c + 2]), y3 = put(o.w, z.w, a.norm[c + 3]);
+    T* out = reinterpret_cast<T*>(a.out) + (size_t)m * a.ld_out + (size_t)h * a.Dv + c;
+    if constexpr (sizeof(T) == 2) {
+      *reinterpret_cast<uint2*>(out) =
+          make_uint2(pack_bf16x2(y0, y1), pack_bf16x2(y2, y3));
+    } else {
+      *reinterpret_cast<float4*>(out) = make_float4(y0, y1, y2, y3);
+    }
+    return;
+  }
   const int64_t unit = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (unit >= (int64_t)g.b.M * a.H) return;
   const int m = unit / a.H, h = unit % a.H;
@@ -741,18 +911,18 @@ static void launch_scan(hipStream_t s, const RecArgs& g, const TQ* q, const TQ* 
 #undef T5D_SC
 }
 
-template <bool DELTA, typename TQ>
-static void launch_chunks(hipStream_t s, const RecArgs& g, const TQ* q,
-                          const TQ* k, const TQ* v, int ldq, int ldk, int ldv,
-                          float q_scale) {
+template <bool DELTA, typename T>
+static void launch_chunks(hipStream_t s, const RecArgs& g) {
+  const int vts = (g.a.Dv + 15) / 16, pairs = g.a.H * g.b.S;
   const dim3 grid(g.chunks, g.a.H, g.b.S), block(256);
-  const dim3 cgrid((g.a.Dv + 15) / 16, g.a.H, g.b.S);
-#define T5D_CH(E_)                                                              \
-  do {                                                                          \
-    hipLaunchKernelGGL((recurrence_chunk_kernel<64 * E_, DELTA, TQ>), grid,     \
-                       block, 0, s, g, q, k, v, ldq, ldk, ldv, q_scale);        \
-    hipLaunchKernelGGL((recurrence_chain_kernel<E_, DELTA>), cgrid, block, 0, s, \
-                       g);                                                      \
+  const dim3 chain((pairs + 7) / 8 * 8 * vts);
+  const size_t lds = (size_t)kChunk * vts * 16 * sizeof(float);
+#define T5D_CH(E_)                                                               \
+  do {                                                                           \
+    hipLaunchKernelGGL((recurrence_chunk_kernel<64 * E_, DELTA, T>), grid, block, \
+                       lds, s, g);                                               \
+    hipLaunchKernelGGL((recurrence_chain_kernel<E_, DELTA>), chain, block, 0, s, \
+                       g);                                                       \
   } while (0)
   if (g.a.D <= 64) T5D_CH(1);
   else if (g.a.D <= 128) T5D_CH(2);
@@ -761,49 +931,51 @@ static void launch_chunks(hipStream_t s, const RecArgs& g, const TQ* q,
 #undef T5D_CH
 }
 
-// The recurrence of a portion: chunks, or token by token (g.wchunk null).
-template <bool DELTA, typename TQ>
-static void launch_recurrence(hipStream_t s, const RecArgs& g, const TQ* q,
-                              const TQ* k, const TQ* v, int ldq, int ldk, int ldv,
-                              float q_scale) {
-  if (g.wchunk != nullptr)
-    launch_chunks<DELTA, TQ>(s, g, q, k, v, ldq, ldk, ldv, q_scale);
-  else
-    launch_scan<DELTA, TQ>(s, g, q, k, v, ldq, ldk, ldv, q_scale);
-}
-
-template <typename T>
-static int run_portions(hipStream_t s, const RecArgs& g) {
+// Prepare and scan.
+template <bool DELTA, typename T>
+static void launch_token_by_token(hipStream_t s, const RecArgs& g) {
   const t5d_recurrence& a = g.a;
   const bool qkv = a.taps > 0 || a.unit;
   const int64_t units = (int64_t)g.b.M * ((qkv ? 2 * a.G + a.H : 0) + a.H);
   hipLaunchKernelGGL(recurrence_prepare_kernel<T>, dim3((unsigned)((units + 3) / 4)),
                      dim3(256), 0, s, g);
-  T5D_CHECK_LAUNCH("recurrence (prepare)");
   if (qkv) {
-    const int gd = a.G * a.D, hv = a.H * a.Dv;
-    if (a.delta)
-      launch_recurrence<true, float>(s, g, g.wq, g.wk, g.wv, gd, gd, hv, 1.f);
-    else
-      launch_recurrence<false, float>(s, g, g.wq, g.wk, g.wv, gd, gd, hv, 1.f);
+    launch_scan<DELTA, float>(s, g, g.wq, g.wk, g.wv, a.G * a.D, a.G * a.D,
+                              a.H * a.Dv, 1.f);
   } else {
     const T* p = reinterpret_cast<const T*>(a.proj);
-    if (a.delta)
-      launch_recurrence<true, T>(s, g, p + a.off_q, p + a.off_k, p + a.off_v, a.ld_proj,
-                           a.ld_proj, a.ld_proj, a.q_scale);
-    else
-      launch_recurrence<false, T>(s, g, p + a.off_q, p + a.off_k, p + a.off_v, a.ld_proj,
-                            a.ld_proj, a.ld_proj, a.q_scale);
+    launch_scan<DELTA, T>(s, g, p + a.off_q, p + a.off_k, p + a.off_v, a.ld_proj,
+                          a.ld_proj, a.ld_proj, a.q_scale);
   }
-  T5D_CHECK_LAUNCH("recurrence (scan)");
+}
+
+template <typename T>
+static int run_portions(hipStream_t s, const RecArgs& g) {
+  const t5d_recurrence& a = g.a;
+  if (g.wchunk != nullptr) {
+    if (a.delta) launch_chunks<true, T>(s, g);
+    else launch_chunks<false, T>(s, g);
+  } else if (a.delta) {
+    launch_token_by_token<true, T>(s, g);
+  } else {
+    launch_token_by_token<false, T>(s, g);
+  }
+  T5D_CHECK_LAUNCH("recurrence (portions)");
   if (a.taps > 1) {
     hipLaunchKernelGGL(recurrence_conv_tail_kernel<T>,
                        dim3((g.C + 255) / 256, g.b.S), dim3(256), 0, s, g);
     T5D_CHECK_LAUNCH("recurrence (convolution tail)");
   }
   const int64_t heads = (int64_t)g.b.M * a.H;
-  hipLaunchKernelGGL(recurrence_finish_kernel<T>, dim3((unsigned)((heads + 3) / 4)),
-                     dim3(256), 0, s, g);
+  const bool vec = a.Dv % 4 == 0 && a.Dv <= 128 && a.ld_out % 4 == 0 &&
+                   a.ld_low % 4 == 0 && a.off_low_gate % 4 == 0 &&
+                   ((uintptr_t)a.out | (uintptr_t)a.low) % 16 == 0;
+  if (vec)
+    hipLaunchKernelGGL((recurrence_finish_kernel<T, true>),
+                       dim3((unsigned)((heads + 7) / 8)), dim3(256), 0, s, g);
+  else
+    hipLaunchKernelGGL((recurrence_finish_kernel<T, false>),
+                       dim3((unsigned)((heads + 3) / 4)), dim3(256), 0, s, g);
   T5D_CHECK_LAUNCH("recurrence (finish)");
   return T5D_OK;
 }
@@ -892,6 +1064,7 @@ extern "C" int t5d_recurrence_run(void* stream, const t5d_recurrence* a,
   const int64_t plain = portion_floats(b->M, a->H, a->G, a->D, a->Dv);
   g.chunks = (b->max_len + kChunk - 1) / kChunk;
   const bool fits =
+      a->taps <= kChunkTaps && a->Dv <= 512 &&
       a->workspace_bytes >=
       4 * (plain + chunk_floats(b->M, b->S, a->H, a->D, a->Dv));
   T5D_REQUIRE(a->workspace_bytes >= 4 * plain && (variant != 3 || fits), T5D_EINVAL,

@@ -92,6 +92,55 @@ window_append_kernel(WinArgs g) {
   }
 }
 
+// The same for bfloat16 rows of whole 16-byte pieces: HP / 8 lanes per vector.
+__global__ void __launch_bounds__(256)
+window_append_vec_kernel(WinArgs g) {
+  T5D_GATED(g.gate);
+  const t5d_window_attention& a = g.a;
+  const int lpv = g.HP / 8;  // 4, 8, 16 or 32: a power of two
+  const int nvec = a.H + 2 * a.G;
+  const int64_t unit = (int64_t)blockIdx.x * (256 / lpv) + threadIdx.x / lpv;
+  const bool on = unit < (int64_t)g.b.M * nvec;
+  const int m = on ? unit / nvec : 0, vec = on ? unit % nvec : 0;
+  const int c = 8 * (threadIdx.x % lpv);
+  const bool query = vec < a.H, key = !query && vec < a.H + a.G;
+  const int h = query ? vec : vec - a.H - (key ? 0 : a.G);
+  const int n = query || key ? a.D : a.Dv;
+  const bf16_t* p = reinterpret_cast<const bf16_t*>(a.proj) + (size_t)m * a.ld_proj +
+                    (query ? a.off_q + h * a.D : key ? a.off_k + h * a.D
+                                                     : a.off_v + h * a.Dv);
+  const float* w = query ? a.q_norm : key ? a.k_norm : nullptr;
+  uint4 v = make_uint4(0, 0, 0, 0);
+  if (on && c < n) v = *reinterpret_cast<const uint4*>(p + c);
+  if (w != nullptr) {
+    float f[8];
+    unpack16(v, f);
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss = fmaf(f[e], f[e], ss);
+    for (int step = 1; step < lpv; step *= 2) ss += __shfl_xor(ss, step, 64);
+    const float inv = 1.0f / sqrtf(ss / (float)n + a.eps);
+    if (c < n) {
+      const float4 x = *reinterpret_cast<const float4*>(w + c);
+      const float4 y = *reinterpret_cast<const float4*>(w + c + 4);
+      v.x = pack_bf16x2(f[0] * inv * x.x, f[1] * inv * x.y);
+      v.y = pack_bf16x2(f[2] * inv * x.z, f[3] * inv * x.w);
+      v.z = pack_bf16x2(f[4] * inv * y.x, f[5] * inv * y.y);
+      v.w = pack_bf16x2(f[6] * inv * y.z, f[7] * inv * y.w);
+    }
+  }
+  if (!on) return;
+  bf16_t* dst;
+  if (query) {
+    dst = reinterpret_cast<bf16_t*>(a.q_rows) + ((size_t)m * a.H + h) * g.HP;
+  } else {
+    const size_t r = ((size_t)g.b.seq_slot[g.b.tok_seq[m]] * a.G + h) * a.ring +
+                     g.b.tok_pos[m] % a.ring;
+    dst = reinterpret_cast<bf16_t*>(key ? a.key_ring : a.value_ring) + r * g.HP;
+  }
+  *reinterpret_cast<uint4*>(dst + c) = v;
+}
+
 // ---- float32 / any size -----------------------------------------------------------
 template <typename T, int NV>
 __global__ void __launch_bounds__(64)
@@ -166,7 +215,7 @@ __device__ __forceinline__ f32x4_v mfma(const Frag& x, const Frag& y, f32x4_v c)
 }
 
 template <int DT>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1)
 window_rows_kernel(WinArgs g) {
   constexpr int HP = DT * 32, VT = DT * 2, KB = 64, MT = 2;
   constexpr int KS = HP + 8, VS = KB + 8;        // LDS row strides (elements)
@@ -223,7 +272,7 @@ window_rows_kernel(WinArgs g) {
   const int wi_hi = start + min(rw + 16 * MT - 1, rows - 1) / gs;
   const int j_begin = max(0, i_lo - W + 1) & ~(KB - 1);
 
-  uint4 kr[DT], vr[NVP][2];
+  uint4 kr[DT], va[NVP], vb[NVP];
   const int kpiece = threadIdx.x % (HP / 8), krow = threadIdx.x / (HP / 8);
   constexpr int KRS = 256 / (HP / 8);            // key rows per pass
   const int vpair = threadIdx.x & 31, vcol = threadIdx.x >> 5;
@@ -237,8 +286,8 @@ window_rows_kernel(WinArgs g) {
     for (int i = 0; i < NVP; ++i)
       if (vcol + 8 * i < HP / 8) {
         const bf16_t* v = V + (r + 2 * vpair) * HP + 8 * (vcol + 8 * i);
-        vr[i][0] = *reinterpret_cast<const uint4*>(v);
-        vr[i][1] = *reinterpret_cast<const uint4*>(v + HP);
+        va[i] = *reinterpret_cast<const uint4*>(v);
+        vb[i] = *reinterpret_cast<const uint4*>(v + HP);
       }
   };
   fetch(j_begin);
@@ -251,15 +300,16 @@ window_rows_kernel(WinArgs g) {
     for (int i = 0; i < NVP; ++i)
       if (vcol + 8 * i < HP / 8) {
         // keys 2p and 2p + 1 of 8 dims: one word per dim
-        const uint32_t x[4] = {vr[i][0].x, vr[i][0].y, vr[i][0].z, vr[i][0].w};
-        const uint32_t y[4] = {vr[i][1].x, vr[i][1].y, vr[i][1].z, vr[i][1].w};
         uint32_t* dst = reinterpret_cast<uint32_t*>(
             s_v + (size_t)(8 * (vcol + 8 * i)) * VS + 2 * vpair);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          dst[(2 * e) * (VS / 2)] = (x[e] & 0xFFFFu) | (y[e] << 16);
-          dst[(2 * e + 1) * (VS / 2)] = (x[e] >> 16) | (y[e] & 0xFFFF0000u);
-        }
+        auto put = [&](int e, uint32_t x, uint32_t y) {
+          dst[(2 * e) * (VS / 2)] = (x & 0xFFFFu) | (y << 16);
+          dst[(2 * e + 1) * (VS / 2)] = (x >> 16) | (y & 0xFFFF0000u);
+        };
+        put(0, va[i].x, vb[i].x);
+        put(1, va[i].y, vb[i].y);
+        put(2, va[i].z, vb[i].z);
+        put(3, va[i].w, vb[i].w);
       }
     __syncthreads();
     if (jt + KB <= i_hi) fetch(jt + KB);
@@ -721,7 +771,17 @@ extern "C" int t5d_window_attention_run(void* stream, const t5d_window_attention
   }
   const int64_t units = (int64_t)b->M * (a->H + 2 * a->G);
   const dim3 agrid((unsigned)((units + 3) / 4)), ablock(256);
-  if (bf16)
+  const bool pieces =
+      bf16 && g.HP <= 256 &&
+      ((a->D | a->Dv | a->off_q | a->off_k | a->off_v | a->ld_proj) & 7) == 0 &&
+      (((uintptr_t)a->proj | (uintptr_t)a->q_rows | (uintptr_t)a->key_ring |
+        (uintptr_t)a->value_ring | (uintptr_t)a->q_norm | (uintptr_t)a->k_norm) &
+       15) == 0;
+  if (pieces)
+    hipLaunchKernelGGL(window_append_vec_kernel,
+                       dim3((unsigned)((units * (g.HP / 8) + 255) / 256)), ablock, 0,
+                       s, g);
+  else if (bf16)
     hipLaunchKernelGGL(window_append_kernel<bf16_t>, agrid, ablock, 0, s, g);
   else
     hipLaunchKernelGGL(window_append_kernel<float>, agrid, ablock, 0, s, g);

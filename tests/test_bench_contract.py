@@ -1,5 +1,5 @@
 """bench.py's command-line contract: one GPU only, one JSON line per run with
-the agreed keys.  The GPU cases run the two short stages whose commands the
+the agreed keys.  The GPU cases run the short stages whose commands the
 profile summaries quote (the default decode run is timed by the driver)."""
 
 import json
@@ -31,6 +31,7 @@ def test_more_than_one_gpu_is_refused_with_a_message():
 @pytest.mark.parametrize('flags', [
     ('--stage', 'dense'),
     ('--stage', 'memory'),
+    ('--stage', 'hybrid', '--hybrid-size', 'base', '--hybrid-batch', '1'),
 ])
 def test_short_stages_print_one_json_line(flags):
   r = run_bench(*flags)

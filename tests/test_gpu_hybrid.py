@@ -228,13 +228,15 @@ class Attention:
     return 2e-6 if self.dt == torch.float32 else 6e-3
 
 
-SHAPES = [(4, 2, 48, 48), (3, 1, 20, 70), (8, 8, 64, 64), (2, 1, 100, 128),
-          (16, 1, 32, 24), (6, 2, 200, 36), (5, 5, 16, 10)]
+SHAPES = [(6, 3, 48, 48), (3, 1, 20, 70), (8, 8, 64, 64), (2, 1, 100, 128),
+          (16, 1, 32, 24), (6, 2, 200, 36), (5, 5, 16, 10), (20, 1, 40, 40)]
+WAVE_SHAPES = SHAPES + [(2, 1, 300, 40), (1, 1, 24, 520)]
 
 
-@pytest.mark.parametrize('dt,variant', [(torch.float32, 0), (torch.bfloat16, 2),
-                                        (torch.bfloat16, 3)])
-@pytest.mark.parametrize('H,G,D,Dv', SHAPES)
+@pytest.mark.parametrize('dt,variant,H,G,D,Dv', [
+    (dt, v, *shape) for dt, v, shapes in (
+        (torch.float32, 0, WAVE_SHAPES), (torch.bfloat16, 2, SHAPES),
+        (torch.bfloat16, 3, WAVE_SHAPES)) for shape in shapes])
 @pytest.mark.parametrize('window', [0, 1, 9, 64, 65])
 def test_window_attention_prompts_and_portions(dt, variant, H, G, D, Dv, window):
   T, portion = 150, 70
@@ -249,7 +251,7 @@ def test_window_attention_prompts_and_portions(dt, variant, H, G, D, Dv, window)
     assert rel(np.concatenate(got), want) < a.tol, cuts
 
 
-@pytest.mark.parametrize('H,G,D,Dv', SHAPES)
+@pytest.mark.parametrize('H,G,D,Dv', SHAPES[:-1])  # up to 16 heads per group
 @pytest.mark.parametrize('window', [0, 1, 9, 64, 65, 600])
 def test_window_attention_step_kernel(H, G, D, Dv, window):
   """One token per sequence for sequences of unequal lengths, ring wrapping."""
@@ -455,9 +457,10 @@ def seq_cols(x, at, n):
   return x[:, at:at + n]
 
 
-REC = [(True, 4, 4, 64, 64, 3), (True, 6, 2, 24, 40, 4), (True, 2, 1, 130, 20, 5),
+REC = [(True, 2, 2, 64, 64, 4), (True, 6, 2, 24, 40, 4), (True, 2, 1, 130, 20, 5),
        (True, 2, 2, 200, 256, 2), (True, 3, 1, 8, 6, 1), (True, 1, 1, 40, 33, 0),
-       (False, 4, 4, 32, 32, 0), (False, 3, 3, 20, 36, 0),
+       (True, 2, 1, 300, 24, 3), (True, 1, 1, 16, 260, 9),
+       (False, 5, 5, 32, 32, 0), (False, 3, 3, 20, 36, 0),
        (False, 2, 2, 256, 100, 0), (False, 5, 5, 72, 10, 0)]
 
 
@@ -472,7 +475,7 @@ def test_recurrence_portions_and_steps(dt, strong, delta, H, G, D, Dv, taps):
   seq = r.sequence(T)
   want = r.oracle(seq)
   assert rel(r.run([(1, 0, T)], [seq]), want) < r.tol
-  for variant in (2, 3):  # token by token, in chunks
+  for variant in (2, 3) if taps <= 8 else (2,):  # token by token, in chunks
     assert rel(r.run([(1, 0, T)], [seq], variant), want) < r.tol, variant
     for cuts in ([1, 2, 3, 5, 8, 24, 25, 41, 57], [16, 32, 64], [2, 4, 6, 70]):
       got, at = [], 0
