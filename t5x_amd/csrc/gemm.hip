@@ -27,9 +27,9 @@ namespace t5d {
 
 // NJ > 0: K is NJ * 256, every wavefront owns exactly NJ k-tile pairs and the K
 // loop is straight-line code (see gemm_big_kernel).
-template <int MP, int NT, typename WT, int NJ = 0>
+template <int MP, int NT, typename WT, int NJ = 0, typename Args = GemmArgs>
 __global__ void __launch_bounds__(256)
-gemm_mfma_kernel(GemmArgs g) {
+gemm_mfma_kernel(Args g) {
   constexpr int ACC = MP * NT;
   constexpr int TN = NT * 16;
   // k-tile pairs in flight per wavefront (an unrolled loop that requests all
@@ -109,10 +109,10 @@ gemm_mfma_kernel(GemmArgs g) {
         const int row = m0 + mt * 16 + arow;
         if (NJ > 0)  // rows past the edge are never stored
           aq[slot_][h][mt] = *reinterpret_cast<const uint4*>(
-              g.A + (size_t)min(row, g.M - 1) * g.lda + (kt + h) * 32 + akoff);
+              g.A + (size_t)min(row, g.M - 1) * row_stride(g) + (kt + h) * 32 + akoff);
         else if (row < g.M && kt + h < KT)
           aq[slot_][h][mt] = *reinterpret_cast<const uint4*>(
-              g.A + (size_t)row * g.lda + (kt + h) * 32 + akoff);
+              g.A + (size_t)row * row_stride(g) + (kt + h) * 32 + akoff);
         else
           aq[slot_][h][mt] = make_uint4(0, 0, 0, 0);
       }
@@ -219,7 +219,7 @@ gemm_mfma_kernel(GemmArgs g) {
     __syncthreads();
   }
 
-  const bool geglu = is_gated(g.epilogue);
+  const bool geglu = gated(g);
   auto tile_sum = [&](int ml, int nl) -> float {
     const int mt = ml >> 4, i = ml & 3, c = (ml & 15) >> 2;
     const int nn = nl >> 4, l = c * 16 + (nl & 15);
@@ -233,7 +233,7 @@ gemm_mfma_kernel(GemmArgs g) {
   auto finish = [&](int e, float r) {
     const int ml = e / TN, nl = e % TN;
     const int m = m0 + ml, n = nt0 * 16 + nl;
-    if (m >= g.M || n >= g.n_store) return;
+    if (m >= g.M || n >= stored_columns(g)) return;
     if (geglu && (nl & 8)) return;
     float v = tile_sum(ml, nl);
     float vg = geglu ? tile_sum(ml, nl + 8) : 0.f;
@@ -386,7 +386,7 @@ norm_gemm_kernel(GemmArgs g) {
     for (int i = 0; i < 4; ++i) red[wave][t * 4 + i][lane] = acc[t][i];
   __syncthreads();
 
-  const bool geglu = is_gated(g.epilogue);
+  const bool geglu = gated(g);
   auto tile_sum = [&](int ml, int nl) -> float {
     const int i = ml & 3, c = (ml & 15) >> 2;
     const int nn = nl >> 4, l = c * 16 + (nl & 15);
@@ -638,11 +638,12 @@ norm_gemm_wide_kernel(GemmArgs g, int G, int halves) {
 // 1/rms, which is common to the whole row, multiplies the finished sum.
 constexpr int kF32Rows = 8, kF32Cols = 16;
 
-template <int WV, bool NORMED>
+// DENSE: what t5d_dense adds (lda, the clamped gated unit).
+template <int WV, bool NORMED, bool DENSE = false>
 __global__ void __launch_bounds__(64 * WV)
 gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
                 const float* __restrict__ residual, float* __restrict__ C,
-                int M, int K, int N, int lda, int epilogue,
+                int M, int K, int N, int lda_arg, int epilogue,
                 const int32_t* gate, const float* __restrict__ norm_scale,
                 float eps, float glu_limit, float glu_alpha) {
   static_assert(WV == 4 || WV == 16, "wavefronts per workgroup");
@@ -653,7 +654,9 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int c = lane & 15, sub = lane >> 4;
-  const bool geglu = is_gated(epilogue);
+  const int lda = DENSE ? lda_arg : K;
+  const bool geglu =
+      epilogue == (DENSE ? T5D_EPI_CLAMPED_GLU : T5D_EPI_GEGLU);
   const int F = N >> 1;
   const int ncols = geglu ? F : N;  // columns of work
   const int n = blockIdx.x * kF32Cols + c;
@@ -782,9 +785,7 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
     if (geglu) {
       float vg = total(MB + m, l) * inv;
       C[(size_t)row * F + col] =
-          epilogue == T5D_EPI_GEGLU
-              ? gelu_tanh(v) * vg
-              : clamped_glu(v, vg, glu_limit, glu_alpha);
+          DENSE ? clamped_glu(v, vg, glu_limit, glu_alpha) : gelu_tanh(v) * vg;
     } else {
       if (epilogue == T5D_EPI_RESIDUAL) v += residual[(size_t)row * N + col];
       C[(size_t)row * N + col] = v;
@@ -947,8 +948,8 @@ static bool plan_big(int M, int K, int N, int w_bytes, GemmPlan* out) {
   return found;
 }
 
-template <typename WT>
-static void launch_mfma(const GemmPlan& p, GemmArgs g, hipStream_t s) {
+template <typename WT, typename Args>
+static void launch_mfma(const GemmPlan& p, Args g, hipStream_t s) {
   g.m_parts = p.m_parts;
   const int groups8 = (p.n_groups + 7) / 8 * 8;
   dim3 grid(groups8 * p.m_parts), block(256);
@@ -956,8 +957,8 @@ static void launch_mfma(const GemmPlan& p, GemmArgs g, hipStream_t s) {
   const int nj = g.K % 256 == 0 ? g.K / 256 : 0;
 #define T5D_GEMM_NJ(MT, NT_, NJ_)                                           \
   if (p.mp == MT && p.nt == NT_ && nj == NJ_) {                             \
-    hipLaunchKernelGGL((gemm_mfma_kernel<MT, NT_, WT, NJ_>), grid, block, 0, \
-                       s, g);                                               \
+    hipLaunchKernelGGL((gemm_mfma_kernel<MT, NT_, WT, NJ_, Args>), grid,     \
+                       block, 0, s, g);                                     \
     return;                                                                 \
   }
   T5D_GEMM_NJ(1, 1, 3) T5D_GEMM_NJ(1, 1, 4)
@@ -966,7 +967,8 @@ static void launch_mfma(const GemmPlan& p, GemmArgs g, hipStream_t s) {
 #undef T5D_GEMM_NJ
 #define T5D_GEMM_CASE(MT, NT_)                                              \
   if (p.mp == MT && p.nt == NT_) {                                          \
-    hipLaunchKernelGGL((gemm_mfma_kernel<MT, NT_, WT>), grid, block, 0, s, g); \
+    hipLaunchKernelGGL((gemm_mfma_kernel<MT, NT_, WT, 0, Args>), grid, block, \
+                       0, s, g);                                            \
     return;                                                                 \
   }
   T5D_GEMM_CASE(1, 1) T5D_GEMM_CASE(1, 2) T5D_GEMM_CASE(1, 4)
@@ -991,15 +993,13 @@ bool t5d::norm_gemm_is_wide(int w_dtype, int K, int N) {
 static void launch_gemm_f32(hipStream_t s, const float* A, const float* W,
                             const float* residual, float* C, int M, int K,
                             int N, int epilogue, const float* norm_scale,
-                            float eps, int lda = 0, float glu_limit = 0.f,
-                            float glu_alpha = 0.f) {
-  if (lda == 0) lda = K;
-  const int ncols = is_gated(epilogue) ? N / 2 : N;
+                            float eps) {
+  const int ncols = epilogue == T5D_EPI_GEGLU ? N / 2 : N;
   dim3 grid((ncols + kF32Cols - 1) / kF32Cols, (M + kF32Rows - 1) / kF32Rows);
 #define T5D_F32_LAUNCH(WV_, NORMED_)                                          \
   hipLaunchKernelGGL((gemm_f32_kernel<WV_, NORMED_>), grid, dim3(64 * WV_), 0, \
-                     s, A, W, residual, C, M, K, N, lda, epilogue, tls_gate,  \
-                     norm_scale, eps, glu_limit, glu_alpha)
+                     s, A, W, residual, C, M, K, N, K, epilogue, tls_gate,    \
+                     norm_scale, eps, 0.f, 0.f)
   if (K >= 128) {
     if (norm_scale) T5D_F32_LAUNCH(16, true);
     else T5D_F32_LAUNCH(16, false);
@@ -1007,6 +1007,21 @@ static void launch_gemm_f32(hipStream_t s, const float* A, const float* W,
     if (norm_scale) T5D_F32_LAUNCH(4, true);
     else T5D_F32_LAUNCH(4, false);
   }
+#undef T5D_F32_LAUNCH
+}
+
+static void launch_dense_f32(hipStream_t s, const float* A, int lda, const float* W,
+                             float* C, int M, int K, int N, int epilogue,
+                             float glu_limit, float glu_alpha) {
+  const int ncols = epilogue == T5D_EPI_CLAMPED_GLU ? N / 2 : N;
+  dim3 grid((ncols + kF32Cols - 1) / kF32Cols, (M + kF32Rows - 1) / kF32Rows);
+#define T5D_F32_LAUNCH(WV_)                                                     \
+  hipLaunchKernelGGL((gemm_f32_kernel<WV_, false, true>), grid, dim3(64 * WV_), \
+                     0, s, A, W, (const float*)nullptr, C, M, K, N, lda,        \
+                     epilogue, tls_gate, (const float*)nullptr, 0.f, glu_limit, \
+                     glu_alpha)
+  if (K >= 128) T5D_F32_LAUNCH(16);
+  else T5D_F32_LAUNCH(4);
 #undef T5D_F32_LAUNCH
 }
 
@@ -1104,7 +1119,6 @@ extern "C" int t5d_gemm(void* stream, int dtype, int w_dtype, int out_dtype,
                           : nullptr;
     g.C = (char*)C + (size_t)m0 * n_out * out_elem;
     g.M = mc; g.K = K; g.N = N;
-    g.dense_rows();
     g.m_parts = 1;
     g.gate = tls_gate;
     g.epilogue = epilogue;
@@ -1132,26 +1146,26 @@ extern "C" int t5d_dense(void* stream, int dtype, int out_dtype, const void* A,
               "t5d_dense: M=%d K=%d N=%d lda=%d", M, K, N, lda);
   T5D_REQUIRE(epilogue == T5D_EPI_NONE || epilogue == T5D_EPI_CLAMPED_GLU,
               T5D_EINVAL, "t5d_dense: epilogue %d", epilogue);
-  const bool gated = is_gated(epilogue);
-  T5D_REQUIRE(gated ? N % 2 == 0 && ldc == N / 2 && n_store == N
+  const bool glu = epilogue == T5D_EPI_CLAMPED_GLU;
+  T5D_REQUIRE(glu ? N % 2 == 0 && ldc == N / 2 && n_store == N
                     : n_store > 0 && n_store <= N && ldc >= n_store,
               T5D_EINVAL, "t5d_dense: N=%d ldc=%d n_store=%d epilogue %d", N, ldc,
               n_store, epilogue);
   hipStream_t s = as_stream(stream);
   if (dtype == T5D_F32) {
-    T5D_REQUIRE(out_dtype == T5D_F32 && n_store == N && (gated || ldc == N),
+    T5D_REQUIRE(out_dtype == T5D_F32 && n_store == N && (glu || ldc == N),
                 T5D_EINVAL,
                 "t5d_dense: float32 writes dense float32 rows (N=%d ldc=%d)", N,
                 ldc);
-    launch_gemm_f32(s, (const float*)A, (const float*)W, nullptr, (float*)C, M, K,
-                    N, epilogue, nullptr, 0.f, lda, glu_limit, glu_alpha);
+    launch_dense_f32(s, (const float*)A, lda, (const float*)W, (float*)C, M, K, N,
+                     epilogue, glu_limit, glu_alpha);
     T5D_CHECK_LAUNCH("t5d_dense(f32)");
     return T5D_OK;
   }
   T5D_REQUIRE(dtype == T5D_BF16, T5D_EINVAL, "t5d_dense: dtype %d", dtype);
   T5D_REQUIRE(out_dtype == T5D_F32
-                  ? !gated
-                  : out_dtype == T5D_BF16 && (gated || (ldc == N && n_store == N)),
+                  ? !glu
+                  : out_dtype == T5D_BF16 && (glu || (ldc == N && n_store == N)),
               T5D_EINVAL,
               "t5d_dense: out_dtype %d with epilogue %d, N=%d ldc=%d n_store=%d",
               out_dtype, epilogue, N, ldc, n_store);
@@ -1164,14 +1178,14 @@ extern "C" int t5d_dense(void* stream, int dtype, int out_dtype, const void* A,
                              M, K, N, epilogue, glu_limit, glu_alpha);
   GemmPlan p;
   if (!plan_big(M, K, N, 2, &p)) p = plan_gemm(M, K, N, 2);
-  GemmArgs g;
+  DenseArgs g;
   g.A = (const bf16_t*)A; g.W = W; g.scales = nullptr; g.residual = nullptr;
   g.C = C; g.M = M; g.K = K; g.N = N; g.m_parts = 1;
   g.gate = tls_gate; g.epilogue = epilogue; g.out_f32 = out_dtype == T5D_F32;
   g.norm_scale = nullptr; g.eps = 0.f;
   g.lda = lda; g.ldc = ldc; g.n_store = n_store;
   g.glu_limit = glu_limit; g.glu_alpha = glu_alpha;
-  if (p.big) launch_gemm_big(T5D_BF16, p, g, nullptr, s);
+  if (p.big) launch_dense_big(p, g, s);
   else launch_mfma<bf16_t>(p, g, s);
   T5D_CHECK_LAUNCH("t5d_dense");
   return T5D_OK;
@@ -1232,7 +1246,6 @@ extern "C" int t5d_gemm_tiled(void* stream, int dtype, int w_dtype,
   g.scales = w_dtype == T5D_I8 ? scales : nullptr;
   g.residual = residual; g.C = C;
   g.M = M; g.K = K; g.N = N; g.m_parts = p.m_parts;
-  g.dense_rows();
   g.gate = tls_gate; g.epilogue = epilogue;
   g.out_f32 = out_dtype == T5D_F32;
   g.norm_scale = nullptr; g.eps = 0.f;
@@ -1314,7 +1327,6 @@ extern "C" int t5d_norm_gemm(void* stream, int dtype, int w_dtype,
   g.scales = w_dtype == T5D_I8 ? scales : nullptr;
   g.residual = nullptr;
   g.C = C; g.M = M; g.K = K; g.N = N;
-  g.dense_rows();
   g.m_parts = (M + 15) / 16;
   g.gate = tls_gate;
   g.epilogue = epilogue;

@@ -24,9 +24,9 @@ namespace t5d {
 // epilogue, to partials[z][M][N]; the kernel that consumes the layer's output
 // (splitk_finish_kernel) adds the parts in ascending order.  No fences, no
 // atomics: the hand-over is the kernel boundary.
-template <int MP, int NT, typename WT, int NJ = 0>
+template <int MP, int NT, typename WT, int NJ = 0, typename Args = GemmArgs>
 __global__ void __launch_bounds__(256, 1)
-gemm_big_kernel(GemmArgs g, int k_parts, float* __restrict__ partials) {
+gemm_big_kernel(Args g, int k_parts, float* __restrict__ partials) {
   constexpr int ACC = MP * NT;
   constexpr int CH = 8;  // accumulator tiles per reduction round
   constexpr int RAW = sizeof(typename WeightTile<WT>::Raw) / 4;
@@ -101,10 +101,10 @@ gemm_big_kernel(GemmArgs g, int k_parts, float* __restrict__ partials) {
         const int row = m0 + mt * 16 + arow;
         if (NJ > 0)  // rows past the edge are never stored
           aq[slot_][h][mt] = *reinterpret_cast<const uint4*>(
-              g.A + (size_t)min(row, g.M - 1) * g.lda + (kt + h) * 32 + akoff);
+              g.A + (size_t)min(row, g.M - 1) * row_stride(g) + (kt + h) * 32 + akoff);
         else if (row < g.M && kt + h < kt_hi)
           aq[slot_][h][mt] = *reinterpret_cast<const uint4*>(
-              g.A + (size_t)row * g.lda + (kt + h) * 32 + akoff);
+              g.A + (size_t)row * row_stride(g) + (kt + h) * 32 + akoff);
         else
           aq[slot_][h][mt] = make_uint4(0, 0, 0, 0);
       }
@@ -187,7 +187,7 @@ gemm_big_kernel(GemmArgs g, int k_parts, float* __restrict__ partials) {
 
   // Cross-wavefront sums, CH tiles per round: (w0 + w2) + (w1 + w3).  Thread
   // (ml, nl) = (tid / 16, tid % 16) finishes element (ml, nl) of every tile.
-  const bool geglu = is_gated(g.epilogue);
+  const bool geglu = gated(g);
   const int ml = threadIdx.x >> 4, nl = threadIdx.x & 15;
   const int rl = ((ml >> 2) << 4) + nl, ri = ml & 3;
 #pragma unroll
@@ -205,7 +205,7 @@ gemm_big_kernel(GemmArgs g, int k_parts, float* __restrict__ partials) {
       if (t0 + q >= ACC) continue;
       const int mt = (t0 + q) / NT, nn = (t0 + q) % NT;
       const int m = m0 + mt * 16 + ml, n = (nt0 + nn) * 16 + nl;
-      if (m >= g.M || n >= g.n_store) continue;
+      if (m >= g.M || n >= stored_columns(g)) continue;
       const int idx = q * 4 + ri;
       float v = (red[0][idx][rl] + red[2][idx][rl]) +
                 (red[1][idx][rl] + red[3][idx][rl]);
@@ -315,6 +315,19 @@ bool gemm_big_has_tile(int mp, int nt) {
   T5D_BIG_TILES(T5D_X)
 #undef T5D_X
   return false;
+}
+
+void launch_dense_big(const GemmPlan& p, DenseArgs g, hipStream_t s) {
+  g.m_parts = p.m_parts;
+  dim3 grid((p.n_groups + 7) / 8 * 8 * p.m_parts), block(256);
+#define T5D_X(MP_, NT_)                                                          \
+  if (p.mp == MP_ && p.nt == NT_) {                                              \
+    hipLaunchKernelGGL((gemm_big_kernel<MP_, NT_, bf16_t, 0, DenseArgs>), grid,  \
+                       block, 0, s, g, 1, (float*)nullptr);                      \
+    return;                                                                      \
+  }
+  T5D_BIG_TILES(T5D_X)
+#undef T5D_X
 }
 
 void launch_gemm_big(int w_dtype, const GemmPlan& p, GemmArgs g,

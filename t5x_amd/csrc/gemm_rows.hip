@@ -128,10 +128,10 @@ __device__ __forceinline__ void rows_epilogue_values(
 // follow one another through the same piece without a wait in between; the
 // empty asm statements keep the compiler from moving one lane's read above
 // another lane's write (to it they are accesses of unrelated addresses).
-// CLAMPED: the gated epilogue is T5D_EPI_CLAMPED_GLU (first column of a pair:
-// gate, second: up) instead of T5D_EPI_GEGLU.
+// DENSE: one of the epilogues of t5d_dense instead: 1 = T5D_EPI_CLAMPED_GLU (first
+// column of a pair: gate, second: up), 2 = float32 rows.
 constexpr int kRowsStageBytes = 16 * 144;
-template <int NT, bool CLAMPED>
+template <int NT, int DENSE>
 __device__ __forceinline__ void rows_epilogue_staged(
     const RowsGemmArgs& g, const f32x4_r (&acc)[kRowsMT][NT], int m0, int nt0,
     int n_tiles, int lane, char* stage) {
@@ -146,7 +146,7 @@ __device__ __forceinline__ void rows_epilogue_staged(
                  ? *reinterpret_cast<const float4*>(g.scales +
                                                     16 * (nt0 + nt) + 4 * gq)
                  : make_float4(1.f, 1.f, 1.f, 1.f);
-  if (!CLAMPED && g.C32 != nullptr) {
+  if constexpr (DENSE == 2) {
     // a lane holds 4 consecutive columns of one row: 64 bytes per row and store
 #pragma unroll
     for (int mt = 0; mt < MT; ++mt) {
@@ -171,7 +171,7 @@ __device__ __forceinline__ void rows_epilogue_staged(
     }
     return;
   }
-  if (CLAMPED || g.epilogue == T5D_EPI_GEGLU) {
+  if (DENSE == 1 || g.epilogue == T5D_EPI_GEGLU) {
     // tile columns 0..7 are wi_0, 8..15 the matching wi_1 columns: the lanes
     // with gq >= 2 hold the gates of the lanes with gq - 2.  32 output columns.
     // Two v_permlane32_swap hand every lane two (value, gate) pairs — the
@@ -194,7 +194,7 @@ __device__ __forceinline__ void rows_epilogue_staged(
             __float_as_uint(acc[mt][nt][1] * sc[nt].y), false, false);
         // [0]: the value (own in the lower half), [1]: its gate
         float h0, h1;
-        if constexpr (CLAMPED) {
+        if constexpr (DENSE == 1) {
           h0 = clamped_glu(__uint_as_float(a[0]), __uint_as_float(a[1]),
                            g.glu_limit, g.glu_alpha);
           h1 = clamped_glu(__uint_as_float(b[0]), __uint_as_float(b[1]),
@@ -271,7 +271,7 @@ __device__ __forceinline__ void rows_epilogue_staged(
 }
 
 // SWAP: weights are the MFMA A operand (C^T is formed).
-template <typename WT, bool SWAP, bool CLAMPED = false>
+template <typename WT, bool SWAP, int DENSE = 0>
 __global__ void __launch_bounds__(256, 2)
 rows_gemm_kernel(RowsGemmArgs g) {
   constexpr int TB = RowsWeightTile<WT>::kTileBytes;
@@ -374,7 +374,7 @@ rows_gemm_kernel(RowsGemmArgs g) {
   if (SWAP) {
     // (the loop ends with a barrier: every wavefront is done with the tiles)
     static_assert(sizeof(s_t[0]) >= 4 * kRowsStageBytes, "stage too small");
-    rows_epilogue_staged<NT, CLAMPED>(
+    rows_epilogue_staged<NT, DENSE>(
         g, acc, m0, nt0, n_tiles, lane,
         reinterpret_cast<char*>(&s_t[0][0][0]) + wave * kRowsStageBytes);
   } else {
@@ -414,7 +414,7 @@ typedef __attribute__((address_space(1))) const void* glb_ptr_t;
 // wavefronts of 128 x 128 (accumulators in the accumulation registers) lasts
 // 257 us: with one wavefront per SIMD nothing covers the operand reads from
 // LDS.
-template <bool SWAP, int NT, int WN, bool CLAMPED = false>
+template <bool SWAP, int NT, int WN, int DENSE = 0>
 __global__ void __launch_bounds__(128 * WN, WN == 2 ? 2 : 1)
 rows_gemm_direct_kernel(RowsGemmArgs g) {
   constexpr int MT = kRowsMT;
@@ -549,7 +549,7 @@ rows_gemm_direct_kernel(RowsGemmArgs g) {
   if (SWAP) {
     static_assert(sizeof(s_t0) >= WAVES * kRowsStageBytes, "stage too small");
     __syncthreads();  // every wavefront is done with the ring
-    rows_epilogue_staged<NT, CLAMPED>(
+    rows_epilogue_staged<NT, DENSE>(
         g, acc, m0, nt0, n_tiles, lane,
         reinterpret_cast<char*>(&s_t0[0][0]) + wave * kRowsStageBytes);
   } else {
@@ -599,19 +599,26 @@ static int launch_rows(hipStream_t s, int w_dtype, const RowsGemmArgs& g,
   const int pick = tile ? tile : t5d_gemm_rows_tile(w_dtype, g.M, g.K, g.N);
   const int wgs192 = m_blocks * ((g.N + 191) / 192),
             wgs256 = m_blocks * ((g.N + 255) / 256);
-  if (g.epilogue == T5D_EPI_CLAMPED_GLU) {  // bfloat16 weights, rows layout
-    if (g.K >= 64 && pick == 3)
-      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, 3, 4, true>),
-                         dim3((unsigned)wgs192), dim3(512), 0, s, g);
-    else if (g.K >= 64 && pick == 2)
-      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 4, true>),
-                         dim3((unsigned)wgs256), dim3(512), 0, s, g);
-    else if (g.K >= 64)
-      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2, true>), grid,
-                         block, 0, s, g);
-    else
-      hipLaunchKernelGGL((rows_gemm_kernel<bf16_t, true, true>), grid, block, 0,
-                         s, g);
+  // bfloat16 weights, rows layout
+#define T5D_ROWS_DENSE(D_)                                                    \
+  do {                                                                        \
+    if (g.K >= 64 && pick == 3)                                               \
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, 3, 4, D_>),           \
+                         dim3((unsigned)wgs192), dim3(512), 0, s, g);         \
+    else if (g.K >= 64 && pick == 2)                                          \
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 4, D_>),     \
+                         dim3((unsigned)wgs256), dim3(512), 0, s, g);         \
+    else if (g.K >= 64)                                                       \
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2, D_>),     \
+                         grid, block, 0, s, g);                               \
+    else                                                                      \
+      hipLaunchKernelGGL((rows_gemm_kernel<bf16_t, true, D_>), grid, block, 0, \
+                         s, g);                                               \
+  } while (0)
+  if (g.epilogue == T5D_EPI_CLAMPED_GLU) {
+    T5D_ROWS_DENSE(1);
+  } else if (g.C32 != nullptr) {
+    T5D_ROWS_DENSE(2);
   } else if (w_dtype == T5D_BF16 && g.K >= 64 && pick == 3) {
     dim3 wgrid((unsigned)wgs192), wblock(512);
     if (swap)
@@ -646,6 +653,7 @@ static int launch_rows(hipStream_t s, int w_dtype, const RowsGemmArgs& g,
     else
       hipLaunchKernelGGL((rows_gemm_kernel<int8_t, false>), grid, block, 0, s, g);
   }
+#undef T5D_ROWS_DENSE
   T5D_CHECK_LAUNCH("t5d_gemm_rows");
   return T5D_OK;
 }

@@ -71,44 +71,61 @@ struct GemmArgs {
   int out_f32;
   const bf16_t* norm_scale;  // norm_gemm_kernel: [K] layer-norm scale
   float eps;
-  // Row strides of A and of a C that is not gated, and how many of the N columns
-  // are stored (gemm_mfma_kernel and gemm_big_kernel; norm_gemm_kernel takes
-  // dense rows).
-  int lda, ldc, n_store;
-  float glu_limit, glu_alpha;  // T5D_EPI_CLAMPED_GLU
-  // rows of K (N) elements, every column stored
-  void dense_rows() { lda = K; ldc = N; n_store = N; glu_limit = glu_alpha = 0.f; }
 };
 
+// What t5d_dense adds: rows with a stride, the first columns only, the clamped
+// gated unit.  The kernels are instantiated once per argument type, so that the
+// plain ones carry none of it (a few instructions in the epilogue of a kernel
+// that lasts 5 us cost the decode loop 1.5 %).
+struct DenseArgs : GemmArgs {
+  int lda, ldc, n_store;       // row strides of A and of a C that is not gated
+  float glu_limit, glu_alpha;  // T5D_EPI_CLAMPED_GLU
+};
+__device__ __forceinline__ int row_stride(const GemmArgs& g) { return g.K; }
+__device__ __forceinline__ int row_stride(const DenseArgs& g) { return g.lda; }
+__device__ __forceinline__ int stored_columns(const GemmArgs& g) { return g.N; }
+__device__ __forceinline__ int stored_columns(const DenseArgs& g) {
+  return g.n_store;
+}
 // Epilogues that pair two weight columns into one output column.
-__host__ __device__ __forceinline__ bool is_gated(int epilogue) {
-  return epilogue == T5D_EPI_GEGLU || epilogue == T5D_EPI_CLAMPED_GLU;
+__device__ __forceinline__ bool gated(const GemmArgs& g) {
+  return g.epilogue == T5D_EPI_GEGLU;
+}
+__device__ __forceinline__ bool gated(const DenseArgs& g) {
+  return g.epilogue == T5D_EPI_CLAMPED_GLU;
 }
 
 // Apply scale + epilogue to one finished column (pair) of row m; `res` is the
 // residual element (fetched early by the caller).
 __device__ __forceinline__ void store_result(const GemmArgs& g, int m, int n,
                                              float v, float v_gate, float res) {
-  if (is_gated(g.epilogue)) {
+  if (g.epilogue == T5D_EPI_GEGLU) {
     const int f = (n >> 4) * 8 + (n & 7);
     const int F = g.N >> 1;
-    if (g.epilogue == T5D_EPI_CLAMPED_GLU) {
-      reinterpret_cast<bf16_t*>(g.C)[(size_t)m * F + f] =
-          f32_to_bf16(clamped_glu(v, v_gate, g.glu_limit, g.glu_alpha));
-      return;
-    }
     float a0 = round_bf16(v), a1 = round_bf16(v_gate);
     float h = round_bf16(round_bf16(gelu_sigmoid_form(a0)) * a1);
     reinterpret_cast<bf16_t*>(g.C)[(size_t)m * F + f] = f32_to_bf16(h);
     return;
   }
-  const size_t o = (size_t)m * g.ldc + n;
+  const size_t o = (size_t)m * g.N + n;
   if (g.out_f32) {
     reinterpret_cast<float*>(g.C)[o] = v;
     return;
   }
   if (g.epilogue == T5D_EPI_RESIDUAL) v = round_bf16(v) + res;
   reinterpret_cast<bf16_t*>(g.C)[o] = f32_to_bf16(v);
+}
+__device__ __forceinline__ void store_result(const DenseArgs& g, int m, int n,
+                                             float v, float v_gate, float) {
+  if (gated(g)) {
+    const int f = (n >> 4) * 8 + (n & 7);
+    reinterpret_cast<bf16_t*>(g.C)[(size_t)m * (g.N >> 1) + f] =
+        f32_to_bf16(clamped_glu(v, v_gate, g.glu_limit, g.glu_alpha));
+    return;
+  }
+  const size_t o = (size_t)m * g.ldc + n;
+  if (g.out_f32) reinterpret_cast<float*>(g.C)[o] = v;
+  else reinterpret_cast<bf16_t*>(g.C)[o] = f32_to_bf16(v);
 }
 
 
@@ -122,6 +139,8 @@ struct GemmPlan {
 // the plan's k_parts parts go there, [k_parts][M][N], nothing else is written.
 void launch_gemm_big(int w_dtype, const GemmPlan& p, GemmArgs g,
                      float* partials, hipStream_t s);
+// The same for t5d_dense (bfloat16 weights, K not split).
+void launch_dense_big(const GemmPlan& p, DenseArgs g, hipStream_t s);
 bool gemm_big_has_tile(int mp, int nt);
 // Sum of split-K parts + scale + residual -> out, optional RMS norm -> normed.
 int launch_splitk_finish(hipStream_t s, const float* partials, int k_parts,
