@@ -698,6 +698,24 @@ def test_greedy_generation_equals_the_oracle(name):
   assert list(model.generate(params, prompts[:2], 12, batch_size=2)) == want[:2]
 
 
+def test_the_host_loop_over_a_dataset():
+  """get_infer_fn pads the last batch, keeps several decoding, restores order."""
+  from t5x_amd import infer
+  cfg, params, model = model_for('all')
+  rs = np.random.RandomState(13)
+  L, n = 16, [4, 7, 1, 9, 2]
+  tokens = rs.randint(1, cfg['vocab'], (5, L)).astype(np.int32)
+  mask = (np.arange(L)[None, :] < np.array(n)[:, None]).astype(np.int32)
+  ds = [(i, {'decoder_input_tokens': tokens[i],
+             'decoder_causal_attention': mask[i]}) for i in range(5)]
+  out = infer.get_infer_fn(model.predict_batch, batch_size=2)(ds, params)
+  assert [i for i, _ in out] == list(range(5))
+  for i, row in out:
+    want = tokens[i, 1:n[i]].tolist() + greedy(cfg, params, tokens[i, :n[i]],
+                                               L - n[i])
+    assert row[:L - 1] == want
+
+
 def test_generation_stops_at_the_end_token():
   cfg, params, model = model_for('all')
   prompt = [3, 1, 4, 1, 5]
