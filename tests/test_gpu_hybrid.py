@@ -623,7 +623,7 @@ def test_small_rings_wrap_in_long_requests(name, dtype):
   cfg, params, module = build(name, dtype, max_portion=5)
   rs = np.random.RandomState(7)
   live = sequences.Sequences(module, params, 1, 700)
-  for n, cuts in ((700, [300, 302, 304]), (31, [30]), (260, [250, 255])):
+  for n, cuts in ((700, [300, 302, 304]), (31, [30]), (260, range(60, 260))):
     tokens = rs.randint(0, cfg['vocab'], n).tolist()
     want = oracle.forward(cfg, params, tokens)
     assert close(feed(live, n, tokens, cuts), want, dtype), n
