@@ -619,18 +619,99 @@ typedef struct {
   const int32_t* seq_off;    /* [S + 1] first token of each portion */
   const int32_t* seq_start;  /* [S] position of that token */
   const int32_t* seq_slot;   /* [S] cache / state slot; slots are distinct */
+  const struct t5d_span* spans;  /* HOST array [n_spans], may be NULL */
+  int n_spans;
 } t5d_ragged;
+
+/* The positions that the queries of a call can see through a window, as
+ * consecutive rows: row off[s] + i is position first[s] + i of portion s, from a
+ * multiple of 64 at or before the first position that its first query sees to a
+ * multiple of 64 at or past its end.  What latent attention expands into keys and
+ * values; a call without the span of a layer's window leaves the latents as they
+ * are. */
+typedef struct t5d_span {
+  int window, rows;          /* rows = off[S] */
+  const int32_t *off, *first;  /* [S + 1], [S], on the device */
+} t5d_span;
 
 /* Bias-free dense layer over any number of rows.  dtype bfloat16: A [M, K] with
  * rows lda apart, W packed (t5d_pack_weight; K % 32, N % 16), out_dtype bfloat16
  * (dense rows of N) or float32 (the first n_store columns, rows ldc apart);
  * float32: W row-major [K, N], dense float32 rows.  epilogue NONE or CLAMPED_GLU
  * (W a geglu-packed gate | up pair, N both, C [M, N / 2], ldc = N / 2,
- * n_store = N).  Up to 128 rows run on the kernels of t5d_gemm, more on those of
+ * n_store = N): min(gate, limit) sigmoid(alpha gate) (clamp(up, limit) + add).  Up to 128 rows run on the kernels of t5d_gemm, more on those of
  * t5d_gemm_rows. */
 int t5d_dense(void* stream, int dtype, int out_dtype, const void* A, int lda,
               const void* W, void* C, int ldc, int n_store, int M, int K, int N,
-              int epilogue, float glu_limit, float glu_alpha);
+              int epilogue, float glu_limit, float glu_alpha, float glu_add);
+
+/* Dense layers of one shape in one launch, their kernels (packed as t5d_dense
+ * takes them) w_stride bytes apart.
+ * tiles given: [n_tiles] of (group, first row, rows, 0), group -1: none.  The
+ * output rows first .. first + rows - 1, at most tile_rows, take that group's
+ * kernel; output row r comes from row rows[r] of A (rows NULL: row r).  tile_rows
+ * as t5d_grouped_tile_rows gives it; 256: C dense rows.
+ * tiles NULL: group h of `groups` takes all M rows, from column h a_step of A to
+ * column h c_step of C (no gated epilogue). */
+typedef struct {
+  int dtype, M, K, N, epilogue;
+  const void* A;
+  int lda;
+  const void* W;
+  int64_t w_stride;
+  void* C;
+  int ldc, n_store;
+  float glu_limit, glu_alpha, glu_add;
+  const int32_t *tiles, *rows;
+  int n_tiles, tile_rows, groups, a_step, c_step;
+} t5d_grouped_dense;
+int t5d_grouped_tile_rows(int dtype, int entries, int groups);
+int t5d_grouped_dense_run(void* stream, const t5d_grouped_dense* a);
+
+/* Tokens sorted by expert, the experts of a token listed by its id. */
+typedef struct {
+  int experts, top, tile_rows, max_tiles;
+  const int32_t* table;      /* [V, top], entries of a row distinct */
+  int32_t* tiles;            /* [max_tiles, 4] for t5d_grouped_dense */
+  int32_t* token_of;         /* [M * top] token of each sorted entry */
+  int32_t* entry_of;         /* [M, top] sorted entry of each token's experts */
+} t5d_route;
+int t5d_route_max_tiles(int entries, int experts, int tile_rows);
+/* One launch for up to 16 layers (HOST array). */
+int t5d_route_tokens(void* stream, const int32_t* tokens, int M, int V,
+                     const t5d_route* layers, int n_layers);
+
+/* out[m, s] = scale * table[ids[m]] for every stream s, float32 [M, streams, ld];
+ * columns d .. ld - 1 zero. */
+int t5d_embed_streams(void* stream, int dtype, const void* table,
+                      const int32_t* ids, float scale, float* out, int M, int d,
+                      int ld, int streams, int V);
+
+/* The row kernel between two dense layers when a token has several float32
+ * residual streams x [M, streams, ld] (hyper-connections):
+ *   b = y_gate[m] y[m] + part_weight sum_t parts[part_row[m, t]]   (any NULL: no)
+ *   x[t] = sum_s mix[s, t] x[s] + spread[t] b      (neither y nor parts: x stays)
+ *   u = sum_s collect[s] x[s];  sum[m] = u;  out[m] = rms(u) * norm as dtype;
+ *   gate_out[m] = sigmoid(gate_w . (rms(u) * norm))
+ * mix NULL: the identity; spread, collect NULL: ones.  rows (no y, no parts): row m
+ * of the outputs comes from x row rows[m].  At most 16 streams; ld a multiple of 8,
+ * at most 16384. */
+typedef struct {
+  int dtype, d, ld, streams, top;
+  float eps, part_weight;
+  const void *y, *parts;     /* [M, ld], [., ld] of dtype */
+  const float* y_gate;       /* [M] */
+  const int32_t* part_row;   /* [M, top] */
+  const float *mix, *spread, *collect;
+  float* x;
+  const float* norm;         /* [d] */
+  void* out;                 /* [M, ld] or NULL */
+  const int32_t* rows;
+  float* sum;                /* [M, ld] or NULL */
+  const float* gate_w;       /* [d] or NULL */
+  float* gate_out;           /* [M] */
+} t5d_hyper_norm;
+int t5d_hyper_norm_run(void* stream, const t5d_hyper_norm* a, int M);
 
 /* out[m] = table[ids[m]] + sinusoid(positions[m]), float32: entry 2i is
  * sin(p 10000^(-2i/d)), entry 2i + 1 its cosine.  table [V, ld] of dtype, columns
@@ -680,6 +761,41 @@ int64_t t5d_window_workspace_bytes(int S, int H, int D, int Dv);
 int t5d_window_attention_run(void* stream, const t5d_window_attention* a,
                              const t5d_ragged* b, int variant);
 
+/* Causal attention over a window with keys and values of H heads that are linear
+ * maps of one cached latent per position, and queries through a latent of their
+ * own (see latent_attention.hip).  HP = t5d_window_head_pad(D, Dv), RP =
+ * t5d_latent_pad(rank), QP = q_rank up to a multiple of 64; padding of weights and
+ * norms is zero. */
+typedef struct {
+  int dtype, H, D, Dv, rank, q_rank;
+  int ring, window;
+  float scale, eps;
+  const void* proj;          /* [M, ld_proj]: inputs of the two latents at */
+  int ld_proj, off_q, off_kv;  /* these columns; off_kv -1: no new latents, the
+                                  ring is another layer's */
+  const float *q_norm, *kv_norm;  /* [QP], [RP] */
+  const float* sink;         /* [H] or NULL */
+  const void* uq;            /* dense [QP, H HP] */
+  const void* ukv;           /* dense [RP, 2 H HP]: keys | values */
+  const void* absorb;        /* H dense [HP, RP]: key maps applied to queries */
+  const void* expand;        /* H dense [RP, Dv up to 16]: value maps */
+  void* latent_ring;         /* [slots, ring, RP]; as the rings above */
+  /* scratch: [M, QP], [M, H HP], [M, H RP] twice, [span_rows, RP],
+   * [span_rows, 2 H HP] */
+  void *cq, *q, *ql, *ol, *lat, *kv;
+  int span_rows;
+  void* out;                 /* [M, H * Dv], rows ld_out apart */
+  int ld_out;
+  void* workspace;           /* t5d_latent_workspace_bytes(rank) or NULL */
+} t5d_latent_attention;
+
+int t5d_latent_pad(int rank);
+int64_t t5d_latent_workspace_bytes(int rank);
+/* variant 0: what suits the call; 1: absorbed, tiles of rows (bfloat16); 2: over the
+ * span of batch->spans (bfloat16); 3: absorbed, a wavefront per token and head. */
+int t5d_latent_attention_run(void* stream, const t5d_latent_attention* a,
+                             const t5d_ragged* b, int variant);
+
 /* Linear recurrence with a decay per key channel (see recurrence.hip). */
 enum { T5D_DECAY_SIGMOID_POWER = 0, T5D_DECAY_EXP_SOFTPLUS = 1 };
 enum { T5D_GATE_SILU = 0, T5D_GATE_SIGMOID_LOW = 1 };
@@ -717,18 +833,46 @@ int64_t t5d_recurrence_workspace_bytes(int M, int S, int H, int G, int D, int Dv
 int t5d_recurrence_run(void* stream, const t5d_recurrence* a, const t5d_ragged* b,
                        int variant);
 
-enum { T5D_MIX_WINDOW_ATTENTION = 0, T5D_MIX_RECURRENCE = 1 };
+/* A mixture of n gated feed-forwards, top of them per token (by a table of token
+ * ids, each with weight 1 / top), and one for every token behind a sigmoid gate. */
+typedef struct {
+  int n, top, F;             /* n 0: the layer has none */
+  const void *glu, *down;    /* n kernels [ld, 2F] gate | up, n [F, ld] */
+  int64_t glu_stride, down_stride;  /* bytes */
+  float limit, alpha, add;
+  const int32_t* table;      /* [V, top] */
+  int shared_F;              /* 0: no shared one */
+  const void *shared_glu, *shared_down;
+  float shared_limit;
+  const float* shared_gate;  /* [d] */
+  /* buffers of a call: t5d_route's; [M top, F], [M top, ld], [M, shared_F], [M] */
+  int32_t *tiles, *token_of, *entry_of;
+  int max_tiles;
+  void *rows, *out, *shared_rows;
+  float* gate;
+} t5d_experts;
+
+enum {
+  T5D_MIX_WINDOW_ATTENTION = 0,
+  T5D_MIX_RECURRENCE = 1,
+  T5D_MIX_LATENT_ATTENTION = 2
+};
 typedef struct {
   int mix;
   int proj_n, low_k, low_n, off_low, out_k, F;
   /* proj [ld, proj_n]; low (or NULL) [low_k, low_n] applied to proj columns
    * off_low ..; out [out_k, ld]; glu (or NULL) [ld, 2F] gate | up; down [F, ld] */
   const void *proj, *low, *out, *glu, *down;
-  float glu_limit, glu_alpha;
-  const float *norm1, *norm1b, *norm2, *norm2b;  /* [d] */
+  float glu_limit, glu_alpha, glu_add;
+  const float *norm1, *norm1b, *norm2, *norm2b;  /* [d]; b: streams 0 */
+  /* hyper-connections of the mixer and of the feed-forward: [streams],
+   * [streams, streams], [streams], or NULL */
+  const float *in1, *mix1, *out1, *in2, *mix2, *out2;
   void *mix_rows, *ff_rows;  /* activations [M, out_k], [M, F]; padding zero */
   t5d_window_attention attention;  /* sizes and constants; the buffers of a */
   t5d_recurrence recurrence;       /* call are filled in by the step */
+  t5d_latent_attention latent;
+  t5d_experts experts;
 } t5d_hybrid_layer;
 
 /* One pass of one layer: looped layers have one entry per pass, each with its own
@@ -736,12 +880,17 @@ typedef struct {
 typedef struct {
   int layer, enter;
   const float* enter_add;
-  void *cache0, *cache1;   /* key / value ring, or state / convolution ring */
+  void *cache0, *cache1;   /* key / value ring, state / convolution ring, or
+                              latent ring and nothing */
 } t5d_hybrid_run;
 
 typedef struct {
   int dtype, d, ld, V, head_n, n_layers, n_runs;
-  float eps;
+  /* 0: one residual stream, embedding + sinusoid, a norm before and after every
+   * branch.  > 0: that many streams x [M, streams, ld], scaled embedding, a norm
+   * before every branch (t5d_hyper_norm) */
+  int streams;
+  float eps, embed_scale;
   const void *embedding;   /* [V, ld] */
   const void *loop_in;     /* [2 ld, ld] or NULL */
   const void *head;        /* [ld, head_n] */

@@ -14,7 +14,7 @@ F32, BF16, I8 = 0, 1, 2
 EPI_NONE, EPI_RESIDUAL, EPI_GEGLU, EPI_CLAMPED_GLU = 0, 1, 2, 3
 DECAY_SIGMOID_POWER, DECAY_EXP_SOFTPLUS = 0, 1
 GATE_SILU, GATE_SIGMOID_LOW = 0, 1
-MIX_WINDOW_ATTENTION, MIX_RECURRENCE = 0, 1
+MIX_WINDOW_ATTENTION, MIX_RECURRENCE, MIX_LATENT_ATTENTION = 0, 1, 2
 OUT_ROWS, OUT_HEADS_KEY, OUT_HEADS_VALUE = 0, 1, 2
 LEAVE_OUT_CROSS_ATTENTION, LEAVE_OUT_SELF_ATTENTION = 1, 2
 
@@ -88,7 +88,7 @@ def _fields(**groups):
 class Ragged(Structure):
   """t5d_ragged."""
   _fields_ = _fields(i='M S max_len', p='tokens tok_pos tok_seq seq_off '
-                     'seq_start seq_slot')
+                     'seq_start seq_slot spans', i2='n_spans')
 
 
 class WindowAttention(Structure):
@@ -97,6 +97,50 @@ class WindowAttention(Structure):
                      i2='ld_proj off_q off_k off_v',
                      p2='q_norm k_norm slopes sink key_ring value_ring q_rows '
                      'out', i3='ld_out', p3='workspace')
+
+
+class Span(Structure):
+  """t5d_span."""
+  _fields_ = _fields(i='window rows', p='off first')
+
+
+class GroupedDense(Structure):
+  """t5d_grouped_dense."""
+  _fields_ = _fields(i='dtype M K N epilogue', p='A', i2='lda', p2='W',
+                     l='w_stride', p3='C', i3='ldc n_store',
+                     f='glu_limit glu_alpha glu_add', p4='tiles rows',
+                     i4='n_tiles tile_rows groups a_step c_step')
+
+
+class Route(Structure):
+  """t5d_route."""
+  _fields_ = _fields(i='experts top tile_rows max_tiles',
+                     p='table tiles token_of entry_of')
+
+
+class HyperNorm(Structure):
+  """t5d_hyper_norm."""
+  _fields_ = _fields(i='dtype d ld streams top', f='eps part_weight',
+                     p='y parts y_gate part_row mix spread collect x norm out '
+                     'rows sum gate_w gate_out')
+
+
+class LatentAttention(Structure):
+  """t5d_latent_attention."""
+  _fields_ = _fields(i='dtype H D Dv rank q_rank ring window', f='scale eps',
+                     p='proj', i2='ld_proj off_q off_kv',
+                     p2='q_norm kv_norm sink uq ukv absorb expand latent_ring cq '
+                     'q ql ol lat kv', i3='span_rows', p3='out', i4='ld_out',
+                     p4='workspace')
+
+
+class Experts(Structure):
+  """t5d_experts."""
+  _fields_ = _fields(i='n top F', p='glu down', l='glu_stride down_stride',
+                     f='limit alpha add', p2='table', i2='shared_F',
+                     p3='shared_glu shared_down', f2='shared_limit',
+                     p4='shared_gate tiles token_of entry_of', i3='max_tiles',
+                     p5='rows out shared_rows gate')
 
 
 class Recurrence(Structure):
@@ -112,10 +156,12 @@ class Recurrence(Structure):
 class HybridLayer(Structure):
   """t5d_hybrid_layer."""
   _fields_ = _fields(i='mix proj_n low_k low_n off_low out_k F',
-                     p='proj low out glu down', f='glu_limit glu_alpha',
-                     p2='norm1 norm1b norm2 norm2b mix_rows ff_rows') + [
+                     p='proj low out glu down', f='glu_limit glu_alpha glu_add',
+                     p2='norm1 norm1b norm2 norm2b in1 mix1 out1 in2 mix2 out2 '
+                     'mix_rows ff_rows') + [
                          ('attention', WindowAttention),
-                         ('recurrence', Recurrence)]
+                         ('recurrence', Recurrence),
+                         ('latent', LatentAttention), ('experts', Experts)]
 
 
 class HybridRun(Structure):
@@ -125,7 +171,8 @@ class HybridRun(Structure):
 
 class HybridModel(Structure):
   """t5d_hybrid_model."""
-  _fields_ = (_fields(i='dtype d ld V head_n n_layers n_runs', f='eps',
+  _fields_ = (_fields(i='dtype d ld V head_n n_layers n_runs streams',
+                      f='eps embed_scale',
                       p='embedding loop_in head final_norm') +
               [('layers', POINTER(HybridLayer)), ('runs', POINTER(HybridRun))] +
               _fields(p='x x0 low h cat proj q_rows y workspace',
@@ -141,7 +188,18 @@ _SIGNATURES = {
     't5d_temperature_sample_step': (c_int, [_P, POINTER(ModelStep),
                                             POINTER(SampleStep)]),
     't5d_dense': (c_int, [_P, c_int, c_int, _P, c_int, _P, _P] + [c_int] * 6 +
-                  [c_float] * 2),
+                  [c_float] * 3),
+    't5d_grouped_tile_rows': (c_int, [c_int] * 3),
+    't5d_grouped_dense_run': (c_int, [_P, POINTER(GroupedDense)]),
+    't5d_route_max_tiles': (c_int, [c_int] * 3),
+    't5d_route_tokens': (c_int, [_P, _P, c_int, c_int, POINTER(Route), c_int]),
+    't5d_embed_streams': (c_int, [_P, c_int, _P, _P, c_float, _P] +
+                          [c_int] * 5),
+    't5d_hyper_norm_run': (c_int, [_P, POINTER(HyperNorm), c_int]),
+    't5d_latent_pad': (c_int, [c_int]),
+    't5d_latent_workspace_bytes': (c_int64, [c_int]),
+    't5d_latent_attention_run': (c_int, [_P, POINTER(LatentAttention),
+                                         POINTER(Ragged), c_int]),
     't5d_embed_sinusoid': (c_int, [_P, c_int] + [_P] * 5 + [c_int] * 4),
     't5d_stream_norm': (c_int, [_P, c_int, c_int] + [_P] * 8 + [c_int] * 3 +
                         [c_float]),

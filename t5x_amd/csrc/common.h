@@ -240,12 +240,13 @@ __device__ __forceinline__ float gelu_sigmoid_form(float x) {
 }
 
 // Gated unit with both branches clamped: g = min(gate, limit),
-// u = clamp(up, -limit, limit) -> g * sigmoid(alpha g) * (u + 1).
+// u = clamp(up, -limit, limit) -> g * sigmoid(alpha g) * (u + add).  An infinite
+// limit with alpha 1 and add 0 is silu(gate) * up.
 __device__ __forceinline__ float clamped_glu(float gate, float up, float limit,
-                                             float alpha) {
+                                             float alpha, float add) {
   const float g = fminf(gate, limit);
   const float u = fminf(fmaxf(up, -limit), limit);
-  return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+  return g / (1.0f + expf(-alpha * g)) * (u + add);
 }
 
 inline hipStream_t as_stream(void* s) { return reinterpret_cast<hipStream_t>(s); }
@@ -274,7 +275,15 @@ bool norm_gemm_is_wide(int w_dtype, int K, int N);
 // The many-row kernels behind t5d_dense (bfloat16, M of any size).
 int launch_dense_rows(hipStream_t s, const void* A, int lda, const void* W,
                       void* C, int out_f32, int ldc, int n_store, int M, int K,
-                      int N, int epilogue, float glu_limit, float glu_alpha);
+                      int N, int epilogue, float glu_limit, float glu_alpha,
+                      float glu_add);
+// Windowed attention (window_attention.hip) whose queries are already in q_rows:
+// over keys and values expanded into the rows of a span (bfloat16, heads up to
+// 256), and one wavefront per (token, head) over rings of rows of HP elements.
+int launch_window_span(hipStream_t s, const t5d_window_attention& a,
+                       const t5d_ragged& b, const t5d_span& span, int ld_kv);
+int launch_window_wave(hipStream_t s, const t5d_window_attention& a,
+                       const t5d_ragged& b, int HP);
 // Embedding rows of the current tokens, read straight from the sequences:
 // ids[r] = seqs[r, *cur_index] (t5d_gather_step_ids + t5d_embed in one kernel).
 int launch_embed_from_seqs(hipStream_t s, int dtype, const void* table,

@@ -41,6 +41,15 @@ gemm_mfma_kernel(Args g) {
   // suffices; large tiles: two buffers and a tree (LDS budget).
   constexpr bool FLAT = ACC <= 4;
   __shared__ float red[FLAT ? 4 : 2][ACC * 4][64];
+  if constexpr (IsGrouped<Args>::value) {
+    T5D_GATED(g.gate);
+    const char* w = reinterpret_cast<const char*>(g.W);
+    bf16_t* c = reinterpret_cast<bf16_t*>(g.C);
+    if (!enter_group(g.grp, g.A, g.lda, w, c, gated(g) ? g.N >> 1 : g.ldc, g.M))
+      return;
+    g.W = w;
+    g.C = c;
+  }
   T5D_GATE_READ(g.gate);
 
   // XCD-aware block mapping: the m_parts workgroups of one column group get
@@ -100,12 +109,27 @@ gemm_mfma_kernel(Args g) {
                          : (APF_CAP > 2 && PF % (APF_CAP - 2) == 0 ? APF_CAP - 2 : 1));
   static_assert(PF % APF == 0, "activation ring out of phase with the weight ring");
   uint4 aq[APF][2][MP];
+  int a_row[MP];  // grouped: which row of A
+  if constexpr (IsGrouped<Args>::value) {
+#pragma unroll
+    for (int mt = 0; mt < MP; ++mt)
+      a_row[mt] = group_row(g.grp, min(m0 + mt * 16 + arow, g.M - 1));
+  }
   auto load_a = [&](int slot_, int j) {
     const int kt = (wave + 4 * j) * 2;
 #pragma unroll
     for (int h = 0; h < 2; ++h)
 #pragma unroll
       for (int mt = 0; mt < MP; ++mt) {
+        if constexpr (IsGrouped<Args>::value) {
+          static_assert(NJ == 0, "grouped layers have no unrolled K loop");
+          // (rows past the edge are never stored)
+          aq[slot_][h][mt] =
+              kt + h < KT ? *reinterpret_cast<const uint4*>(
+                                g.A + (size_t)a_row[mt] * g.lda + (kt + h) * 32 + akoff)
+                          : make_uint4(0, 0, 0, 0);
+          continue;
+        }
         const int row = m0 + mt * 16 + arow;
         if (NJ > 0)  // rows past the edge are never stored
           aq[slot_][h][mt] = *reinterpret_cast<const uint4*>(
@@ -639,13 +663,20 @@ norm_gemm_wide_kernel(GemmArgs g, int G, int halves) {
 constexpr int kF32Rows = 8, kF32Cols = 16;
 
 // DENSE: what t5d_dense adds (lda, the clamped gated unit).
-template <int WV, bool NORMED, bool DENSE = false>
+// GROUPED: what t5d_grouped_dense adds (see GroupTiles), with C's row stride and
+// the columns stored.
+struct F32Group {
+  GroupTiles grp;
+  int ldc, n_store;
+};
+template <int WV, bool NORMED, bool DENSE = false, bool GROUPED = false>
 __global__ void __launch_bounds__(64 * WV)
 gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
                 const float* __restrict__ residual, float* __restrict__ C,
                 int M, int K, int N, int lda_arg, int epilogue,
                 const int32_t* gate, const float* __restrict__ norm_scale,
-                float eps, float glu_limit, float glu_alpha) {
+                float eps, float glu_limit, float glu_alpha, float glu_add,
+                F32Group gr) {
   static_assert(WV == 4 || WV == 16, "wavefronts per workgroup");
   constexpr int MB = kF32Rows;
   constexpr int RW = WV == 4 ? 4 : 8;  // partial sums held in LDS at once
@@ -660,7 +691,12 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
   const int F = N >> 1;
   const int ncols = geglu ? F : N;  // columns of work
   const int n = blockIdx.x * kF32Cols + c;
-  const int m0 = blockIdx.y * MB;
+  int m0 = blockIdx.y * MB;
+  if constexpr (GROUPED) {
+    if (!enter_group(gr.grp, A, lda, W, C, geglu ? F : gr.ldc, M)) return;
+    m0 = gr.grp.tiles != nullptr ? 0 : blockIdx.z * MB;
+  }
+  const int ldc = geglu ? F : GROUPED ? gr.ldc : N;
   const bool active = n < ncols;
   float acc0[MB], acc1[MB], ssq[MB];
 #pragma unroll
@@ -685,8 +721,8 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
         const int row = m0 + m;
         ax[m] = ay[m] = make_float4(0.f, 0.f, 0.f, 0.f);
         if (row < M) {
-          const float4* ap =
-              reinterpret_cast<const float4*>(A + (size_t)row * lda + kk);
+          const float4* ap = reinterpret_cast<const float4*>(
+              A + (size_t)(GROUPED ? group_row(gr.grp, row) : row) * lda + kk);
           ax[m] = ap[0];
           ay[m] = ap[1];
         }
@@ -724,7 +760,9 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
 #pragma unroll
     for (int m = 0; m < MB; ++m) {
       const int row = m0 + m;
-      const float a = row < M ? A[(size_t)row * lda + k] : 0.f;
+      const float a =
+          row < M ? A[(size_t)(GROUPED ? group_row(gr.grp, row) : row) * lda + k]
+                  : 0.f;
       if constexpr (normed) ssq[m] = fmaf(a, a, ssq[m]);
       acc0[m] = fmaf(a, w0, acc0[m]);
       acc1[m] = fmaf(a, w1, acc1[m]);
@@ -777,6 +815,7 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
     const int col = blockIdx.x * kF32Cols + l;
     const int row = m0 + m;
     if (row >= M || col >= ncols) continue;
+    if (GROUPED && !geglu && col >= gr.n_store) continue;
     float v = total(m, l);
     // every lane subrange saw its own k of the row: the total is the row's
     const float inv =
@@ -784,11 +823,12 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
     v *= inv;
     if (geglu) {
       float vg = total(MB + m, l) * inv;
-      C[(size_t)row * F + col] =
-          DENSE ? clamped_glu(v, vg, glu_limit, glu_alpha) : gelu_tanh(v) * vg;
+      C[(size_t)row * ldc + col] =
+          DENSE ? clamped_glu(v, vg, glu_limit, glu_alpha, glu_add)
+                : gelu_tanh(v) * vg;
     } else {
       if (epilogue == T5D_EPI_RESIDUAL) v += residual[(size_t)row * N + col];
-      C[(size_t)row * N + col] = v;
+      C[(size_t)row * ldc + col] = v;
     }
   }
 }
@@ -999,7 +1039,7 @@ static void launch_gemm_f32(hipStream_t s, const float* A, const float* W,
 #define T5D_F32_LAUNCH(WV_, NORMED_)                                          \
   hipLaunchKernelGGL((gemm_f32_kernel<WV_, NORMED_>), grid, dim3(64 * WV_), 0, \
                      s, A, W, residual, C, M, K, N, K, epilogue, tls_gate,    \
-                     norm_scale, eps, 0.f, 0.f)
+                     norm_scale, eps, 0.f, 0.f, 0.f, F32Group())
   if (K >= 128) {
     if (norm_scale) T5D_F32_LAUNCH(16, true);
     else T5D_F32_LAUNCH(16, false);
@@ -1012,14 +1052,14 @@ static void launch_gemm_f32(hipStream_t s, const float* A, const float* W,
 
 static void launch_dense_f32(hipStream_t s, const float* A, int lda, const float* W,
                              float* C, int M, int K, int N, int epilogue,
-                             float glu_limit, float glu_alpha) {
+                             float glu_limit, float glu_alpha, float glu_add) {
   const int ncols = epilogue == T5D_EPI_CLAMPED_GLU ? N / 2 : N;
   dim3 grid((ncols + kF32Cols - 1) / kF32Cols, (M + kF32Rows - 1) / kF32Rows);
 #define T5D_F32_LAUNCH(WV_)                                                     \
   hipLaunchKernelGGL((gemm_f32_kernel<WV_, false, true>), grid, dim3(64 * WV_), \
                      0, s, A, W, (const float*)nullptr, C, M, K, N, lda,        \
                      epilogue, tls_gate, (const float*)nullptr, 0.f, glu_limit, \
-                     glu_alpha)
+                     glu_alpha, glu_add, F32Group())
   if (K >= 128) T5D_F32_LAUNCH(16);
   else T5D_F32_LAUNCH(4);
 #undef T5D_F32_LAUNCH
@@ -1140,7 +1180,7 @@ extern "C" int t5d_gemm(void* stream, int dtype, int w_dtype, int out_dtype,
 extern "C" int t5d_dense(void* stream, int dtype, int out_dtype, const void* A,
                          int lda, const void* W, void* C, int ldc, int n_store,
                          int M, int K, int N, int epilogue, float glu_limit,
-                         float glu_alpha) {
+                         float glu_alpha, float glu_add) {
   T5D_REQUIRE(A && W && C, T5D_EINVAL, "t5d_dense: null pointer");
   T5D_REQUIRE(M > 0 && M < (1 << 28) && K > 0 && N > 0 && lda >= K, T5D_EINVAL,
               "t5d_dense: M=%d K=%d N=%d lda=%d", M, K, N, lda);
@@ -1158,7 +1198,7 @@ extern "C" int t5d_dense(void* stream, int dtype, int out_dtype, const void* A,
                 "t5d_dense: float32 writes dense float32 rows (N=%d ldc=%d)", N,
                 ldc);
     launch_dense_f32(s, (const float*)A, lda, (const float*)W, (float*)C, M, K, N,
-                     epilogue, glu_limit, glu_alpha);
+                     epilogue, glu_limit, glu_alpha, glu_add);
     T5D_CHECK_LAUNCH("t5d_dense(f32)");
     return T5D_OK;
   }
@@ -1175,7 +1215,7 @@ extern "C" int t5d_dense(void* stream, int dtype, int out_dtype, const void* A,
               "t5d_dense: operands must be 16-byte aligned");
   if (M > kMaxRows)
     return launch_dense_rows(s, A, lda, W, C, out_dtype == T5D_F32, ldc, n_store,
-                             M, K, N, epilogue, glu_limit, glu_alpha);
+                             M, K, N, epilogue, glu_limit, glu_alpha, glu_add);
   GemmPlan p;
   if (!plan_big(M, K, N, 2, &p)) p = plan_gemm(M, K, N, 2);
   DenseArgs g;
@@ -1184,10 +1224,108 @@ extern "C" int t5d_dense(void* stream, int dtype, int out_dtype, const void* A,
   g.gate = tls_gate; g.epilogue = epilogue; g.out_f32 = out_dtype == T5D_F32;
   g.norm_scale = nullptr; g.eps = 0.f;
   g.lda = lda; g.ldc = ldc; g.n_store = n_store;
-  g.glu_limit = glu_limit; g.glu_alpha = glu_alpha;
+  g.glu_limit = glu_limit; g.glu_alpha = glu_alpha; g.glu_add = glu_add;
   if (p.big) launch_dense_big(p, g, s);
   else launch_mfma<bf16_t>(p, g, s);
   T5D_CHECK_LAUNCH("t5d_dense");
+  return T5D_OK;
+}
+
+extern "C" int t5d_grouped_tile_rows(int dtype, int entries, int groups) {
+  if (entries <= 0 || groups <= 0) return -1;
+  if (dtype == T5D_F32) return kF32Rows;
+  const int each = (entries + groups - 1) / groups;
+  return each <= 16 ? 16 : each <= 64 ? 64 : 256;
+}
+
+extern "C" int t5d_grouped_dense_run(void* stream, const t5d_grouped_dense* a) {
+  T5D_REQUIRE(a && a->A && a->W && a->C, T5D_EINVAL,
+              "t5d_grouped_dense_run: null pointer");
+  T5D_REQUIRE(a->K > 0 && a->N > 0 && a->lda > 0 && a->w_stride > 0, T5D_EINVAL,
+              "t5d_grouped_dense_run: K=%d N=%d lda=%d", a->K, a->N, a->lda);
+  T5D_REQUIRE(a->epilogue == T5D_EPI_NONE || a->epilogue == T5D_EPI_CLAMPED_GLU,
+              T5D_EINVAL, "t5d_grouped_dense_run: epilogue %d", a->epilogue);
+  const bool glu = a->epilogue == T5D_EPI_CLAMPED_GLU;
+  T5D_REQUIRE(glu ? a->N % 2 == 0 : a->n_store > 0 && a->n_store <= a->N &&
+                                        a->ldc >= a->n_store,
+              T5D_EINVAL, "t5d_grouped_dense_run: N=%d ldc=%d n_store=%d", a->N,
+              a->ldc, a->n_store);
+  T5D_REQUIRE(a->tiles ? a->n_tiles > 0 && a->n_tiles <= 65535
+                       : a->groups > 0 && a->groups <= 65535 && a->M > 0 &&
+                             a->M < (1 << 28) && !glu && !a->rows,
+              T5D_EINVAL, "t5d_grouped_dense_run: tiles=%d groups=%d M=%d",
+              a->n_tiles, a->groups, a->M);
+  const int gy = a->tiles ? a->n_tiles : a->groups;
+  GroupTiles grp;
+  grp.tiles = (const int4*)a->tiles; grp.rows = a->rows;
+  grp.w_stride = a->w_stride; grp.a_step = a->a_step; grp.c_step = a->c_step;
+  hipStream_t s = as_stream(stream);
+  if (a->dtype == T5D_F32) {
+    T5D_REQUIRE(!a->tiles || a->tile_rows == kF32Rows, T5D_EINVAL,
+                "t5d_grouped_dense_run: tiles of %d rows", a->tile_rows);
+    T5D_REQUIRE(a->w_stride % 4 == 0, T5D_EINVAL,
+                "t5d_grouped_dense_run: kernels %lld bytes apart",
+                (long long)a->w_stride);
+    F32Group gr;
+    gr.grp = grp; gr.ldc = a->ldc; gr.n_store = a->n_store;
+    gr.grp.w_stride = a->w_stride / 4;
+    const int ncols = glu ? a->N / 2 : a->N;
+    const int64_t parts = a->tiles ? 1 : (a->M + kF32Rows - 1) / kF32Rows;
+    T5D_REQUIRE(parts <= 65535, T5D_ELIMIT, "t5d_grouped_dense_run: M=%d", a->M);
+    const dim3 grid((ncols + kF32Cols - 1) / kF32Cols, gy, (unsigned)parts);
+#define T5D_F32_LAUNCH(WV_)                                                      \
+  hipLaunchKernelGGL((gemm_f32_kernel<WV_, false, true, true>), grid,            \
+                     dim3(64 * WV_), 0, s, (const float*)a->A, (const float*)a->W, \
+                     (const float*)nullptr, (float*)a->C, a->M, a->K, a->N, a->lda, \
+                     a->epilogue, tls_gate, (const float*)nullptr, 0.f,          \
+                     a->glu_limit, a->glu_alpha, a->glu_add, gr)
+    if (a->K >= 128) T5D_F32_LAUNCH(16);
+    else T5D_F32_LAUNCH(4);
+#undef T5D_F32_LAUNCH
+    T5D_CHECK_LAUNCH("t5d_grouped_dense_run(f32)");
+    return T5D_OK;
+  }
+  T5D_REQUIRE(a->dtype == T5D_BF16, T5D_EINVAL, "t5d_grouped_dense_run: dtype %d",
+              a->dtype);
+  T5D_REQUIRE(a->K % 32 == 0 && a->N % 16 == 0 && a->lda % 8 == 0 &&
+                  a->a_step % 8 == 0 && a->w_stride % 16 == 0 &&
+                  (((uintptr_t)a->A | (uintptr_t)a->W | (uintptr_t)a->tiles) % 16) == 0,
+              T5D_EINVAL, "t5d_grouped_dense_run: K=%d N=%d lda=%d alignment", a->K,
+              a->N, a->lda);
+  GroupedArgs g;
+  g.A = (const bf16_t*)a->A; g.W = a->W; g.scales = nullptr; g.residual = nullptr;
+  g.C = a->C; g.M = a->M; g.K = a->K; g.N = a->N; g.m_parts = 1;
+  g.gate = tls_gate; g.epilogue = a->epilogue; g.out_f32 = 0;
+  g.norm_scale = nullptr; g.eps = 0.f;
+  g.lda = a->lda; g.ldc = a->ldc; g.n_store = glu ? a->N : a->n_store;
+  g.glu_limit = a->glu_limit; g.glu_alpha = a->glu_alpha; g.glu_add = a->glu_add;
+  g.grp = grp;
+  const int NT = 2;
+  const unsigned gx = (unsigned)((a->N / 16 + NT - 1) / NT + 7) / 8 * 8;
+  if (a->tiles && a->tile_rows == 256) {
+    T5D_REQUIRE(a->K >= 64 && (glu || (a->ldc == a->N && a->n_store == a->N)) &&
+                    ((uintptr_t)a->C % 16) == 0 && a->N % 16 == 0,
+                T5D_EINVAL, "t5d_grouped_dense_run: tiles of 256 rows with K=%d "
+                "N=%d ldc=%d", a->K, a->N, a->ldc);
+    return launch_grouped_rows(s, g, a->n_tiles);
+  }
+  if (a->tiles && a->tile_rows == 16) {
+    hipLaunchKernelGGL((gemm_mfma_kernel<1, 2, bf16_t, 0, GroupedArgs>),
+                       dim3(gx, gy), dim3(256), 0, s, g);
+  } else if (a->tiles) {
+    T5D_REQUIRE(a->tile_rows == 64, T5D_EINVAL,
+                "t5d_grouped_dense_run: tiles of %d rows", a->tile_rows);
+    hipLaunchKernelGGL((gemm_mfma_kernel<4, 2, bf16_t, 0, GroupedArgs>),
+                       dim3(gx, gy), dim3(256), 0, s, g);
+  } else if (a->M <= 16) {
+    hipLaunchKernelGGL((gemm_mfma_kernel<1, 2, bf16_t, 0, GroupedArgs>),
+                       dim3(gx, gy), dim3(256), 0, s, g);
+  } else {
+    g.m_parts = (a->M + 63) / 64;
+    hipLaunchKernelGGL((gemm_mfma_kernel<4, 2, bf16_t, 0, GroupedArgs>),
+                       dim3(gx * g.m_parts, gy), dim3(256), 0, s, g);
+  }
+  T5D_CHECK_LAUNCH("t5d_grouped_dense_run");
   return T5D_OK;
 }
 

@@ -17,6 +17,7 @@
 // consecutive ROWS of one column — whichever makes the 8-byte stores
 // contiguous in the requested output layout.
 #include "common.h"
+#include "gemm_tiles.h"
 
 namespace t5d {
 
@@ -73,7 +74,9 @@ struct RowsGemmArgs {
   int lda;                 // row stride of A
   float* C32;              // float32 output rows instead of C (rows layout, no
   int ldc, n_store;        // epilogue): row stride, columns stored of the N
-  float glu_limit, glu_alpha;  // T5D_EPI_CLAMPED_GLU
+  float glu_limit, glu_alpha, glu_add;  // T5D_EPI_CLAMPED_GLU
+  const int32_t* gate;     // GROUPED kernels only, with the next
+  GroupTiles grp;
 };
 
 __device__ __forceinline__ uint2 pack4(float a, float b, float c, float d) {
@@ -196,9 +199,9 @@ __device__ __forceinline__ void rows_epilogue_staged(
         float h0, h1;
         if constexpr (DENSE == 1) {
           h0 = clamped_glu(__uint_as_float(a[0]), __uint_as_float(a[1]),
-                           g.glu_limit, g.glu_alpha);
+                           g.glu_limit, g.glu_alpha, g.glu_add);
           h1 = clamped_glu(__uint_as_float(b[0]), __uint_as_float(b[1]),
-                           g.glu_limit, g.glu_alpha);
+                           g.glu_limit, g.glu_alpha, g.glu_add);
         } else {
           h0 = round_bf16(gelu_sigmoid_form(round_bf16(__uint_as_float(a[0])))) *
                round_bf16(__uint_as_float(a[1]));
@@ -414,7 +417,8 @@ typedef __attribute__((address_space(1))) const void* glb_ptr_t;
 // wavefronts of 128 x 128 (accumulators in the accumulation registers) lasts
 // 257 us: with one wavefront per SIMD nothing covers the operand reads from
 // LDS.
-template <bool SWAP, int NT, int WN, int DENSE = 0>
+// GROUPED: see GroupTiles (gemm_tiles.h); blockIdx.y is the tile of rows.
+template <bool SWAP, int NT, int WN, int DENSE = 0, bool GROUPED = false>
 __global__ void __launch_bounds__(128 * WN, WN == 2 ? 2 : 1)
 rows_gemm_direct_kernel(RowsGemmArgs g) {
   constexpr int MT = kRowsMT;
@@ -440,6 +444,11 @@ rows_gemm_direct_kernel(RowsGemmArgs g) {
   __shared__ uint4 s_t0[TILES][64];
   __shared__ uint4 s_t1[TILES][64];
   __shared__ uint4 s_t2[TILES][64];
+  if constexpr (GROUPED) {
+    T5D_GATED(g.gate);
+    if (!enter_group(g.grp, g.A, g.lda, g.W, g.C, DENSE == 1 ? g.N >> 1 : g.N, g.M))
+      return;
+  }
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int l16 = lane & 15, gq = lane >> 4;
@@ -459,12 +468,12 @@ rows_gemm_direct_kernel(RowsGemmArgs g) {
   const char* arow[AL];
   const char* wtile[WL];
 #pragma unroll
-  for (int i = 0; i < AL; ++i)
-    arow[i] = reinterpret_cast<const char*>(
-        g.A +
-        (size_t)min(m_blk * kRowsBM + 16 * (wave + WAVES * i) + ld_row,
-                    g.M - 1) *
-            g.lda + 8 * ld_piece);
+  for (int i = 0; i < AL; ++i) {
+    int row = min(m_blk * kRowsBM + 16 * (wave + WAVES * i) + ld_row, g.M - 1);
+    if constexpr (GROUPED) row = group_row(g.grp, row);
+    arow[i] = reinterpret_cast<const char*>(g.A + (size_t)row * g.lda +
+                                            8 * ld_piece);
+  }
 #pragma unroll
   for (int i = 0; i < WL; ++i)
     wtile[i] = g.W + (size_t)min(n_blk * (BN / 16) +
@@ -711,14 +720,16 @@ extern "C" int t5d_gemm_rows_tiled(void* stream, int w_dtype, const void* A,
   g.epilogue = epilogue; g.layout = out_layout;
   g.E = E; g.Ep = Ep; g.H = H;
   g.lda = K; g.C32 = nullptr; g.ldc = g.n_store = N;
-  g.glu_limit = g.glu_alpha = 0.f;
+  g.glu_limit = g.glu_alpha = g.glu_add = 0.f;
+  g.gate = nullptr; g.grp = GroupTiles();
   return launch_rows(as_stream(stream), w_dtype, g, tile);
 }
 
 int t5d::launch_dense_rows(hipStream_t s, const void* A, int lda,
                            const void* W, void* C, int out_f32, int ldc,
                            int n_store, int M, int K, int N, int epilogue,
-                           float glu_limit, float glu_alpha) {
+                           float glu_limit, float glu_alpha,
+                           float glu_add) {
   RowsGemmArgs g;
   g.A = (const bf16_t*)A; g.W = (const char*)W;
   g.scales = nullptr; g.residual = nullptr;
@@ -728,6 +739,29 @@ int t5d::launch_dense_rows(hipStream_t s, const void* A, int lda,
   g.epilogue = epilogue; g.layout = T5D_OUT_ROWS;
   g.E = g.Ep = g.H = 0;
   g.lda = lda; g.ldc = ldc; g.n_store = n_store;
-  g.glu_limit = glu_limit; g.glu_alpha = glu_alpha;
+  g.gate = nullptr; g.grp = GroupTiles();
+  g.glu_limit = glu_limit; g.glu_alpha = glu_alpha; g.glu_add = glu_add;
   return launch_rows(s, T5D_BF16, g, 0);
+}
+
+int t5d::launch_grouped_rows(hipStream_t s, const GroupedArgs& a, int n_tiles) {
+  RowsGemmArgs g;
+  g.A = a.A; g.W = (const char*)a.W;
+  g.scales = nullptr; g.residual = nullptr;
+  g.C = (bf16_t*)a.C; g.C32 = nullptr;
+  g.M = 0; g.K = a.K; g.N = a.N;
+  g.epilogue = a.epilogue; g.layout = T5D_OUT_ROWS;
+  g.E = g.Ep = g.H = 0;
+  g.lda = a.lda; g.ldc = a.ldc; g.n_store = a.n_store;
+  g.glu_limit = a.glu_limit; g.glu_alpha = a.glu_alpha; g.glu_add = a.glu_add;
+  g.gate = a.gate; g.grp = a.grp;
+  const dim3 grid((g.N + kRowsBN - 1) / kRowsBN, n_tiles), block(256);
+  if (g.epilogue == T5D_EPI_CLAMPED_GLU)
+    hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2, 1, true>), grid,
+                       block, 0, s, g);
+  else
+    hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2, 0, true>), grid,
+                       block, 0, s, g);
+  T5D_CHECK_LAUNCH("t5d_grouped_dense_run(rows)");
+  return T5D_OK;
 }

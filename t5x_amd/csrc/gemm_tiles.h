@@ -79,13 +79,56 @@ struct GemmArgs {
 // that lasts 5 us cost the decode loop 1.5 %).
 struct DenseArgs : GemmArgs {
   int lda, ldc, n_store;       // row strides of A and of a C that is not gated
-  float glu_limit, glu_alpha;  // T5D_EPI_CLAMPED_GLU
+  float glu_limit, glu_alpha, glu_add;  // T5D_EPI_CLAMPED_GLU
 };
 __device__ __forceinline__ int row_stride(const GemmArgs& g) { return g.K; }
 __device__ __forceinline__ int row_stride(const DenseArgs& g) { return g.lda; }
 __device__ __forceinline__ int stored_columns(const GemmArgs& g) { return g.N; }
 __device__ __forceinline__ int stored_columns(const DenseArgs& g) {
   return g.n_store;
+}
+// What t5d_grouped_dense adds: one launch over many kernels of one shape, which
+// are w_stride bytes apart.  With tiles, workgroups with blockIdx.y = t work on
+// tile t = (group, first row, rows, -): up to a workgroup's height of consecutive
+// output rows that all take that group's kernel (group -1: nothing); row r of the
+// output comes from row rows[r] of A (rows null: from row r).  Without tiles group
+// blockIdx.y takes all M rows from column group * a_step of A to column
+// group * c_step of C.
+struct GroupTiles {
+  const int4* tiles;
+  const int32_t* rows;
+  int64_t w_stride;
+  int a_step, c_step;
+};
+struct GroupedArgs : DenseArgs {
+  GroupTiles grp;
+};
+template <typename Args> struct IsGrouped { static constexpr bool value = false; };
+template <> struct IsGrouped<GroupedArgs> { static constexpr bool value = true; };
+// Points A, W, C (of elements of a_bytes, bytes, c_bytes), the row list and M at
+// this workgroup's group; false: there is nothing to do.
+template <typename AP, typename WP, typename CP>
+__device__ __forceinline__ bool enter_group(GroupTiles& grp, AP& A, int lda, WP& W,
+                                            CP& C, int ldc, int& M) {
+  if (grp.tiles != nullptr) {
+    const int4 t = grp.tiles[blockIdx.y];
+    const int group = __builtin_amdgcn_readfirstlane(t.x);
+    const int first = __builtin_amdgcn_readfirstlane(t.y);
+    M = __builtin_amdgcn_readfirstlane(t.z);
+    if (group < 0 || M <= 0) return false;
+    if (grp.rows != nullptr) grp.rows += first;
+    else A += (int64_t)first * lda;
+    W += (int64_t)group * grp.w_stride;
+    C += (int64_t)first * ldc;
+  } else {
+    A += (int64_t)blockIdx.y * grp.a_step;
+    W += (int64_t)blockIdx.y * grp.w_stride;
+    C += (int64_t)blockIdx.y * grp.c_step;
+  }
+  return true;
+}
+__device__ __forceinline__ int group_row(const GroupTiles& grp, int row) {
+  return grp.rows != nullptr ? grp.rows[row] : row;
 }
 // Epilogues that pair two weight columns into one output column.
 __device__ __forceinline__ bool gated(const GemmArgs& g) {
@@ -120,7 +163,7 @@ __device__ __forceinline__ void store_result(const DenseArgs& g, int m, int n,
   if (gated(g)) {
     const int f = (n >> 4) * 8 + (n & 7);
     reinterpret_cast<bf16_t*>(g.C)[(size_t)m * (g.N >> 1) + f] =
-        f32_to_bf16(clamped_glu(v, v_gate, g.glu_limit, g.glu_alpha));
+        f32_to_bf16(clamped_glu(v, v_gate, g.glu_limit, g.glu_alpha, g.glu_add));
     return;
   }
   const size_t o = (size_t)m * g.ldc + n;
@@ -141,6 +184,8 @@ void launch_gemm_big(int w_dtype, const GemmPlan& p, GemmArgs g,
                      float* partials, hipStream_t s);
 // The same for t5d_dense (bfloat16 weights, K not split).
 void launch_dense_big(const GemmPlan& p, DenseArgs g, hipStream_t s);
+// Grouped layers on the many-row kernel (gemm_rows.hip): tiles of 256 rows.
+int launch_grouped_rows(hipStream_t s, const GroupedArgs& g, int n_tiles);
 bool gemm_big_has_tile(int mp, int nt);
 // Sum of split-K parts + scale + residual -> out, optional RMS norm -> normed.
 int launch_splitk_finish(hipStream_t s, const float* partials, int k_parts,

@@ -40,6 +40,10 @@ struct WinArgs {
   int HP, gs, splits;
   float* parts;  // [S, G, splits, gs, HP + 2]
   const int32_t* gate;
+  // window_rows_kernel over a span instead of rings: position first[s] + i of
+  // portion s is row off[s] + i, rows ld_kv apart, a head's HP columns side by side
+  const int32_t *span_off, *span_first;
+  int ld_kv;
 };
 
 // ---- norms of the new queries and keys, ring update ------------------------------
@@ -214,7 +218,7 @@ __device__ __forceinline__ f32x4_v mfma(const Frag& x, const Frag& y, f32x4_v c)
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(x.v, y.v, c, 0, 0, 0);
 }
 
-template <int DT>
+template <int DT, bool SPAN = false>
 __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1)
 window_rows_kernel(WinArgs g) {
   constexpr int HP = DT * 32, VT = DT * 2, KB = 64, MT = 2;
@@ -234,9 +238,12 @@ window_rows_kernel(WinArgs g) {
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int n16 = lane & 15, gq = lane >> 4;
   const int W = a.window > 0 ? a.window : (1 << 30);
-  const size_t base = ((size_t)g.b.seq_slot[seq] * a.G + kv) * a.ring;
-  const bf16_t* K = reinterpret_cast<const bf16_t*>(a.key_ring) + base * HP;
-  const bf16_t* V = reinterpret_cast<const bf16_t*>(a.value_ring) + base * HP;
+  const size_t base = SPAN ? (size_t)g.span_off[seq] * g.ld_kv + (size_t)kv * HP
+                           : ((size_t)g.b.seq_slot[seq] * a.G + kv) * a.ring * HP;
+  const bf16_t* K = reinterpret_cast<const bf16_t*>(a.key_ring) + base;
+  const bf16_t* V = reinterpret_cast<const bf16_t*>(a.value_ring) + base;
+  const int ld_kv = SPAN ? g.ld_kv : HP;
+  const int first = SPAN ? g.span_first[seq] : 0;
 
   const float scale2 = a.scale * kLog2e;
   int pos[MT], tok[MT], head[MT];
@@ -277,17 +284,17 @@ window_rows_kernel(WinArgs g) {
   constexpr int KRS = 256 / (HP / 8);            // key rows per pass
   const int vpair = threadIdx.x & 31, vcol = threadIdx.x >> 5;
   auto fetch = [&](int jt) {
-    const size_t r = (size_t)(jt % a.ring);
+    const size_t r = (size_t)(SPAN ? jt - first : jt % a.ring);
 #pragma unroll
     for (int i = 0; i < DT; ++i)
-      kr[i] = *reinterpret_cast<const uint4*>(K + (r + krow + KRS * i) * HP +
+      kr[i] = *reinterpret_cast<const uint4*>(K + (r + krow + KRS * i) * ld_kv +
                                               8 * kpiece);
 #pragma unroll
     for (int i = 0; i < NVP; ++i)
       if (vcol + 8 * i < HP / 8) {
-        const bf16_t* v = V + (r + 2 * vpair) * HP + 8 * (vcol + 8 * i);
+        const bf16_t* v = V + (r + 2 * vpair) * ld_kv + 8 * (vcol + 8 * i);
         va[i] = *reinterpret_cast<const uint4*>(v);
-        vb[i] = *reinterpret_cast<const uint4*>(v + HP);
+        vb[i] = *reinterpret_cast<const uint4*>(v + ld_kv);
       }
   };
   fetch(j_begin);
@@ -693,6 +700,41 @@ static void launch_wave(hipStream_t s, const WinArgs& g) {
 #undef T5D_WW
 }
 
+static WinArgs win_args(const t5d_window_attention& a, const t5d_ragged& b, int HP) {
+  WinArgs g = {};
+  g.a = a; g.b = b;
+  g.HP = HP; g.gs = a.H / a.G; g.splits = 1;
+  g.parts = (float*)a.workspace;
+  g.gate = tls_gate;
+  return g;
+}
+
+int launch_window_span(hipStream_t s, const t5d_window_attention& a,
+                       const t5d_ragged& b, const t5d_span& span, int ld_kv) {
+  WinArgs g = win_args(a, b, t5d_window_head_pad(a.D, a.Dv));
+  g.span_off = span.off; g.span_first = span.first; g.ld_kv = ld_kv;
+  const int64_t tiles = ((int64_t)b.max_len * g.gs + 127) / 128;
+  const dim3 grid((unsigned)tiles, b.S, a.G), block(256);
+#define T5D_SPAN(DT_) \
+  hipLaunchKernelGGL((window_rows_kernel<DT_, true>), grid, block, 0, s, g)
+  if (g.HP == 32) T5D_SPAN(1);
+  else if (g.HP == 64) T5D_SPAN(2);
+  else if (g.HP == 128) T5D_SPAN(4);
+  else T5D_SPAN(8);
+#undef T5D_SPAN
+  T5D_CHECK_LAUNCH("window attention (span)");
+  return T5D_OK;
+}
+
+int launch_window_wave(hipStream_t s, const t5d_window_attention& a,
+                       const t5d_ragged& b, int HP) {
+  const WinArgs g = win_args(a, b, HP);
+  if (a.dtype == T5D_BF16) launch_wave<bf16_t>(s, g);
+  else launch_wave<float>(s, g);
+  T5D_CHECK_LAUNCH("window attention (wave)");
+  return T5D_OK;
+}
+
 }  // namespace t5d
 
 using namespace t5d;
@@ -736,13 +778,9 @@ extern "C" int t5d_window_attention_run(void* stream, const t5d_window_attention
               a->ring, a->window, b->max_len);
   T5D_REQUIRE(variant >= 0 && variant <= 3, T5D_EINVAL,
               "t5d_window_attention_run: variant %d", variant);
-  WinArgs g;
-  g.a = *a; g.b = *b;
-  g.HP = t5d_window_head_pad(a->D, a->Dv);
+  WinArgs g = win_args(*a, *b, t5d_window_head_pad(a->D, a->Dv));
   T5D_REQUIRE(g.HP > 0, T5D_ELIMIT, "t5d_window_attention_run: head size %d / %d",
               a->D, a->Dv);
-  g.gs = a->H / a->G; g.splits = 1; g.parts = (float*)a->workspace;
-  g.gate = tls_gate;
   hipStream_t s = as_stream(stream);
   const bool bf16 = a->dtype == T5D_BF16;
   const int GS = step_group(g.gs, g.HP);

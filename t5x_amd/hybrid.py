@@ -1,22 +1,25 @@
-"""Decoder-only models whose layers mix windowed softmax attention with linear
-recurrences, on the HIP kernels behind t5d_hybrid_step.
+"""Decoder-only models whose layers mix windowed softmax attention, latent
+attention and linear recurrences, on the HIP kernels behind t5d_hybrid_step.
 
 A model is a list of layers, each a mixer from MIXERS (with sizes of its own) and
-an optional gated feed-forward, over a float32 residual stream; a range of layers
-may run several times in a row (a loop), every pass with caches of its own.
+an optional feed-forward — one gated unit, or a mixture of them chosen by token id
+— over a float32 residual stream, or several that hyper-connections mix.  A range of
+layers may run several times in a row (a loop), every pass with caches of its own.
+What a family of models fixes beside that is its Design.
 Sequences are fed in portions of any length: what a sequence carries from one
-portion to the next — a ring of keys and values per attention pass, a matrix
-state and the convolution's last inputs per recurrent pass — lives in its slot of
-the cache tree, and a portion that starts at position 0 starts from nothing
-whatever the slot held before.
+portion to the next — a ring of keys and values (or of the latents they come from)
+per attention pass, a matrix state and the convolution's last inputs per recurrent
+pass — lives in its slot of the cache tree, and a portion that starts at position 0
+starts from nothing whatever the slot held before.
 
 Weights are packed once per parameter set.  All widths are padded to the tiles of
 the matrix-core kernels with zero weights, so the padding columns of every
 activation are zero.
 """
 
+import ctypes
 import dataclasses
-from typing import Any, Mapping, Optional, Tuple
+from typing import Any, Mapping, Optional, Tuple, Union
 
 import numpy as np
 import torch
@@ -26,8 +29,33 @@ from t5x_amd import network
 from t5x_amd import ops
 
 _ACT = {'float32': torch.float32, 'bfloat16': torch.bfloat16}
-GLU_ALPHA = 1.702     # of the clamped gated unit
 UNIT_EPS = 1e-6       # inside the root of the unit norms
+# A call expands the latents its windows show into keys and values where they are
+# at most this many per new token.
+SPAN_ROWS = 2
+
+
+@dataclasses.dataclass(frozen=True)
+class Design:
+  """What every model of an architecture has in common.
+  streams: one residual stream with hyper-connections between as many as the
+  configuration says, a scaled embedding and a norm before every branch; else one
+  stream, the embedding plus a sinusoid of the position, a norm before and after.
+  dense: the gated unit of a feed-forward that is not a mixture; every unit is
+  min(g, limit) sigmoid(alpha g) (clamp(u, limit) + add), as (alpha, add), and
+  dense_limit None reads the limit from the configuration."""
+  streams: bool
+  dense: Tuple[float, float]
+  dense_limit: Optional[float] = None
+
+
+CLAMPED_UNIT = (1.702, 1.0)
+SILU_UNIT = (1.0, 0.0)
+
+DESIGNS = {
+    'Mokivik': Design(streams=False, dense=CLAMPED_UNIT),
+    'Nutizen': Design(streams=True, dense=SILU_UNIT, dense_limit=float('inf')),
+}
 
 
 @dataclasses.dataclass(frozen=True)
@@ -42,18 +70,42 @@ class MixerConfig:
   scale: float = 1.0     # attention: factor of q . k
   taps: int = 0          # convolution length, 0 = none
   tau: float = 1.0       # decay = sigmoid(z)^(1 / tau)
+  q_rank: int = 0        # latent attention: sizes of the queries' latent and
+  kv_rank: int = 0       # of the cached one
+  kv_from: Optional[int] = None  # the layer whose cached latents it reads
+  reach: int = 0         # window that the ring serves: the widest of its readers
 
 
 @dataclasses.dataclass(frozen=True)
 class FeedForwardConfig:
   ff: int
   limit: float
+  alpha: float = CLAMPED_UNIT[0]
+  add: float = CLAMPED_UNIT[1]
+
+
+@dataclasses.dataclass(frozen=True)
+class ExpertsConfig:
+  """A mixture: a table gives each token id `top` of `experts` units, each with
+  weight 1 / top; a shared one runs for every token behind a sigmoid gate."""
+  experts: int
+  top: int
+  expert: FeedForwardConfig
+  shared: Optional[FeedForwardConfig] = None
 
 
 @dataclasses.dataclass(frozen=True)
 class LayerConfig:
   mixer: MixerConfig
-  mlp: Optional[FeedForwardConfig] = None
+  mlp: Union[None, FeedForwardConfig, ExpertsConfig] = None
+
+  @property
+  def experts(self) -> Optional[ExpertsConfig]:
+    return self.mlp if isinstance(self.mlp, ExpertsConfig) else None
+
+  @property
+  def dense(self) -> Optional[FeedForwardConfig]:
+    return self.mlp if isinstance(self.mlp, FeedForwardConfig) else None
 
 
 @dataclasses.dataclass(frozen=True)
@@ -72,10 +124,14 @@ class HybridConfig:
   layers: Tuple[LayerConfig, ...]
   loop: Optional[LoopConfig] = None
   dtype: str = 'bfloat16'
+  streams: int = 0           # 0: one residual stream, see Design
+  hyper: bool = False        # hyper-connections between the streams
+  embed_scale: float = 1.0
 
   @classmethod
   def from_dict(cls, c: Mapping[str, Any], dtype: str = 'bfloat16'):
     """From a parsed config.json; raises on what these kernels do not compute."""
+    design = DESIGNS[c.get('architecture', 'Mokivik')]
     layers = []
     for i, entry in enumerate(c['layers']):
       kind, m, mlp = entry['type'], entry['mixer'], entry.get('mlp')
@@ -87,16 +143,31 @@ class HybridConfig:
           dim=int(m['dim']), vdim=int(m['vdim']),
           window=int((m.get('mask') or {}).get('size', 0)),
           scale=float(m.get('scale', 1.0)), taps=int(m.get('conv', 0)),
-          tau=float(m.get('tau', 1.0)))
+          tau=float(m.get('tau', 1.0)), q_rank=int(m.get('q_rank', 0)),
+          kv_rank=int(m.get('kv_rank', 0)), kv_from=m.get('kv_from'))
       if mixer.heads % mixer.kv_heads:
         raise ValueError(f'layer {i}: {mixer.heads} heads over '
                          f'{mixer.kv_heads} key/value heads')
-      if mlp is not None:
-        if mlp.get('kind', 'dense') != 'dense':
-          raise ValueError(f'layer {i}: unknown feed-forward {mlp["kind"]!r}')
-        mlp = FeedForwardConfig(int(mlp['ff']), float(mlp['limit']))
-      layers.append(LayerConfig(mixer, mlp))
+      if mixer.kv_from is not None:
+        j = mixer.kv_from
+        src = layers[j].mixer if 0 <= j < i else None
+        if (src is None or src.type != kind or src.kv_from is not None or
+            src.kv_rank != mixer.kv_rank):
+          raise ValueError(f'layer {i}: no latents of size {mixer.kv_rank} '
+                           f'in layer {j}')
+      layers.append(LayerConfig(mixer, _feed_forward(mlp, design, i)))
+    for i, layer in enumerate(layers):
+      windows = [l.mixer.window for j, l in enumerate(layers)
+                 if i in (j, l.mixer.kv_from)]
+      reach = 0 if 0 in windows else max(windows)
+      layers[i] = dataclasses.replace(
+          layer, mixer=dataclasses.replace(layer.mixer, reach=reach))
     loop = c.get('loop')
+    if design.streams and loop is not None:
+      raise ValueError('a loop over layers with several residual streams')
+    if not design.streams and any(
+        l.experts or l.mixer.kv_from is not None for l in layers):
+      raise ValueError('experts and shared latents need a design with streams')
     if loop is not None:
       loop = LoopConfig(int(loop['start']), int(loop['stop']),
                         int(loop['times']))
@@ -106,7 +177,10 @@ class HybridConfig:
       raise ValueError(f'unsupported dtype {dtype!r}')
     return cls(vocab_size=int(c['vocab']), width=int(c['width']),
                eps=float(c['norm']['eps']), layers=tuple(layers), loop=loop,
-               dtype=dtype)
+               dtype=dtype,
+               streams=int(c.get('streams', 1)) if design.streams else 0,
+               hyper=design.streams and 'streams' in c,
+               embed_scale=float((c.get('embedding') or {}).get('scale', 1.0)))
 
   def runs(self):
     """The layers in the order they run: (layer, pass that starts here or
@@ -119,6 +193,11 @@ class HybridConfig:
     return ([(i, None) for i in range(loop.start)] + body +
             [(i, None) for i in range(loop.stop, n)])
 
+  def span_windows(self):
+    """Windows of the layers that attend to expanded latents."""
+    return sorted({l.mixer.window for l in self.layers
+                   if l.mixer.type == 'latent_attention'})
+
   def param_shapes(self):
     """name -> shape of every tensor."""
     W, V = self.width, self.vocab_size
@@ -126,17 +205,57 @@ class HybridConfig:
     if self.loop is not None:
       out['loop.in'] = (W, 2 * W)
       out['loop.step'] = (self.loop.times, W)
+    n = self.streams
+
+    def unit(prefix, F):
+      out[prefix + 'gate'] = out[prefix + 'up'] = (F, W)
+      out[prefix + 'down'] = (W, F)
+
+    def around(p, q):  # what stands before and after branch q of a layer
+      out[f'{p}norm{q}'] = (W,)
+      if not n:
+        out[f'{p}norm{q}b'] = (W,)
+      if self.hyper:
+        out.update({f'{p}hc{q}.in': (n,), f'{p}hc{q}.out': (n,),
+                    f'{p}hc{q}.mix': (n, n)})
+
     for i, layer in enumerate(self.layers):
       p = f'l{i}.'
-      out[p + 'norm1'] = out[p + 'norm1b'] = (W,)
+      around(p, 1)
       out.update({p + 'mix.' + k: v for k, v in
                   MIXERS[layer.mixer.type].shapes(layer.mixer, W).items()})
       if layer.mlp is not None:
-        F = layer.mlp.ff
-        out[p + 'norm2'] = out[p + 'norm2b'] = (W,)
-        out[p + 'mlp.gate'] = out[p + 'mlp.up'] = (F, W)
-        out[p + 'mlp.down'] = (W, F)
+        around(p, 2)
+      if layer.dense:
+        unit(p + 'mlp.', layer.dense.ff)
+      elif layer.experts:
+        x = layer.experts
+        out[p + 'mlp.table'] = (V, x.top)
+        for e in range(x.experts):
+          unit(f'{p}mlp.e{e}.', x.expert.ff)
+        if x.shared:
+          unit(p + 'mlp.shared.', x.shared.ff)
+          out[p + 'mlp.shared.sg'] = (1, W)
     return out
+
+
+def _feed_forward(c, design: Design, i: int):
+  """The feed-forward that layer i's configuration names."""
+  if c is None:
+    return None
+  kind = c.get('kind', 'dense')
+  if kind == 'dense':
+    limit = design.dense_limit
+    return FeedForwardConfig(int(c['ff']), float(c['limit'] if limit is None
+                                                 else limit), *design.dense)
+  if kind != 'moe':
+    raise ValueError(f'layer {i}: unknown feed-forward {kind!r}')
+  unit = lambda u: FeedForwardConfig(int(u['ff']), float(u['limit']))
+  experts, top = int(c['router']['experts']), int(c['router']['top'])
+  if not 0 < top <= experts:
+    raise ValueError(f'layer {i}: {top} of {experts} experts')
+  return ExpertsConfig(experts, top, unit(c['expert']),
+                       unit(c['shared']) if c.get('shared') else None)
 
 
 def _pad(n: int, to: int) -> int:
@@ -213,10 +332,122 @@ class _AttentionMixer:
 
   leaves = ('key_ring', 'value_ring')
 
+  @staticmethod
+  def bytes_per_row(m, ring_len, el):
+    return 2 * m.kv_heads * ring_len(m.window) * el * _lib.load(
+    ).t5d_window_head_pad(m.dim, m.vdim)
+
+  @staticmethod
+  def ring(tensors):
+    return tensors[0].shape[2]
+
+  @staticmethod
+  def set_ring(layer, ring):
+    layer.attention.ring = ring
+
+
+class _LatentAttentionMixer:
+  """Sliding-window attention with a sink whose keys and values are linear maps of
+  a cached latent, the layer's own or an earlier layer's, and whose queries come
+  through a latent too."""
+
+  @staticmethod
+  def shapes(m, width):
+    out = {'dq': (m.q_rank, width), 'dq.norm': (m.q_rank,),
+           'uq': (m.heads * m.dim, m.q_rank),
+           'uk': (m.heads * m.dim, m.kv_rank),
+           'uv': (m.heads * m.vdim, m.kv_rank), 'sink': (m.heads,),
+           'o': (width, m.heads * m.vdim)}
+    if m.kv_from is None:
+      out.update({'dkv': (m.kv_rank, width), 'dkv.norm': (m.kv_rank,)})
+    return out
+
+  @staticmethod
+  def pads(m):
+    """(columns per head of queries, keys and values; of the cached latent; of
+    the queries' latent)."""
+    lib = _lib.load()
+    hp, rp = lib.t5d_window_head_pad(m.dim, m.vdim), lib.t5d_latent_pad(m.kv_rank)
+    if hp < 0 or rp < 0:
+      raise ValueError(f'head size {m.dim} / {m.vdim} or latent size {m.kv_rank} '
+                       'is not supported')
+    return hp, rp, _pad(m.q_rank, 64)
+
+  @classmethod
+  def fill(cls, layer, m, get, keep, eps, ld, pack):
+    H, D, Dv, rank = m.heads, m.dim, m.vdim, m.kv_rank
+    hp, rp, qp = cls.pads(m)
+    cols = _Columns()
+    own = m.kv_from is None
+    for name in ('dq', 'dkv') if own else ('dq',):
+      cols.add(name, get(name))
+    layer.mix = _lib.MIX_LATENT_ATTENTION
+    layer.proj_n = _pad(cols.n, 16)
+    layer.proj = pack(cols.matrix(ld))
+    a = layer.latent
+    a.H, a.D, a.Dv, a.rank, a.q_rank = H, D, Dv, rank, m.q_rank
+    a.window, a.scale, a.eps = m.window, m.scale, eps
+    a.off_q, a.off_kv = cols.at['dq'], cols.at['dkv'] if own else -1
+
+    def padded(w, *shape):
+      out = torch.zeros(shape, dtype=torch.float32, device=w.device)
+      out[tuple(slice(n) for n in w.shape)] = w
+      return out
+
+    a.q_norm = keep(padded(get('dq.norm'), qp))
+    if own:
+      a.kv_norm = keep(padded(get('dkv.norm'), rp))
+    a.sink = keep(get('sink'))
+    uq = padded(get('uq').reshape(H, D, m.q_rank), H, hp, qp)
+    uk = padded(get('uk').reshape(H, D, rank), H, hp, rp)
+    uv = padded(get('uv').reshape(H, Dv, rank), H, hp, rp)
+    a.uq = pack(uq.reshape(H * hp, qp).t().contiguous())
+    a.ukv = pack(torch.cat([uk, uv]).reshape(2 * H * hp, rp).t().contiguous())
+    a.absorb = pack.many(list(uk))[0]
+    vp = _pad(Dv, 16)
+    uv = padded(get('uv').reshape(H, Dv, rank), H, vp, rp)
+    a.expand = pack.many([w.t().contiguous() for w in uv])[0]
+
+  @classmethod
+  def cache(cls, m, rows, ring_len, act, dev):
+    if m.kv_from is not None:
+      return {}
+    return {'latent_ring': torch.zeros((rows, ring_len(m.reach), cls.pads(m)[1]),
+                                       dtype=act, device=dev)}
+
+  leaves = ('latent_ring', None)
+
+  @classmethod
+  def bytes_per_row(cls, m, ring_len, el):
+    return 0 if m.kv_from is not None else (
+        ring_len(m.reach) * cls.pads(m)[1] * el)
+
+  @staticmethod
+  def ring(tensors):
+    return tensors[0].shape[1]
+
+  @staticmethod
+  def set_ring(layer, ring):
+    layer.latent.ring = ring
+
 
 class _RecurrentMixer:
   """What the linear recurrences share."""
   leaves = ('state', 'conv_ring')
+
+  @staticmethod
+  def bytes_per_row(m, ring_len, el):
+    del ring_len
+    return 4 * m.heads * m.dim * m.vdim + el * m.taps * (
+        2 * m.kv_heads * m.dim + m.heads * m.vdim)
+
+  @staticmethod
+  def ring(tensors):
+    del tensors  # a state of fixed size
+
+  @staticmethod
+  def set_ring(layer, ring):
+    pass
 
   @staticmethod
   def cache(m, rows, ring_len, act, dev):
@@ -316,7 +547,8 @@ class _ChannelDeltaMixer(_RecurrentMixer):
 
 
 MIXERS = {'attention': _AttentionMixer, 'gla': _GatedLinearMixer,
-          'channel_delta': _ChannelDeltaMixer}
+          'channel_delta': _ChannelDeltaMixer,
+          'latent_attention': _LatentAttentionMixer}
 
 
 # ------------------------------------------------------------------------------
@@ -333,7 +565,8 @@ class HybridWeights:
     act = self.act_dtype
     self.ld = ld = _pad(cfg.width, 64)
     self._kept = []
-    for name, shape in cfg.param_shapes().items():
+    shapes = cfg.param_shapes()
+    for name, shape in shapes.items():
       if name not in params:
         raise ValueError(f'parameter {name!r} is missing')
       have = tuple(np.shape(params[name]))
@@ -352,6 +585,21 @@ class HybridWeights:
       w = ops.pack_weight(kernel, act, act, gate_kernel=gate)
       self._kept.append(w.data)
       return w.data.data_ptr()
+
+    def pack_many(kernels, gates=None):
+      """Kernels of one shape one after the other -> (address, bytes of each)."""
+      first = out = None
+      for i, kernel in enumerate(kernels):
+        gate = gates[i] if gates is not None else None
+        data = ops.pack_weight(kernel, act, act, gate_kernel=gate).data
+        if out is None:
+          first, out = data, torch.empty((len(kernels),) + tuple(data.shape),
+                                         dtype=data.dtype, device=data.device)
+        out[i] = data
+      self._kept.append(out)
+      return out.data_ptr(), first.numel() * first.element_size()
+
+    pack.many = pack_many
 
     def padded(name, k, n):
       """Transposed to input-major and padded to [k, n]."""
@@ -380,19 +628,50 @@ class HybridWeights:
     for i, lc in enumerate(cfg.layers):
       layer, m = self.layers[i], lc.mixer
       mix = lambda name, i=i: get(f'l{i}.mix.{name}')
-      layer.norm1, layer.norm1b = (keep(get(f'l{i}.{n}'))
-                                   for n in ('norm1', 'norm1b'))
+      around = [('norm1', 'norm1'), ('norm1b', 'norm1b')]
+      around += [(f'{leaf}1', f'hc1.{leaf}') for leaf in ('in', 'mix', 'out')]
+      if lc.mlp is not None:
+        around += [(field.replace('1', '2'), name.replace('1', '2'))
+                   for field, name in around]
+      for field, name in around:
+        if f'l{i}.{name}' in shapes:
+          setattr(layer, field, keep(get(f'l{i}.{name}')))
       MIXERS[m.type].fill(layer, m, mix, keep, cfg.eps, ld, pack)
       layer.out_k = _pad(m.heads * m.vdim, 64)
       layer.out = pack(padded(f'l{i}.mix.o', layer.out_k, ld))
-      if lc.mlp is not None:
-        layer.F = F = _pad(lc.mlp.ff, 64)
-        layer.norm2, layer.norm2b = (keep(get(f'l{i}.{n}'))
-                                     for n in ('norm2', 'norm2b'))
-        layer.glu = pack(padded(f'l{i}.mlp.gate', ld, F),
-                         padded(f'l{i}.mlp.up', ld, F))
-        layer.down = pack(padded(f'l{i}.mlp.down', F, ld))
-        layer.glu_limit, layer.glu_alpha = lc.mlp.limit, GLU_ALPHA
+
+      def unit(prefix, ff, pack=pack):
+        F = _pad(ff, 64)
+        return (F, pack(padded(prefix + 'gate', ld, F),
+                        padded(prefix + 'up', ld, F)),
+                pack(padded(prefix + 'down', F, ld)))
+
+      if lc.dense:
+        layer.F, layer.glu, layer.down = unit(f'l{i}.mlp.', lc.dense.ff)
+        layer.glu_limit, layer.glu_alpha, layer.glu_add = (
+            lc.dense.limit, lc.dense.alpha, lc.dense.add)
+      elif lc.experts:
+        x, e, p = lc.experts, layer.experts, f'l{i}.mlp.'
+        table = torch.as_tensor(np.asarray(
+            params[p + 'table'].cpu() if isinstance(params[p + 'table'],
+                                                    torch.Tensor)
+            else params[p + 'table']).astype(np.int64))
+        if int(table.min()) < 0 or int(table.max()) >= x.experts:
+          raise ValueError(f'parameter {p}table names experts beyond the '
+                           f'{x.experts} there are')
+        e.table = keep(table, torch.int32)
+        e.n, e.top, e.F = x.experts, x.top, _pad(x.expert.ff, 64)
+        each = lambda leaf, *shape, p=p, n=x.experts: [
+            padded(f'{p}e{k}.{leaf}', *shape) for k in range(n)]
+        e.glu, e.glu_stride = pack.many(each('gate', ld, e.F),
+                                        each('up', ld, e.F))
+        e.down, e.down_stride = pack.many(each('down', e.F, ld))
+        e.limit, e.alpha, e.add = x.expert.limit, x.expert.alpha, x.expert.add
+        if x.shared:
+          e.shared_F, e.shared_glu, e.shared_down = unit(p + 'shared.',
+                                                         x.shared.ff)
+          e.shared_limit = x.shared.limit
+          e.shared_gate = keep(get(p + 'shared.sg').reshape(-1))
 
   def nbytes(self):
     return sum(t.numel() * t.element_size() for t in self._kept)
@@ -408,16 +687,18 @@ class _Buffers:
     self.layers = (_lib.HybridLayer * len(cfg.layers))()
     self._kept = kept = []
 
-    def rows(n, dtype=act, zero=False):
-      t = (torch.zeros if zero else torch.empty)((tokens, n), dtype=dtype,
+    def rows(n, dtype=act, zero=False, per=1):
+      t = (torch.zeros if zero else torch.empty)((tokens * per, n), dtype=dtype,
                                                  device=device)
       kept.append(t)
       return t
 
     lib = _lib.load()
     f32 = torch.float32
-    self.x, self.x0 = rows(ld, f32), rows(ld, f32)
-    self.h, self.cat, self.y = rows(ld), rows(2 * ld), rows(ld)
+    self.x = rows(ld * max(1, cfg.streams), f32)
+    self.h, self.y = rows(ld), rows(ld)
+    self.x0, self.cat = ((rows(ld, f32), rows(2 * ld)) if cfg.loop else
+                         (None, None))
     self.proj = rows(max(l.proj_n for l in w.layers))
     low_n = max(l.low_n for l in w.layers)
     self.low = rows(low_n, f32) if low_n else None
@@ -435,9 +716,11 @@ class _Buffers:
       self.layers[i] = w.layers[i]
       layer, m = self.layers[i], lc.mixer
       layer.mix_rows = pooled(m.heads * m.vdim, layer.out_k)
-      if lc.mlp is not None:
-        layer.ff_rows = pooled(lc.mlp.ff, layer.F)
-      if layer.mix == _lib.MIX_WINDOW_ATTENTION:
+      if lc.dense:
+        layer.ff_rows = pooled(lc.dense.ff, layer.F)
+      if layer.mix == _lib.MIX_LATENT_ATTENTION:
+        ws = max(ws, lib.t5d_latent_workspace_bytes(m.kv_rank))
+      elif layer.mix == _lib.MIX_WINDOW_ATTENTION:
         hp = lib.t5d_window_head_pad(m.dim, m.vdim)
         q_cols = max(q_cols, m.heads * hp)
         ws = max(ws, lib.t5d_window_workspace_bytes(seqs, m.heads, m.dim,
@@ -449,13 +732,63 @@ class _Buffers:
             m.vdim))
     self.q_rows = rows(q_cols) if q_cols else None
     self.workspace = torch.empty((ws,), dtype=torch.uint8, device=device)
+    self._latent_buffers(cfg, act, rows)
+    self._expert_buffers(cfg, ld, act, rows, device)
+
+  def _latent_buffers(self, cfg, act, rows):
+    """Scratch of the latent attention layers, which run one after the other."""
+    layers = [(l.latent, cfg.layers[i].mixer) for i, l in enumerate(self.layers)
+              if l.mix == _lib.MIX_LATENT_ATTENTION]
+    if not layers:
+      return
+    pads = [(m.heads,) + _LatentAttentionMixer.pads(m) for _, m in layers]
+    cq, q = rows(max(p[3] for p in pads)), rows(max(p[0] * p[1] for p in pads))
+    ql, ol = (rows(max(p[0] * p[2] for p in pads)) for _ in range(2))
+    # keys and values expanded from the latents of a span: where portions can
+    # be longer than a token, and for bfloat16 only
+    spans = act == torch.bfloat16 and self.tokens > self.seqs
+    if spans:
+      lat = rows(max(p[2] for p in pads), per=SPAN_ROWS)
+      kv = rows(max(2 * p[0] * p[1] for p in pads), per=SPAN_ROWS)
+    for a, _ in layers:
+      a.cq, a.q, a.ql, a.ol = (t.data_ptr() for t in (cq, q, ql, ol))
+      if spans:
+        a.lat, a.kv = lat.data_ptr(), kv.data_ptr()
+        a.span_rows = SPAN_ROWS * self.tokens
+
+  def _expert_buffers(self, cfg, ld, act, rows, device):
+    """What the mixtures share, and each one's sorted tokens (found for all of
+    them at the start of a call)."""
+    layers = [l.experts for l in self.layers if l.experts.n]
+    if not layers:
+      return
+    lib = _lib.load()
+    top = max(e.top for e in layers)
+    hidden = rows(max(e.F * e.top for e in layers))
+    out, gate = rows(ld * top), rows(1, torch.float32)
+    shared = max(e.shared_F for e in layers)
+    shared = rows(shared) if shared else None
+    least = 8 if act == torch.float32 else 16  # rows of the smallest tiles
+
+    def ints(n):
+      t = torch.full((n,), -1, dtype=torch.int32, device=device)
+      self._kept.append(t)
+      return t.data_ptr()
+
+    for e in layers:
+      n = self.tokens * e.top
+      e.max_tiles = lib.t5d_route_max_tiles(n, e.n, least)
+      e.tiles, e.token_of, e.entry_of = ints(4 * e.max_tiles), ints(n), ints(n)
+      e.rows, e.out, e.gate = (t.data_ptr() for t in (hidden, out, gate))
+      e.shared_rows = _lib.ptr(shared)
 
 
 class Portions:
   """The token arrays of one call (t5d_ragged), uploaded as one int32 array.
-  portions: (slot, position of the first token, token ids) per sequence."""
+  portions: (slot, position of the first token, token ids) per sequence.
+  windows: of the layers that expand latents (t5d_span)."""
 
-  def __init__(self, portions, want_rows, device):
+  def __init__(self, portions, want_rows, device, windows=()):
     lens = np.array([len(t) for _, _, t in portions], np.int32)
     self.M, self.S = int(lens.sum()), len(portions)
     self.max_len = int(lens.max())
@@ -467,17 +800,35 @@ class Portions:
     tokens = np.concatenate([np.asarray(t, np.int32) for _, _, t in portions])
     want = np.asarray(want_rows, np.int32)
     parts = [tokens, pos, seq, off, start, slot, want]
+    spans = []
+    if self.max_len > 1:
+      end = (start + lens + 63) // 64 * 64
+      for window in windows:
+        first = start * 0
+        if window:
+          first = np.maximum(0, start - window + 1) // 64 * 64
+        rows = np.concatenate([[0], np.cumsum(end - first)])
+        if rows[-1] <= SPAN_ROWS * self.M:
+          spans.append((window, int(rows[-1]), len(parts)))
+          parts += [rows.astype(np.int32), first.astype(np.int32)]
     self.data = torch.from_numpy(np.concatenate(parts)).to(device)
     r = self.ragged = _lib.Ragged()
     r.M, r.S, r.max_len = self.M, self.S, self.max_len
     at = self.data.data_ptr()
-    for name, part in zip(('tokens', 'tok_pos', 'tok_seq', 'seq_off',
-                           'seq_start', 'seq_slot', 'want'), parts):
-      if name == 'want':
-        self.want_ptr, self.n_want = at, len(part)
-      else:
-        setattr(r, name, at)
+    addresses = []
+    for part in parts:
+      addresses.append(at)
       at += 4 * len(part)
+    for name, address in zip(('tokens', 'tok_pos', 'tok_seq', 'seq_off',
+                              'seq_start', 'seq_slot'), addresses):
+      setattr(r, name, address)
+    self.want_ptr, self.n_want = addresses[6], len(want)
+    self._spans = (_lib.Span * max(1, len(spans)))()
+    for s, (window, rows, n) in zip(self._spans, spans):
+      s.window, s.rows = window, rows
+      s.off, s.first = addresses[n], addresses[n + 1]
+    r.spans = ctypes.cast(self._spans, ctypes.c_void_p)
+    r.n_spans = len(spans)
 
 
 class StepRows:
@@ -532,9 +883,7 @@ class HybridDecoder(network.DecodeContexts):
     layer run, and cache_index [rows] = positions each slot holds.  portion: the
     longest portion it will be fed (max_portion)."""
     cfg, dev = self.config, self._dev()
-    portion = min(portion or self.max_portion, self.max_portion, max_len)
-    ring_len = lambda window: _pad(
-        max_len if window == 0 else window - 1 + portion, 64)
+    ring_len = self._ring_len(max_len, portion)
     act = _ACT[cfg.dtype]
     tree = {}
     for r, (i, _) in enumerate(cfg.runs()):
@@ -543,20 +892,24 @@ class HybridDecoder(network.DecodeContexts):
     return {'decoder': tree,
             'cache_index': torch.zeros((rows,), dtype=torch.int32, device=dev)}
 
-  def cache_bytes(self, rows: int, max_len: int, portion=None) -> int:
-    cfg, n = self.config, 0
+  def _ring_len(self, max_len, portion):
+    """window -> positions in a ring (window 0: all)."""
     portion = min(portion or self.max_portion, self.max_portion, max_len)
+    return lambda window: _pad(
+        max_len if window == 0 else window - 1 + portion, 64)
+
+  def cache_bytes(self, rows: int, max_len: int, portion=None) -> int:
+    cfg, ring_len = self.config, self._ring_len(max_len, portion)
     el = 2 if cfg.dtype == 'bfloat16' else 4
-    for i, _ in cfg.runs():
-      m = cfg.layers[i].mixer
-      if m.type == 'attention':
-        ring = max_len if m.window == 0 else m.window - 1 + portion
-        n += 2 * m.kv_heads * _pad(ring, 64) * el * _lib.load(
-        ).t5d_window_head_pad(m.dim, m.vdim)
-      else:
-        n += 4 * m.heads * m.dim * m.vdim + el * m.taps * (
-            2 * m.kv_heads * m.dim + m.heads * m.vdim)
-    return rows * n
+    mixers = [cfg.layers[i].mixer for i, _ in cfg.runs()]
+    return rows * sum(MIXERS[m.type].bytes_per_row(m, ring_len, el)
+                      for m in mixers)
+
+  def _run_cache(self, cache, run, layer):
+    """The cache leaf that a run of a layer reads and writes."""
+    src = self.config.layers[layer].mixer.kv_from
+    # (layers with shared latents run once each: run = layer)
+    return cache['decoder'][f'run_{run if src is None else src}']
 
   # -- the step function --------------------------------------------------------
   def _buffers(self, w, tokens, seqs):
@@ -581,9 +934,8 @@ class HybridDecoder(network.DecodeContexts):
     cruns = (_lib.HybridRun * len(runs))()
     kept = []
     for r, (i, start) in enumerate(runs):
-      m, leaf = cfg.layers[i].mixer, cache['decoder'][f'run_{r}']
-      names = MIXERS[m.type].leaves
-      c = [leaf.get(n) for n in names]
+      m, leaf = cfg.layers[i].mixer, self._run_cache(cache, r, i)
+      c = [leaf.get(n) for n in MIXERS[m.type].leaves]
       for t in c:
         if t is not None and not t.is_contiguous():
           raise ValueError(f'cache leaf of run {r} is not contiguous')
@@ -591,13 +943,13 @@ class HybridDecoder(network.DecodeContexts):
       cruns[r].layer, cruns[r].enter = i, int(start is not None)
       cruns[r].enter_add = w.loop_steps[start] if start is not None else None
       cruns[r].cache0, cruns[r].cache1 = P(c[0]), P(c[1])
-      if m.type == 'attention':
-        layers[i].attention.ring = c[0].shape[2]
+      MIXERS[m.type].set_ring(layers[i], MIXERS[m.type].ring(c))
     mod = _lib.HybridModel()
     mod.dtype = _lib.dtype_code(w.act_dtype)
     mod.d, mod.ld, mod.V, mod.head_n = (cfg.width, w.ld, cfg.vocab_size,
                                         w.head_n)
     mod.n_layers, mod.n_runs, mod.eps = len(cfg.layers), len(runs), cfg.eps
+    mod.streams, mod.embed_scale = cfg.streams, cfg.embed_scale
     mod.embedding, mod.loop_in = w.embedding, w.loop_in
     mod.head, mod.final_norm = w.head, w.final_norm
     mod.layers, mod.runs = layers, cruns
@@ -619,7 +971,7 @@ class HybridDecoder(network.DecodeContexts):
     return self._step[1]
 
   def _run(self, w, cache, portions, want_rows, trace=None):
-    p = Portions(portions, want_rows, self._dev())
+    p = Portions(portions, want_rows, self._dev(), self.config.span_windows())
     bufs = self._buffers(w, p.M, p.S)
     model = self._model_for(w, bufs, cache)
     logits = None
@@ -682,9 +1034,10 @@ class HybridDecoder(network.DecodeContexts):
     limit = self.max_tokens
     for r, (i, _) in enumerate(self.config.runs()):
       m = self.config.layers[i].mixer
-      if m.type != 'attention':
+      leaf, mixer = self._run_cache(cache, r, i), MIXERS[m.type]
+      ring = mixer.ring([leaf.get(n) for n in mixer.leaves])
+      if ring is None:
         continue
-      ring = cache['decoder'][f'run_{r}']['key_ring'].shape[2]
       if m.window:
         limit = min(limit, ring - m.window + 1)
       for _, start, toks in portions:
@@ -789,7 +1142,9 @@ class HybridSampleStep(network.SampleStepGraph):
 def init_params(cfg: HybridConfig, seed: int = 0, device=None, rank: int = 64):
   """Random parameters by tensor name, generated on the device: linear weights
   normal(0, 1/sqrt(fan_in)), norms 1 + 0.1 normal, low-rank stages of `rank`,
-  decay biases spread so that memories last from a few tokens to hundreds."""
+  decay biases spread so that memories last from a few tokens to hundreds,
+  hyper-connections near one stream passed on and written to, tables of distinct
+  random experts."""
   device = device or torch.device('cuda')
   gen = torch.Generator(device=device)
   gen.manual_seed(seed)
@@ -798,7 +1153,15 @@ def init_params(cfg: HybridConfig, seed: int = 0, device=None, rank: int = 64):
   for name, shape in cfg.param_shapes().items():
     shape = tuple(rank if s is None else s for s in shape)
     leaf = name.rsplit('.', 1)[-1]
-    if 'norm' in leaf:
+    if leaf == 'table':
+      experts = cfg.layers[int(name[1:name.index('.')])].experts.experts
+      out[name] = torch.rand((shape[0], experts), generator=gen,
+                             device=device).argsort(1)[:, :shape[1]].to(torch.int32)
+    elif '.hc' in name:
+      out[name] = 0.1 * normal(shape) + (
+          torch.eye(shape[0], device=device) if leaf == 'mix' else
+          1.0 / cfg.streams if leaf == 'in' else 1.0)
+    elif 'norm' in leaf:
       out[name] = 1.0 + 0.1 * normal(shape)
     elif leaf == 'conv':
       out[name] = normal(shape) / np.sqrt(shape[1])

@@ -778,7 +778,7 @@ def dense(a, w: PackedWeight, out=None, out_dtype=None, n_store=None,
           glu=None):
   """a @ W over any number of rows (t5d_dense).  a [M, >= K] with unit column
   stride; n_store: only the first columns (float32 output of bfloat16 rows);
-  glu (limit, alpha): W is a gate | up pair and the clamped gated unit is
+  glu (limit, alpha, add): W is a gate | up pair and the clamped gated unit is
   applied."""
   if not a.is_cuda or a.dim() != 2 or a.stride(1) != 1 or a.shape[1] != w.K:
     raise ValueError(f'a is {tuple(a.shape)}; kernel K={w.K}')
@@ -794,11 +794,11 @@ def dense(a, w: PackedWeight, out=None, out_dtype=None, n_store=None,
   _chk(out, 'out', out_dtype, 2)
   if tuple(out.shape) != (M, cols):
     raise ValueError(f'out shape {tuple(out.shape)} != {(M, cols)}')
-  limit, alpha = glu or (0.0, 0.0)
+  limit, alpha, add = glu or (0.0, 0.0, 0.0)
   _lib.call('t5d_dense', _s(), _lib.dtype_code(a.dtype),
             _lib.dtype_code(out_dtype), a.data_ptr(), a.stride(0),
             w.data.data_ptr(), out.data_ptr(), cols, n_store, M, w.K, w.N, epi,
-            float(limit), float(alpha))
+            float(limit), float(alpha), float(add))
   return out
 
 

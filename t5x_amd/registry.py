@@ -59,6 +59,8 @@ ARCHITECTURES = {
     'T5.1.1': Architecture(_t5_module, _t5_model, checkpoints.load_params),
     'Mokivik': Architecture(_hybrid_module, _decoder_only_model,
                             _safetensors_params),
+    'Nutizen': Architecture(_hybrid_module, _decoder_only_model,
+                            _safetensors_params),
 }
 
 

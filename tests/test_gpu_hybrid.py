@@ -66,7 +66,7 @@ def test_clamped_glu(dt, M, K, F):
   a = dev(2 * rs.randn(M, K), dt)
   gate, up = (dev(rs.randn(K, F) / np.sqrt(K)) for _ in range(2))
   got = ops.dense(a, ops.pack_weight(gate, dt, gate_kernel=up),
-                  glu=(limit, alpha))
+                  glu=(limit, alpha, 1.0))
   g = np.minimum(host(a) @ host(gate.to(dt)), limit)
   u = np.clip(host(a) @ host(up.to(dt)), -limit, limit)
   want = g * oracle.sigmoid(alpha * g) * (u + 1)

@@ -225,7 +225,7 @@ def test_kernel_entry_points_check_their_arguments():
   assert lib.t5d_recurrence_run(None, r, b, 0) == -3
   assert b'512' in lib.t5d_last_error()
   assert lib.t5d_dense(None, _lib.BF16, _lib.BF16, 16, 64, 16, 16, 32, 32, 4,
-                       60, 32, 0, 0.0, 0.0) == -1
+                       60, 32, 0, 0.0, 0.0, 0.0) == -1
   assert lib.t5d_hybrid_step(None, _lib.HybridModel(), b, None, 0, None) == -1
 
 
