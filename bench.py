@@ -70,7 +70,8 @@ def parse_args():
   ap.add_argument('--lanes', type=int, default=None,
                   help='batch slices stepped concurrently (default: library)')
   ap.add_argument('--stage', default='decode',
-                  choices=['decode', 'encoder', 'dense', 'memory', 'hybrid'],
+                  choices=['decode', 'encoder', 'dense', 'memory', 'hybrid',
+                           'latent'],
                   help="'encoder': the once-per-batch stage before the decode "
                        'loop (encoder forward + cross K/V projection); a step '
                        "is one batch.  'dense': the decoder's dense layers on "
@@ -85,13 +86,15 @@ def parse_args():
                        'throughput of a decoder-only hybrid model (--hybrid-'
                        'size), its mixer kernels on their own, and beside them '
                        'a T5.1.1 encoder and decoder of the same width and '
-                       'depth')
+                       "depth.  'latent': the same for a model with latent "
+                       'attention, hyper-connections and experts by token '
+                       'table, beside a hybrid model of attention layers only')
   ap.add_argument('--hybrid-size', default='large',
                   choices=sorted(HYBRID_SIZES),
-                  help='width and feed-forward of --stage hybrid')
+                  help='width and feed-forward of --stage hybrid and latent')
   ap.add_argument('--hybrid-batch', type=int, default=None,
-                  help='prompts prefilled together with --stage hybrid '
-                       '(default 4)')
+                  help='prompts prefilled together with --stage hybrid and '
+                       'latent (default 4)')
   ap.add_argument('--in-flight', type=int, default=None,
                   help='also measure this many whole decodes of different '
                        'batches running on the device at once (default for '
@@ -1018,22 +1021,8 @@ class HybridStage:
     self.torch, self.hybrid, self.network = torch, hybrid, network
     W, F = HYBRID_SIZES[size]
     self.W, self.F, self.B, self.T, self.R = W, F, batch, prompt, rows
-    H = W // 128
-    mixers = {
-        'channel_delta': {'heads': H, 'kv_heads': H, 'dim': 128, 'vdim': 128,
-                          'conv': 4},
-        'gla': {'heads': H, 'dim': 128, 'vdim': 128, 'tau': 12.0},
-        'attention': {'heads': H, 'kv_heads': max(1, H // 4), 'dim': 128,
-                      'vdim': 128, 'mask': {'size': self.WINDOW},
-                      'scale': 128 ** -0.5}}
-    order = ['channel_delta', 'gla', 'channel_delta', 'attention']
-    mlp = {'kind': 'dense', 'ff': F, 'limit': 7.0}
-    self.config = {
-        'architecture': 'Mokivik', 'width': W, 'vocab': self.VOCAB,
-        'norm': {'eps': 1e-6},
-        'layers': [{'type': t, 'mixer': mixers[t], 'mlp': mlp}
-                   for t in (order * 2)[:self.LAYERS]]}
-    self.H = H
+    self.H = W // 128
+    self.config = self.make_config(W, F, self.H)
     self.cfg = hybrid.HybridConfig.from_dict(self.config, 'bfloat16')
     self.module = hybrid.HybridDecoder(self.cfg)
     self.module.max_portion = self.T   # a prompt is one portion
@@ -1041,6 +1030,24 @@ class HybridStage:
     self.params = hybrid.init_params(self.cfg, seed)
     self.w = self.module.decoder_weights(self.params)
     self.rs = np.random.Generator(np.random.PCG64(seed))
+
+  ORDER = ['channel_delta', 'gla', 'channel_delta', 'attention']
+  KERNEL_LAYERS = (3, 0, 1)
+
+  def make_config(self, W, F, H):
+    mixers = {
+        'channel_delta': {'heads': H, 'kv_heads': H, 'dim': 128, 'vdim': 128,
+                          'conv': 4},
+        'gla': {'heads': H, 'dim': 128, 'vdim': 128, 'tau': 12.0},
+        'attention': {'heads': H, 'kv_heads': max(1, H // 4), 'dim': 128,
+                      'vdim': 128, 'mask': {'size': self.WINDOW},
+                      'scale': 128 ** -0.5}}
+    mlp = {'kind': 'dense', 'ff': F, 'limit': 7.0}
+    return {
+        'architecture': 'Mokivik', 'width': W, 'vocab': self.VOCAB,
+        'norm': {'eps': 1e-6},
+        'layers': [{'type': t, 'mixer': mixers[t], 'mlp': mlp}
+                   for t in (self.ORDER * self.LAYERS)[:self.LAYERS]]}
 
   def prompts(self, n, length):
     return self.rs.integers(1, self.VOCAB, size=(n, length)).astype(np.int32)
@@ -1141,7 +1148,7 @@ class HybridStage:
       cache = self.module.init_cache(S, self.T + 64, portion=n)
       bufs.proj.normal_()
       M = S * n
-      for i in (3, 0, 1):
+      for i in self.KERNEL_LAYERS:
         kind = self.cfg.layers[i].mixer.type
         layer, leaf = bufs.layers[i], cache['decoder'][f'run_{i}']
         if kind == 'attention':
@@ -1185,6 +1192,204 @@ class HybridStage:
                     'achieved': round(rate, 1), 'peak': peak, 'unit': unit,
                     'frac': round(rate / peak, 4)})
     return out
+
+
+class AttentionStage(HybridStage):
+  """The hybrid family's attention layers only: the closest relative of
+  LatentStage."""
+
+  ORDER = ['attention']
+  KERNEL_LAYERS = (1,)
+
+  def kernels(self):
+    return super().kernels() + self.row_kernels()
+
+  def row_kernels(self):
+    """The feed-forward's dense layers and the row kernel."""
+    from t5x_amd import ops
+    torch, W, F = self.torch, self.W, self.F
+    out = []
+    for mode, M in (('prefill', self.B * self.T), ('decode', self.R)):
+      bf = lambda *s: torch.randn(s, device='cuda').to(torch.bfloat16)
+      f = lambda *s: torch.randn(s, device='cuda')
+      a = bf(M, W)
+      glu = ops.pack_weight(f(W, F), torch.bfloat16, gate_kernel=f(W, F))
+      down, hidden = ops.pack_weight(f(F, W), torch.bfloat16), bf(M, F)
+      for name, x, w, kw, width in (
+          ('gated dense', a, glu, {'glu': (7.0, 1.7, 1.0)}, F),
+          ('dense', hidden, down, {}, W)):
+        y = bf(M, width)
+        sec = time_kernel(torch, lambda: ops.dense(x, w, out=y, **kw), 10)
+        out.append(dense_entry(name, mode, sec, 2.0 * M * w.K * w.N,
+                               2.0 * w.K * w.N + 2.0 * M * (w.K + width)))
+      x, y, n = f(M, W), bf(M, W), f(W)
+      sec = time_kernel(torch, lambda: ops.stream_norm(
+          x, W, torch.bfloat16, y=y, norm=n), 10)
+      out.append(rate_entry(f'stream_norm ({mode})', sec, 12.0 * M * W, 'GB/s'))
+    return out
+
+
+def rate_entry(name, sec, work, unit):
+  peak = MFMA_BF16_PEAK_TFLOPS if unit == 'TFLOP/s' else HBM_PEAK_GBPS
+  rate = work / sec / (1e12 if unit == 'TFLOP/s' else 1e9)
+  return {'kernel': name, 'us': round(sec * 1e6, 2), 'achieved': round(rate, 1),
+          'peak': peak, 'unit': unit, 'frac': round(rate / peak, 4)}
+
+
+def dense_entry(name, mode, sec, flops, bytes_):
+  """A dense layer against the roof that binds it."""
+  if flops / (MFMA_BF16_PEAK_TFLOPS * 1e12) > bytes_ / (HBM_PEAK_GBPS * 1e9):
+    return rate_entry(f'{name} ({mode})', sec, flops, 'TFLOP/s')
+  return rate_entry(f'{name} ({mode})', sec, bytes_, 'GB/s')
+
+
+class LatentStage(HybridStage):
+  """Latent attention (latents of 512, some layers reading another's), 4
+  residual streams, a dense first feed-forward and mixtures behind it: 4 of 64
+  experts per token and a shared one, together as wide as the dense one."""
+
+  EXPERTS, TOP, RANK, STREAMS = 64, 4, 512, 4
+
+  def make_config(self, W, F, H):
+    mixer = {'heads': H, 'dim': 128, 'vdim': 128, 'q_rank': W // 2,
+             'kv_rank': self.RANK, 'mask': {'size': self.WINDOW},
+             'scale': 128 ** -0.5}
+    moe = {'kind': 'moe', 'router': {'experts': self.EXPERTS, 'top': self.TOP},
+           'expert': {'ff': F // 8, 'limit': 7.0},
+           'shared': {'ff': F // 2, 'limit': 7.0}}
+    layers = []
+    for i in range(self.LAYERS):
+      m = dict(mixer, kv_from=i // 4 * 4 + 1) if i % 4 > 1 else mixer
+      layers.append({'type': 'latent_attention', 'mixer': m,
+                     'mlp': moe if i else {'kind': 'dense', 'ff': F}})
+    return {'architecture': 'Nutizen', 'width': W, 'vocab': self.VOCAB,
+            'norm': {'eps': 1e-6}, 'embedding': {'scale': 1.0},
+            'streams': self.STREAMS, 'layers': layers}
+
+  def kernels(self):
+    from t5x_amd import _lib, ops
+    torch, H, W, D = self.torch, self.H, self.W, 128
+    rank, q_rank, n = self.RANK, W // 2, self.STREAMS
+    out = []
+    for mode in ('prefill', 'decode'):
+      S, T = (self.B, self.T) if mode == 'prefill' else (self.R, 1)
+      start, M = (0, S * T) if mode == 'prefill' else (self.T, S)
+      tokens = self.prompts(S, T)
+      portions = self.hybrid.Portions(
+          [(s, start, tokens[s]) for s in range(S)], [], 'cuda',
+          self.cfg.span_windows())
+      bufs = self.hybrid._Buffers(self.w, M, S, 'cuda')
+      cache = self.module.init_cache(S, self.T + 64, portion=T)
+      bufs.proj.normal_()
+      bufs.h.normal_()
+      layer, a = bufs.layers[1], bufs.layers[1].latent
+      a.dtype, a.proj, a.ld_proj = _lib.BF16, bufs.proj.data_ptr(), layer.proj_n
+      ring = cache['decoder']['run_1']['latent_ring']
+      a.latent_ring, a.ring = ring.data_ptr(), ring.shape[1]
+      a.out, a.ld_out = layer.mix_rows, layer.out_k
+      a.workspace = bufs.workspace.data_ptr()
+      sec = time_kernel(torch, lambda: ops.latent_attention(
+          a, portions.ragged), 10)
+      if mode == 'prefill':
+        seen = np.minimum(np.arange(self.T) + 1, self.WINDOW).sum()
+        flops = 4.0 * D * S * H * seen + 2.0 * M * H * D * (q_rank + 2 * rank)
+        out.append(rate_entry('latent attention (prefill)', sec, flops, 'TFLOP/s'))
+      else:
+        # the latents once, the three maps once, activations
+        bytes_ = 2.0 * (S * self.WINDOW * rank + H * D * (q_rank + 2 * rank) +
+                        M * H * (2 * D + 4 * rank))
+        out.append(rate_entry('latent attention (decode)', sec, bytes_, 'GB/s'))
+      e, top = layer.experts, self.TOP
+      r = _lib.Route()
+      r.experts, r.top, r.table = e.n, e.top, e.table
+      r.tile_rows = _lib.load().t5d_grouped_tile_rows(_lib.BF16, M * top, e.n)
+      r.max_tiles = _lib.load().t5d_route_max_tiles(M * top, e.n, r.tile_rows)
+      r.tiles, r.token_of, r.entry_of = e.tiles, e.token_of, e.entry_of
+      route = lambda: _lib.call('t5d_route_tokens', _lib.stream_handle(),
+                                portions.ragged.tokens, M, self.VOCAB, r, 1)
+      sec = time_kernel(torch, route, 10)
+      out.append(rate_entry(f'route ({mode})', sec, 12.0 * M * top, 'GB/s'))
+      table = self.params['l1.mlp.table'].cpu().numpy()
+      used = len(np.unique(table[tokens.ravel()]))
+      F = e.F
+      for name, K, N, A, lda, rows, C, ldc, w, stride, epi in (
+          ('gated experts', W, 2 * F, bufs.h.data_ptr(), self.w.ld, e.token_of,
+           e.rows, F, e.glu, e.glu_stride, ops.EPI_CLAMPED_GLU),
+          ('experts', F, W, e.rows, F, None, e.out, self.w.ld, e.down,
+           e.down_stride, ops.EPI_NONE)):
+        d = _lib.GroupedDense()
+        d.dtype, d.M, d.K, d.N, d.epilogue = _lib.BF16, M, K, N, epi
+        d.A, d.lda, d.W, d.w_stride = A, lda, w, stride
+        d.C, d.ldc, d.n_store = C, ldc, N
+        d.glu_limit, d.glu_alpha, d.glu_add = e.limit, e.alpha, e.add
+        d.tiles, d.rows, d.n_tiles, d.tile_rows = (e.tiles, rows, r.max_tiles,
+                                                   r.tile_rows)
+        sec = time_kernel(torch, lambda: _lib.call(
+            't5d_grouped_dense_run', _lib.stream_handle(), d), 10)
+        out.append(dense_entry(
+            name, mode, sec, 2.0 * M * top * K * N,
+            2.0 * used * K * N + 2.0 * M * top * (K + ldc)))
+      x = torch.randn((M, n, W), device='cuda')
+      y = torch.randn((M, W), device='cuda').to(torch.bfloat16)
+      f = lambda *s: torch.randn(s, device='cuda')
+      mix, spread, collect, norm = f(n, n) / 4, f(n), f(n), f(W)
+      sec = time_kernel(torch, lambda: ops.hyper_norm(
+          x, W, torch.bfloat16, y=y, mix=mix, spread=spread, collect=collect,
+          norm=norm), 10)
+      out.append(rate_entry(f'hyper_norm ({mode})', sec,
+                            M * W * (8.0 * n + 4.0), 'GB/s'))
+    return out
+
+
+def main_latent(args):
+  """Prefill and decode of a model with latent attention beside a hybrid model of
+  attention layers of equal width, depth and active feed-forward.  A step is one
+  prefill of the batch; `value` is its rate."""
+  size, batch = args.hybrid_size, args.hybrid_batch or 4
+  steps = min(args.steps, 10)
+  w = LatentStage(size, batch, 4096, 64, args.seed)
+  kernels = w.kernels()
+  prefill, decode = w.prefill(steps), w.decode(64)
+  M = w.B * w.T
+  del w.params, w.module, w.w
+  like = AttentionStage(size, batch, 4096, 64, args.seed)
+  like_kernels = like.kernels()
+  like_prefill, like_decode = like.prefill(steps), like.decode(64)
+  best = max((k for k in kernels if 'prefill' in k['kernel']),
+             key=lambda k: k['us'])
+  out = {
+      'metric': 'prefilled tokens/sec, decoder-only model with latent attention '
+                f'({size}) on 1 GPU',
+      'value': round(M / prefill, 1), 'unit': 'tokens/s', 'n_gpus': 1,
+      'steps': steps, 'warmup': 1, 'ms_per_step': round(prefill * 1e3, 4),
+      'higher_is_better': True, 'scaling': 'weak', 'vs_baseline': None,
+      'dtype': 'bf16', 'data': 'synthetic',
+      'config': {
+          'workload': f'{w.LAYERS} layers of width {w.W}, {w.STREAMS} streams, '
+                      f'latents of {w.RANK}, {w.H} heads of 128 over {w.WINDOW} '
+                      f'positions, feed-forward {w.F} / {w.TOP} of {w.EXPERTS} '
+                      f'experts of {w.F // 8} and a shared one of {w.F // 2}; '
+                      f'{w.B} prompts of {w.T} tokens; decode of {w.R} rows at '
+                      f'position {w.T}',
+          'name': size, 'stage': 'latent',
+          'decode': {'rows': w.R, 'ms_per_step': round(decode * 1e3, 4),
+                     'tokens_per_s': round(w.R / decode, 1)},
+          'attention_model': {
+              'what': f'{w.LAYERS} windowed attention layers of the hybrid '
+                      f'family, {like.H} heads over {max(1, like.H // 4)} '
+                      f'key/value heads, feed-forward {like.F}',
+              'prefill_tokens_per_s': round(M / like_prefill, 1),
+              'decode_ms_per_step': round(like_decode * 1e3, 4),
+              'decode_tokens_per_s': round(like.R / like_decode, 1),
+              'kernels': like_kernels},
+          'kernels': kernels},
+      'roofline': {'kernel': best['kernel'],
+                   'bound': 'mfma' if best['unit'] == 'TFLOP/s' else 'hbm',
+                   'achieved': best['achieved'], 'peak': best['peak'],
+                   'unit': best['unit'], 'frac': best['frac'],
+                   'traffic': None, 'avg_launch_us': best['us']},
+  }
+  print(json.dumps(out))
 
 
 def main_hybrid(args):
@@ -1253,6 +1458,8 @@ def main():
     return main_dense(args)
   if args.stage == 'hybrid':
     return main_hybrid(args)
+  if args.stage == 'latent':
+    return main_latent(args)
   if args.stage == 'memory':
     return main_memory(args)
   w = Workload(args.config, args.seed, args.lanes)

@@ -85,30 +85,40 @@ def spread(streams, mix, out, y):
   return np.einsum('st,snw->tnw', mix, streams) + out[:, None, None] * y
 
 
+def connections(w, n, q):
+  """Hyper-connections (in, mix, out) of branch q of the layer named n; without
+  any a branch takes the one stream and adds to it."""
+  if n + f'hc{q}.in' not in w:
+    return np.ones(1), np.eye(1), np.ones(1)
+  return tuple(w[n + f'hc{q}.{k}'] for k in ('in', 'mix', 'out'))
+
+
 def forward(cfg, w, tokens, trace=None):
   """Logits [T, vocab] of one sequence; `trace` (a list) receives the sum of the
   residual streams after every layer."""
   w = {k: np.asarray(v, np.float64) for k, v in w.items()}
   eps, tokens = cfg['norm']['eps'], np.asarray(tokens)
   x = w['embed'][tokens] * cfg['embedding']['scale']
-  x = np.repeat(x[None], cfg['streams'], axis=0)
+  x = np.repeat(x[None], cfg.get('streams') or 1, axis=0)
   latents = {}
   for i, layer in enumerate(cfg['layers']):
     n, m, mlp = f'l{i}.', layer['mixer'], layer.get('mlp')
     mix = lambda name, n=n: w[n + 'mix.' + name]
     ff = lambda name, n=n: w[n + 'mlp.' + name]
-    h = rms(collect(x, w[n + 'hc1.in']), eps) * w[n + 'norm1']
+    h_in, h_mix, h_out = connections(w, n, 1)
+    h = rms(collect(x, h_in), eps) * w[n + 'norm1']
     src = m.get('kv_from')
     latents[i] = latent(h, mix, eps) if src is None else latents[src]
     y = latent_attention(h, latents[i], m, mix, eps)
-    x = spread(x, w[n + 'hc1.mix'], w[n + 'hc1.out'], y)
+    x = spread(x, h_mix, h_out, y)
     if mlp is not None:
-      h = rms(collect(x, w[n + 'hc2.in']), eps) * w[n + 'norm2']
+      h_in, h_mix, h_out = connections(w, n, 2)
+      h = rms(collect(x, h_in), eps) * w[n + 'norm2']
       if mlp['kind'] == 'dense':
         y = silu_glu(h, ff)
       else:
         y = table_experts(h, tokens, mlp, ff)
-      x = spread(x, w[n + 'hc2.mix'], w[n + 'hc2.out'], y)
+      x = spread(x, h_mix, h_out, y)
     if trace is not None:
       trace.append(x.sum(axis=0))
   return rms(x.sum(axis=0), eps) * w['final.norm'] @ w['head'].T

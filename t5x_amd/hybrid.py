@@ -556,6 +556,34 @@ MIXERS = {'attention': _AttentionMixer, 'gla': _GatedLinearMixer,
 # ------------------------------------------------------------------------------
 
 
+class Packer:
+  """Packs input-major float32 kernels for the dense layers and keeps the packed
+  tensors in the list `kept`."""
+
+  def __init__(self, act_dtype, kept):
+    self.act_dtype, self.kept = act_dtype, kept
+
+  def _data(self, kernel, gate):
+    act = self.act_dtype
+    return ops.pack_weight(kernel, act, act, gate_kernel=gate).data
+
+  def __call__(self, kernel, gate=None):
+    self.kept.append(self._data(kernel, gate))
+    return self.kept[-1].data_ptr()
+
+  def many(self, kernels, gates=None):
+    """Kernels of one shape one after the other -> (address, bytes of each)."""
+    gates = gates or [None] * len(kernels)
+    out = None
+    for i, (kernel, gate) in enumerate(zip(kernels, gates)):
+      data = self._data(kernel, gate)
+      if out is None:
+        out = data.new_empty((len(kernels),) + tuple(data.shape))
+      out[i] = data
+    self.kept.append(out)
+    return out.data_ptr(), out[0].numel() * out.element_size()
+
+
 class HybridWeights:
   """The parameters of a model, cast and packed once on the device, and the
   t5d_hybrid_layer descriptions that name them."""
@@ -581,25 +609,7 @@ class HybridWeights:
       self._kept.append(t)
       return t.data_ptr()
 
-    def pack(kernel, gate=None):
-      w = ops.pack_weight(kernel, act, act, gate_kernel=gate)
-      self._kept.append(w.data)
-      return w.data.data_ptr()
-
-    def pack_many(kernels, gates=None):
-      """Kernels of one shape one after the other -> (address, bytes of each)."""
-      first = out = None
-      for i, kernel in enumerate(kernels):
-        gate = gates[i] if gates is not None else None
-        data = ops.pack_weight(kernel, act, act, gate_kernel=gate).data
-        if out is None:
-          first, out = data, torch.empty((len(kernels),) + tuple(data.shape),
-                                         dtype=data.dtype, device=data.device)
-        out[i] = data
-      self._kept.append(out)
-      return out.data_ptr(), first.numel() * first.element_size()
-
-    pack.many = pack_many
+    pack = Packer(act, self._kept)
 
     def padded(name, k, n):
       """Transposed to input-major and padded to [k, n]."""
@@ -640,7 +650,7 @@ class HybridWeights:
       layer.out_k = _pad(m.heads * m.vdim, 64)
       layer.out = pack(padded(f'l{i}.mix.o', layer.out_k, ld))
 
-      def unit(prefix, ff, pack=pack):
+      def unit(prefix, ff):
         F = _pad(ff, 64)
         return (F, pack(padded(prefix + 'gate', ld, F),
                         padded(prefix + 'up', ld, F)),
@@ -880,15 +890,17 @@ class HybridDecoder(network.DecodeContexts):
   # -- caches -----------------------------------------------------------------
   def init_cache(self, rows: int, max_len: int, portion: Optional[int] = None):
     """A cache tree for `rows` slots of up to `max_len` positions: one scope per
-    layer run, and cache_index [rows] = positions each slot holds.  portion: the
-    longest portion it will be fed (max_portion)."""
+    layer run that keeps something, and cache_index [rows] = positions each slot
+    holds.  portion: the longest portion it will be fed (max_portion)."""
     cfg, dev = self.config, self._dev()
     ring_len = self._ring_len(max_len, portion)
     act = _ACT[cfg.dtype]
     tree = {}
     for r, (i, _) in enumerate(cfg.runs()):
       m = cfg.layers[i].mixer
-      tree[f'run_{r}'] = MIXERS[m.type].cache(m, rows, ring_len, act, dev)
+      leaves = MIXERS[m.type].cache(m, rows, ring_len, act, dev)
+      if leaves:  # (nothing where another layer's are read)
+        tree[f'run_{r}'] = leaves
     return {'decoder': tree,
             'cache_index': torch.zeros((rows,), dtype=torch.int32, device=dev)}
 

@@ -865,3 +865,114 @@ def recurrence(desc, ragged, variant=0):
   """t5d_recurrence_run over filled-in descriptions (_lib.Recurrence,
   _lib.Ragged)."""
   _lib.call('t5d_recurrence_run', _s(), desc, ragged, int(variant))
+
+
+def latent_attention(desc, ragged, variant=0):
+  """t5d_latent_attention_run over filled-in descriptions (_lib.LatentAttention,
+  _lib.Ragged)."""
+  _lib.call('t5d_latent_attention_run', _s(), desc, ragged, int(variant))
+
+
+def embed_streams(table, ids, scale, width, streams):
+  """float32 [M, streams, ld]: every stream of a token its scaled table row
+  (columns beyond `width` zero)."""
+  _chk(table, 'table', ndim=2)
+  _chk(ids, 'ids', torch.int32, 1)
+  V, ld = table.shape
+  out = torch.empty((ids.shape[0], streams, ld), dtype=torch.float32,
+                    device=table.device)
+  _lib.call('t5d_embed_streams', _s(), _lib.dtype_code(table.dtype),
+            table.data_ptr(), ids.data_ptr(), float(scale), out.data_ptr(),
+            ids.shape[0], int(width), ld, int(streams), V)
+  return out
+
+
+def hyper_norm(x, width, dtype, y=None, y_gate=None, parts=None, part_row=None,
+               part_weight=1.0, mix=None, spread=None, collect=None, norm=None,
+               rows=None, want_sum=False, gate_w=None, eps=1e-6):
+  """The row kernel over several float32 streams x [M, streams, ld]
+  (t5d_hyper_norm): adds the branch y + parts and mixes the streams in place, and
+  returns (normed weighted sum as dtype, its float32 sum, sigmoid gate), None where
+  not asked for."""
+  _chk(x, 'x', torch.float32, 3)
+  M, n, ld = x.shape
+  for t, name, shape in (
+      (y_gate, 'y_gate', (M,)), (mix, 'mix', (n, n)), (spread, 'spread', (n,)),
+      (collect, 'collect', (n,)), (norm, 'norm', (width,)),
+      (gate_w, 'gate_w', (width,))):
+    if t is not None:
+      _chk(t, name, torch.float32, len(shape))
+      if tuple(t.shape) != shape:
+        raise ValueError(f'{name} must be {shape}')
+  for t, name, rows_ in ((y, 'y', M), (parts, 'parts', None)):
+    if t is not None:
+      _chk(t, name, dtype, 2)
+      if t.shape[1] != ld or (rows_ is not None and t.shape[0] != rows_):
+        raise ValueError(f'{name} is {tuple(t.shape)}')
+  a = _lib.HyperNorm()
+  a.dtype, a.d, a.ld, a.streams = _lib.dtype_code(dtype), int(width), ld, n
+  if parts is not None:
+    _chk(part_row, 'part_row', torch.int32, 2)
+    if part_row.shape[0] != M or int(part_row.max()) >= parts.shape[0]:
+      raise ValueError('part_row must be [M, top] rows of parts')
+    a.top = part_row.shape[1]
+  count = M
+  if rows is not None:
+    _chk(rows, 'rows', torch.int32, 1)
+    count = rows.shape[0]
+  make = lambda *shape, dtype=torch.float32: torch.empty(shape, dtype=dtype,
+                                                         device=x.device)
+  out = make(count, ld, dtype=dtype) if norm is not None else None
+  total = make(count, ld) if want_sum else None
+  gate = make(count) if gate_w is not None else None
+  a.eps, a.part_weight = float(eps), float(part_weight)
+  for name, t in (('y', y), ('parts', parts), ('y_gate', y_gate),
+                  ('part_row', part_row), ('mix', mix), ('spread', spread),
+                  ('collect', collect), ('x', x), ('norm', norm), ('out', out),
+                  ('rows', rows), ('sum', total), ('gate_w', gate_w),
+                  ('gate_out', gate)):
+    setattr(a, name, _lib.ptr(t))
+  _lib.call('t5d_hyper_norm_run', _s(), a, count)
+  return out, total, gate
+
+
+def route_tokens(tokens, table, experts, dtype, tile_rows=None):
+  """Tokens [M] sorted by the experts that `table` [V, top] lists for their ids:
+  (tiles [n, 4], token_of [M top], entry_of [M, top], rows per tile)."""
+  _chk(tokens, 'tokens', torch.int32, 1)
+  _chk(table, 'table', torch.int32, 2)
+  lib, M, (V, top) = _lib.load(), tokens.shape[0], table.shape
+  r = _lib.Route()
+  r.experts, r.top = int(experts), top
+  r.tile_rows = tile_rows or lib.t5d_grouped_tile_rows(_lib.dtype_code(dtype),
+                                                       M * top, experts)
+  r.max_tiles = lib.t5d_route_max_tiles(M * top, experts, r.tile_rows)
+  ints = lambda *shape: torch.empty(shape, dtype=torch.int32,
+                                    device=tokens.device)
+  tiles, token_of, entry_of = ints(r.max_tiles, 4), ints(M * top), ints(M, top)
+  r.table, r.tiles = table.data_ptr(), tiles.data_ptr()
+  r.token_of, r.entry_of = token_of.data_ptr(), entry_of.data_ptr()
+  _lib.call('t5d_route_tokens', _s(), tokens.data_ptr(), M, V, r, 1)
+  return tiles, token_of, entry_of, r.tile_rows
+
+
+def grouped_dense(a, kernels, out, tiles=None, rows=None, tile_rows=0,
+                  groups=0, a_step=0, c_step=0, n_store=None, glu=None):
+  """Dense layers of one shape in one launch (t5d_grouped_dense).  kernels: a list
+  of PackedWeight of one shape; out [rows, columns] is written; tiles and rows as
+  route_tokens gives them, or groups of columns."""
+  w = kernels[0]
+  data = torch.stack([k.data for k in kernels])
+  d = _lib.GroupedDense()
+  d.dtype, d.M, d.K, d.N = _lib.dtype_code(a.dtype), a.shape[0], w.K, w.N
+  d.epilogue = EPI_NONE if glu is None else EPI_CLAMPED_GLU
+  d.A, d.lda, d.W = a.data_ptr(), a.stride(0), data.data_ptr()
+  d.w_stride = w.data.numel() * w.data.element_size()
+  d.C, d.ldc = out.data_ptr(), out.stride(0)
+  d.n_store = n_store or w.N
+  d.glu_limit, d.glu_alpha, d.glu_add = glu or (0.0, 0.0, 0.0)
+  d.tiles, d.rows = _lib.ptr(tiles), _lib.ptr(rows)
+  d.n_tiles, d.tile_rows = (0 if tiles is None else tiles.shape[0]), tile_rows
+  d.groups, d.a_step, d.c_step = groups, a_step, c_step
+  _lib.call('t5d_grouped_dense_run', _s(), d)
+  return out

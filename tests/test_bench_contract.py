@@ -32,6 +32,7 @@ def test_more_than_one_gpu_is_refused_with_a_message():
     ('--stage', 'dense'),
     ('--stage', 'memory'),
     ('--stage', 'hybrid', '--hybrid-size', 'base', '--hybrid-batch', '1'),
+    ('--stage', 'latent', '--hybrid-size', 'base', '--hybrid-batch', '1'),
 ])
 def test_short_stages_print_one_json_line(flags):
   r = run_bench(*flags)

@@ -589,7 +589,7 @@ def test_logits_whole_in_portions_and_token_by_token(name, dtype):
   cfg, params, module = build(name, dtype)
   rs = np.random.RandomState(5)
   tokens = rs.randint(0, cfg['vocab'], 150).tolist()
-  want = oracle.forward(cfg, params, tokens)
+  want = cases.forward(cfg, params, tokens)
   live = sequences.Sequences(module, params, 2, 200)
   whole = feed(live, 'a', tokens, [])
   assert close(whole, want, dtype)
@@ -601,12 +601,13 @@ def test_logits_whole_in_portions_and_token_by_token(name, dtype):
 
 
 @pytest.mark.parametrize('dtype', ['float32', 'bfloat16'])
-def test_residual_stream_after_every_layer_run(dtype):
+@pytest.mark.parametrize('name', ['all', 'latent', 'latent_plain'])
+def test_residual_stream_after_every_layer_run(name, dtype):
   from t5x_amd import sequences
-  cfg, params, module = build('all', dtype)
+  cfg, params, module = build(name, dtype)
   tokens = np.random.RandomState(6).randint(0, cfg['vocab'], 20).tolist()
   want, got = [], []
-  oracle.forward(cfg, params, tokens, want)
+  cases.forward(cfg, params, tokens, want)
   live = sequences.Sequences(module, params, 1, 32)
   live.step([('a', tokens, [])], trace=got)
   assert got[0].shape == (len(want), 20, cfg['width'])
@@ -615,7 +616,7 @@ def test_residual_stream_after_every_layer_run(dtype):
 
 
 @pytest.mark.parametrize('dtype', ['float32', 'bfloat16'])
-@pytest.mark.parametrize('name', ['all', 'all_looped', 'odd_values'])
+@pytest.mark.parametrize('name', ['all', 'all_looped', 'odd_values'] + cases.LATENT)
 def test_small_rings_wrap_in_long_requests(name, dtype):
   """Rings as small as the windows allow, reused slots, a request far longer than
   every ring."""
@@ -625,21 +626,22 @@ def test_small_rings_wrap_in_long_requests(name, dtype):
   live = sequences.Sequences(module, params, 1, 700)
   for n, cuts in ((700, [300, 302, 304]), (31, [30]), (260, range(60, 260))):
     tokens = rs.randint(0, cfg['vocab'], n).tolist()
-    want = oracle.forward(cfg, params, tokens)
+    want = cases.forward(cfg, params, tokens)
     assert close(feed(live, n, tokens, cuts), want, dtype), n
 
 
 @pytest.mark.parametrize('dtype', ['float32', 'bfloat16'])
-def test_mixed_batches_match_each_alone(dtype):
+@pytest.mark.parametrize('name', ['all', 'latent', 'latent_one_stream'])
+def test_mixed_batches_match_each_alone(name, dtype):
   """Prompts, portions and single tokens of unequal requests in one step, slots
   given back and taken again in between."""
   from t5x_amd import sequences
-  cfg, params, module = build('all', dtype, max_tokens=90)
+  cfg, params, module = build(name, dtype, max_tokens=90)
   rs = np.random.RandomState(8)
   live = sequences.Sequences(module, params, 3, 128)
   req = {n: rs.randint(0, cfg['vocab'], l).tolist() for n, l in
          (('a', 100), ('b', 41), ('c', 1), ('d', 77), ('e', 23))}
-  want = {n: oracle.forward(cfg, params, t) for n, t in req.items()}
+  want = {n: cases.forward(cfg, params, t) for n, t in req.items()}
   at = dict.fromkeys(req, 0)
   plan = [{'a': 60, 'b': 1, 'c': 1}, {'a': 1, 'b': 2, 'd': 70}, {'d': 7, 'b': 37},
           {'b': 1, 'a': 2}, {'e': 20, 'a': 30}, {'e': 1, 'a': 1}, {'a': 6, 'e': 2}]
@@ -663,7 +665,7 @@ def test_wanted_places_come_in_the_order_asked_for():
   tokens = list(range(20))
   live = sequences.Sequences(module, params, 2, 32)
   got = host(live.step([('a', tokens, [19, 0, 7, 7]), ('b', tokens[:3], [1])]))
-  want = oracle.forward(cfg, params, tokens)
+  want = cases.forward(cfg, params, tokens)
   assert err(got, want[[19, 0, 7, 7, 1]]).max() < 2e-5
 
 
@@ -673,7 +675,7 @@ def test_wanted_places_come_in_the_order_asked_for():
 def greedy(cfg, params, prompt, n):
   tokens = list(prompt)
   for _ in range(n):
-    tokens.append(int(np.argmax(oracle.forward(cfg, params, tokens)[-1])))
+    tokens.append(int(np.argmax(cases.forward(cfg, params, tokens)[-1])))
   return tokens[len(prompt):]
 
 
@@ -685,7 +687,7 @@ def model_for(name, dtype='float32', eos=-1, **kw):
       module, models.Vocabulary(eos), decode_fn=kw.pop('decode_fn', fn))
 
 
-@pytest.mark.parametrize('name', ['all', 'no_loop'])
+@pytest.mark.parametrize('name', ['all', 'no_loop'] + cases.LATENT)
 def test_greedy_generation_equals_the_oracle(name):
   """Unequal prompts in batches, several in flight, float32: exact tokens."""
   cfg, params, model = model_for(name)
@@ -726,12 +728,13 @@ def test_generation_stops_at_the_end_token():
   assert list(stopping.generate(params, [prompt], 14))[0] == cut
 
 
-def test_replayed_graph_equals_the_step_by_step_loop():
+@pytest.mark.parametrize('name', ['all', 'latent'])
+def test_replayed_graph_equals_the_step_by_step_loop(name):
   """The captured loop against the loop that calls the step function every
   iteration (a state callback keeps it off the graph), bit for bit, twice."""
   from t5x_amd import decoding, models
   for dtype in ('float32', 'bfloat16'):
-    cfg, params, model = model_for('all', dtype)
+    cfg, params, model = model_for(name, dtype)
     rs = np.random.RandomState(10)
     L, lens = 40, [7, 20, 1]
     batch = {'decoder_input_tokens': rs.randint(1, cfg['vocab'], (3, L)),
@@ -761,9 +764,10 @@ def test_replayed_graph_equals_the_step_by_step_loop():
           np.broadcast_to(batch['decoder_input_tokens'][r, 1:n], (2, n - 1)))
 
 
-def test_beam_search_equals_the_oracle():
+@pytest.mark.parametrize('name', ['no_loop', 'latent'])
+def test_beam_search_equals_the_oracle(name):
   from t5x_amd import decoding
-  cfg, params, model = model_for('no_loop', eos=1,
+  cfg, params, model = model_for(name, eos=1,
                                  decode_fn=decoding.beam_search)
   rs = np.random.RandomState(11)
   B, K, L, lens = 2, 3, 12, np.array([6, 3])
@@ -783,7 +787,7 @@ def test_beam_search_equals_the_oracle():
     logits = np.zeros((len(h), cfg['vocab']), np.float32)
     for r in range(len(h)):
       h[r, 0, at[r]] = state.cur_token[r, 0]
-      logits[r] = oracle.forward(cfg, params, h[r, 0, :at[r] + 1])[-1]
+      logits[r] = cases.forward(cfg, params, h[r, 0, :at[r] + 1])[-1]
     return logits, {'history': h,
                     'cache_index': state.cache['cache_index'] + 1}
 
@@ -795,13 +799,15 @@ def test_beam_search_equals_the_oracle():
 
 
 @pytest.mark.parametrize('dtype', ['float32', 'bfloat16'])
-def test_saved_model_through_the_commands(tmp_path, monkeypatch, capsys, dtype):
+@pytest.mark.parametrize('name', ['all', 'latent'])
+def test_saved_model_through_the_commands(tmp_path, monkeypatch, capsys, name,
+                                          dtype):
   from t5x_amd import generate, trace_replay
-  cfg = cases.CONFIGS['all']
+  cfg = cases.CONFIGS[name]
   params = cases.random_params(cfg, seed=3)
   cases.save_model(tmp_path, cfg, params)
   tokens = np.random.RandomState(12).randint(0, cfg['vocab'], 30).tolist()
-  want = oracle.forward(cfg, params, tokens)
+  want = cases.forward(cfg, params, tokens)
   steps = [{'step': 0, 'entries': [{'id': 'a', 'tokens': tokens[:21],
                                     'want': [0, 20]}], 'end': []},
            {'step': 1, 'entries': [{'id': 'a', 'tokens': tokens[21:22],
