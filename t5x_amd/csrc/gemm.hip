@@ -45,7 +45,8 @@ gemm_mfma_kernel(Args g) {
     T5D_GATED(g.gate);
     const char* w = reinterpret_cast<const char*>(g.W);
     bf16_t* c = reinterpret_cast<bf16_t*>(g.C);
-    if (!enter_group(g.grp, g.A, g.lda, w, c, gated(g) ? g.N >> 1 : g.ldc, g.M))
+    if (!enter_group(g.grp, blockIdx.y, g.A, g.lda, w, c,
+                     gated(g) ? g.N >> 1 : g.ldc, g.M))
       return;
     g.W = w;
     g.C = c;
@@ -693,7 +694,7 @@ gemm_f32_kernel(const float* __restrict__ A, const float* __restrict__ W,
   const int n = blockIdx.x * kF32Cols + c;
   int m0 = blockIdx.y * MB;
   if constexpr (GROUPED) {
-    if (!enter_group(gr.grp, A, lda, W, C, geglu ? F : gr.ldc, M)) return;
+    if (!enter_group(gr.grp, blockIdx.y, A, lda, W, C, geglu ? F : gr.ldc, M)) return;
     m0 = gr.grp.tiles != nullptr ? 0 : blockIdx.z * MB;
   }
   const int ldc = geglu ? F : GROUPED ? gr.ldc : N;
@@ -1317,9 +1318,10 @@ extern "C" int t5d_grouped_dense_run(void* stream, const t5d_grouped_dense* a) {
                 "t5d_grouped_dense_run: tiles of %d rows", a->tile_rows);
     hipLaunchKernelGGL((gemm_mfma_kernel<4, 2, bf16_t, 0, GroupedArgs>),
                        dim3(gx, gy), dim3(256), 0, s, g);
-  } else if (a->M <= 16) {
+  } else if (a->M <= 64) {
+    g.m_parts = (a->M + 15) / 16;
     hipLaunchKernelGGL((gemm_mfma_kernel<1, 2, bf16_t, 0, GroupedArgs>),
-                       dim3(gx, gy), dim3(256), 0, s, g);
+                       dim3(gx * g.m_parts, gy), dim3(256), 0, s, g);
   } else {
     g.m_parts = (a->M + 63) / 64;
     hipLaunchKernelGGL((gemm_mfma_kernel<4, 2, bf16_t, 0, GroupedArgs>),

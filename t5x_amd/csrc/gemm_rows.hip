@@ -77,6 +77,7 @@ struct RowsGemmArgs {
   float glu_limit, glu_alpha, glu_add;  // T5D_EPI_CLAMPED_GLU
   const int32_t* gate;     // GROUPED kernels only, with the next
   GroupTiles grp;
+  int n_tiles;
 };
 
 __device__ __forceinline__ uint2 pack4(float a, float b, float c, float d) {
@@ -417,7 +418,7 @@ typedef __attribute__((address_space(1))) const void* glb_ptr_t;
 // wavefronts of 128 x 128 (accumulators in the accumulation registers) lasts
 // 257 us: with one wavefront per SIMD nothing covers the operand reads from
 // LDS.
-// GROUPED: see GroupTiles (gemm_tiles.h); blockIdx.y is the tile of rows.
+// GROUPED: see GroupTiles (gemm_tiles.h).
 template <bool SWAP, int NT, int WN, int DENSE = 0, bool GROUPED = false>
 __global__ void __launch_bounds__(128 * WN, WN == 2 ? 2 : 1)
 rows_gemm_direct_kernel(RowsGemmArgs g) {
@@ -444,16 +445,27 @@ rows_gemm_direct_kernel(RowsGemmArgs g) {
   __shared__ uint4 s_t0[TILES][64];
   __shared__ uint4 s_t1[TILES][64];
   __shared__ uint4 s_t2[TILES][64];
+  int group_n_blk = 0;
   if constexpr (GROUPED) {
     T5D_GATED(g.gate);
-    if (!enter_group(g.grp, g.A, g.lda, g.W, g.C, DENSE == 1 ? g.N >> 1 : g.N, g.M))
+    // 4 consecutive tiles of rows, most of them of one group, on one XCD, all
+    // columns of a tile in a row: rows and kernels come from that XCD's L2.
+    const int n_blocks = ((g.N >> 4) + BN / 16 - 1) / (BN / 16);
+    const int xcd = blockIdx.x & 7, slot = blockIdx.x >> 3;
+    const int t = slot / n_blocks;
+    const int tile = ((t >> 2) * 8 + xcd) * 4 + (t & 3);
+    if (tile >= g.n_tiles ||
+        !enter_group(g.grp, tile, g.A, g.lda, g.W, g.C, DENSE == 1 ? g.N >> 1 : g.N,
+                     g.M))
       return;
+    group_n_blk = slot % n_blocks;
   }
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int l16 = lane & 15, gq = lane >> 4;
   const int m_blocks = (g.M + kRowsBM - 1) / kRowsBM;
-  const int m_blk = blockIdx.x % m_blocks, n_blk = blockIdx.x / m_blocks;
+  const int m_blk = GROUPED ? 0 : blockIdx.x % m_blocks;
+  const int n_blk = GROUPED ? group_n_blk : blockIdx.x / m_blocks;
   const int wm = wave / WN, wn = wave % WN;
   const int m0 = m_blk * kRowsBM + wm * (16 * MT);
   const int nt0 = n_blk * (BN / 16) + wn * NT;
@@ -721,7 +733,7 @@ extern "C" int t5d_gemm_rows_tiled(void* stream, int w_dtype, const void* A,
   g.E = E; g.Ep = Ep; g.H = H;
   g.lda = K; g.C32 = nullptr; g.ldc = g.n_store = N;
   g.glu_limit = g.glu_alpha = g.glu_add = 0.f;
-  g.gate = nullptr; g.grp = GroupTiles();
+  g.gate = nullptr; g.grp = GroupTiles(); g.n_tiles = 0;
   return launch_rows(as_stream(stream), w_dtype, g, tile);
 }
 
@@ -739,7 +751,7 @@ int t5d::launch_dense_rows(hipStream_t s, const void* A, int lda,
   g.epilogue = epilogue; g.layout = T5D_OUT_ROWS;
   g.E = g.Ep = g.H = 0;
   g.lda = lda; g.ldc = ldc; g.n_store = n_store;
-  g.gate = nullptr; g.grp = GroupTiles();
+  g.gate = nullptr; g.grp = GroupTiles(); g.n_tiles = 0;
   g.glu_limit = glu_limit; g.glu_alpha = glu_alpha; g.glu_add = glu_add;
   return launch_rows(s, T5D_BF16, g, 0);
 }
@@ -754,14 +766,28 @@ int t5d::launch_grouped_rows(hipStream_t s, const GroupedArgs& a, int n_tiles) {
   g.E = g.Ep = g.H = 0;
   g.lda = a.lda; g.ldc = a.ldc; g.n_store = a.n_store;
   g.glu_limit = a.glu_limit; g.glu_alpha = a.glu_alpha; g.glu_add = a.glu_add;
-  g.gate = a.gate; g.grp = a.grp;
-  const dim3 grid((g.N + kRowsBN - 1) / kRowsBN, n_tiles), block(256);
-  if (g.epilogue == T5D_EPI_CLAMPED_GLU)
-    hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2, 1, true>), grid,
-                       block, 0, s, g);
-  else
-    hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2, 0, true>), grid,
-                       block, 0, s, g);
+  g.gate = a.gate; g.grp = a.grp; g.n_tiles = n_tiles;
+  const unsigned t32 = (unsigned)(n_tiles + 31) / 32 * 32;
+  const unsigned n128 = (g.N + 127) / 128, n256 = (g.N + 255) / 256;
+  const bool glu = g.epilogue == T5D_EPI_CLAMPED_GLU;
+  // the 256 x 256 tile unless much of its last column block would be empty
+  if (n256 * 256 <= n128 * 128 + 64) {
+    const dim3 grid(t32 * n256), block(512);
+    if (glu)
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 4, 1, true>), grid,
+                         block, 0, s, g);
+    else
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 4, 0, true>), grid,
+                         block, 0, s, g);
+  } else {
+    const dim3 grid(t32 * n128), block(256);
+    if (glu)
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2, 1, true>), grid,
+                         block, 0, s, g);
+    else
+      hipLaunchKernelGGL((rows_gemm_direct_kernel<true, kRowsNT, 2, 0, true>), grid,
+                         block, 0, s, g);
+  }
   T5D_CHECK_LAUNCH("t5d_grouped_dense_run(rows)");
   return T5D_OK;
 }

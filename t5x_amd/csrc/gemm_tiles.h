@@ -88,12 +88,12 @@ __device__ __forceinline__ int stored_columns(const DenseArgs& g) {
   return g.n_store;
 }
 // What t5d_grouped_dense adds: one launch over many kernels of one shape, which
-// are w_stride bytes apart.  With tiles, workgroups with blockIdx.y = t work on
-// tile t = (group, first row, rows, -): up to a workgroup's height of consecutive
-// output rows that all take that group's kernel (group -1: nothing); row r of the
-// output comes from row rows[r] of A (rows null: from row r).  Without tiles group
-// blockIdx.y takes all M rows from column group * a_step of A to column
-// group * c_step of C.
+// are w_stride bytes apart.  With tiles, some workgroups (those with blockIdx.y =
+// t, unless said otherwise) work on tile t = (group, first row, rows, -): up to a
+// workgroup's height of consecutive output rows that all take that group's kernel
+// (group -1: nothing); row r of the output comes from row rows[r] of A (rows null:
+// from row r).  Without tiles group blockIdx.y takes all M rows from column
+// group * a_step of A to column group * c_step of C.
 struct GroupTiles {
   const int4* tiles;
   const int32_t* rows;
@@ -105,13 +105,13 @@ struct GroupedArgs : DenseArgs {
 };
 template <typename Args> struct IsGrouped { static constexpr bool value = false; };
 template <> struct IsGrouped<GroupedArgs> { static constexpr bool value = true; };
-// Points A, W, C (of elements of a_bytes, bytes, c_bytes), the row list and M at
-// this workgroup's group; false: there is nothing to do.
+// Points A, W, C, the row list and M at tile (or group) i; false: there is nothing
+// to do.
 template <typename AP, typename WP, typename CP>
-__device__ __forceinline__ bool enter_group(GroupTiles& grp, AP& A, int lda, WP& W,
-                                            CP& C, int ldc, int& M) {
+__device__ __forceinline__ bool enter_group(GroupTiles& grp, int i, AP& A, int lda,
+                                            WP& W, CP& C, int ldc, int& M) {
   if (grp.tiles != nullptr) {
-    const int4 t = grp.tiles[blockIdx.y];
+    const int4 t = grp.tiles[i];
     const int group = __builtin_amdgcn_readfirstlane(t.x);
     const int first = __builtin_amdgcn_readfirstlane(t.y);
     M = __builtin_amdgcn_readfirstlane(t.z);
@@ -121,9 +121,9 @@ __device__ __forceinline__ bool enter_group(GroupTiles& grp, AP& A, int lda, WP&
     W += (int64_t)group * grp.w_stride;
     C += (int64_t)first * ldc;
   } else {
-    A += (int64_t)blockIdx.y * grp.a_step;
-    W += (int64_t)blockIdx.y * grp.w_stride;
-    C += (int64_t)blockIdx.y * grp.c_step;
+    A += (int64_t)i * grp.a_step;
+    W += (int64_t)i * grp.w_stride;
+    C += (int64_t)i * grp.c_step;
   }
   return true;
 }

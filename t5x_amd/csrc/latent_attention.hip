@@ -26,7 +26,7 @@ struct LatentArgs {
   t5d_latent_attention a;
   t5d_ragged b;
   int HP, RP, QP, splits;
-  float* parts;  // [M, H, splits, RP + 2]
+  float* parts;  // [M, H, splits, RP + 4]: sums, maximum, sum of weights
   const int32_t* gate;
 };
 
@@ -125,7 +125,10 @@ latent_tile_kernel(LatentArgs g) {
   constexpr int RP = DT * 32, KB = 64, R = 16 * HG;
   constexpr int KS = RP + 8, VS = KB + 8, PS = KB + 8;  // LDS row strides
   constexpr int CT = RP / 16 / 4;                       // column tiles per wavefront
-  constexpr int PIECES = RP / 8 / 8;                    // pair pieces per thread
+  constexpr int LPR = RP / 8;                           // lanes on one position
+  constexpr int PPI = 64 / LPR;                         // positions per load
+  constexpr int QUADS = 4 / PPI;                        // 4 positions, per thread
+  static_assert(PPI >= 1 && PPI <= 4, "latents of 128, 256 or 512");
   __shared__ __align__(16) bf16_t s_k[KB * KS];         // [position][column]
   __shared__ __align__(16) bf16_t s_v[RP * VS];         // [column][position]
   __shared__ __align__(16) bf16_t s_p[2][R * PS];       // weights, remainders
@@ -174,34 +177,41 @@ latent_tile_kernel(LatentArgs g) {
   const int j_begin = (max(0, i_lo - W + 1) & ~(KB - 1)) + KB * part;
   const int j_step = KB * g.splits;
 
-  uint4 va[PIECES], vb[PIECES];
-  const int pair = threadIdx.x & 31, col = threadIdx.x >> 5;
+  // A thread loads 8 columns of 4 consecutive positions (whole positions per
+  // wavefront and load: consecutive memory), so the transposed copy takes 8 bytes
+  // per column.  Its 16-byte pieces (8 positions) are XOR-swizzled by the column.
+  uint4 lat[QUADS][4];
+  const int piece = lane % LPR;
+  const int quad0 = 4 * wave + lane / LPR;  // positions 4 quad ..
   auto fetch = [&](int jt) {
-    const bf16_t* c = ring + ((size_t)(jt % a.ring) + 2 * pair) * RP + 8 * col;
+    const bf16_t* c = ring + ((size_t)(jt % a.ring) + 4 * quad0) * RP + 8 * piece;
 #pragma unroll
-    for (int i = 0; i < PIECES; ++i) {
-      va[i] = *reinterpret_cast<const uint4*>(c + 64 * i);
-      vb[i] = *reinterpret_cast<const uint4*>(c + RP + 64 * i);
-    }
+    for (int i = 0; i < QUADS; ++i)
+#pragma unroll
+      for (int k = 0; k < 4; ++k)
+        lat[i][k] = *reinterpret_cast<const uint4*>(c + (4 * PPI * i + k) * RP);
   };
   if (j_begin <= i_hi) fetch(j_begin);
   for (int jt = j_begin; jt <= i_hi; jt += j_step) {
     __syncthreads();  // the previous tile has been read
 #pragma unroll
-    for (int i = 0; i < PIECES; ++i) {
-      const int c = 8 * (col + 8 * i);
-      *reinterpret_cast<uint4*>(s_k + (2 * pair) * KS + c) = va[i];
-      *reinterpret_cast<uint4*>(s_k + (2 * pair + 1) * KS + c) = vb[i];
-      // positions 2p and 2p + 1 of 8 columns: one word per column
-      uint32_t* dst = reinterpret_cast<uint32_t*>(s_v + (size_t)c * VS + 2 * pair);
-      auto put = [&](int e, uint32_t x, uint32_t y) {
-        dst[(2 * e) * (VS / 2)] = (x & 0xFFFFu) | (y << 16);
-        dst[(2 * e + 1) * (VS / 2)] = (x >> 16) | (y & 0xFFFF0000u);
+    for (int i = 0; i < QUADS; ++i) {
+      const int quad = quad0 + PPI * i;
+#pragma unroll
+      for (int k = 0; k < 4; ++k)
+        *reinterpret_cast<uint4*>(s_k + (4 * quad + k) * KS + 8 * piece) = lat[i][k];
+      bf16_t* dst = s_v + (size_t)(8 * piece) * VS +
+                    8 * ((quad >> 1) ^ ((piece >> 1) & 7)) + 4 * (quad & 1);
+      auto put = [&](int e, uint32_t p, uint32_t q, uint32_t r, uint32_t s) {
+        *reinterpret_cast<uint2*>(dst + (2 * e) * VS) =
+            make_uint2((p & 0xFFFFu) | (q << 16), (r & 0xFFFFu) | (s << 16));
+        *reinterpret_cast<uint2*>(dst + (2 * e + 1) * VS) = make_uint2(
+            (p >> 16) | (q & 0xFFFF0000u), (r >> 16) | (s & 0xFFFF0000u));
       };
-      put(0, va[i].x, vb[i].x);
-      put(1, va[i].y, vb[i].y);
-      put(2, va[i].z, vb[i].z);
-      put(3, va[i].w, vb[i].w);
+      put(0, lat[i][0].x, lat[i][1].x, lat[i][2].x, lat[i][3].x);
+      put(1, lat[i][0].y, lat[i][1].y, lat[i][2].y, lat[i][3].y);
+      put(2, lat[i][0].z, lat[i][1].z, lat[i][2].z, lat[i][3].z);
+      put(3, lat[i][0].w, lat[i][1].w, lat[i][2].w, lat[i][3].w);
     }
     __syncthreads();
     if (jt + j_step <= i_hi) fetch(jt + j_step);
@@ -268,9 +278,10 @@ latent_tile_kernel(LatentArgs g) {
       }
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct) {
+        const int tile = CT * wave + ct;  // (two pieces of 8 columns)
         Frag vf;
         vf.u = *reinterpret_cast<const uint4*>(
-            s_v + (16 * (CT * wave + ct) + n16) * VS + 32 * kb + 8 * gq);
+            s_v + (16 * tile + n16) * VS + 8 * ((4 * kb + gq) ^ (tile & 7)));
 #pragma unroll
         for (int hg = 0; hg < HG; ++hg) {
           o[ct][hg] = mfma(vf, hi[hg], o[ct][hg]);
@@ -293,12 +304,11 @@ latent_tile_kernel(LatentArgs g) {
     if (r0 + r >= rows) continue;
     float den = (s_max[0][r] + s_max[1][r]) + (s_max[2][r] + s_max[3][r]);
     if (g.splits > 1) {
-      float* out = g.parts + ((size_t)vec[hg] * g.splits + part) * (RP + 2);
+      float* out = g.parts + ((size_t)vec[hg] * g.splits + part) * (RP + 4);
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct)
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-          out[16 * (CT * wave + ct) + 4 * gq + i] = o[ct][hg][i];
+        *reinterpret_cast<float4*>(out + 16 * (CT * wave + ct) + 4 * gq) =
+            make_float4(o[ct][hg][0], o[ct][hg][1], o[ct][hg][2], o[ct][hg][3]);
       if (wave == 0 && gq == 0) {
         out[RP] = mx[hg];
         out[RP + 1] = den;
@@ -322,28 +332,42 @@ latent_tile_kernel(LatentArgs g) {
   }
 }
 
-// The parts of latent_tile_kernel: one wavefront per (token, head).
-__global__ void __launch_bounds__(64)
+// The parts of latent_tile_kernel: one workgroup of RP / 4 threads per (token,
+// head), every part's loads in flight together.
+template <int SPLITS>
+__global__ void __launch_bounds__(128)
 latent_merge_kernel(LatentArgs g) {
   T5D_GATED(g.gate);
   const t5d_latent_attention& a = g.a;
-  const int vec = blockIdx.x, RP = g.RP;
-  const float* p = g.parts + (size_t)vec * g.splits * (RP + 2);
+  const int vec = blockIdx.x, RP = g.RP, stride = RP + 4;
+  const float* p = g.parts + (size_t)vec * SPLITS * stride;
+  const int d = 4 * threadIdx.x;
+  float4 o[SPLITS];
+  float2 ml[SPLITS];
+#pragma unroll
+  for (int s = 0; s < SPLITS; ++s) {
+    o[s] = *reinterpret_cast<const float4*>(p + s * stride + d);
+    ml[s] = *reinterpret_cast<const float2*>(p + s * stride + RP);
+  }
   const float sink2 = a.sink != nullptr ? a.sink[vec % a.H] * kLog2e : kNoMax;
   float top = sink2;
-  for (int s = 0; s < g.splits; ++s) top = fmaxf(top, p[s * (RP + 2) + RP]);
+#pragma unroll
+  for (int s = 0; s < SPLITS; ++s) top = fmaxf(top, ml[s].x);
   float den = a.sink != nullptr ? exp2f(sink2 - top) : 0.f;
-  for (int s = 0; s < g.splits; ++s) {
-    const float f = exp2f(p[s * (RP + 2) + RP] - top);
-    den = fmaf(f, p[s * (RP + 2) + RP + 1], den);
+  float4 num = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+  for (int s = 0; s < SPLITS; ++s) {
+    const float f = exp2f(ml[s].x - top);
+    den = fmaf(f, ml[s].y, den);
+    num.x = fmaf(f, o[s].x, num.x);
+    num.y = fmaf(f, o[s].y, num.y);
+    num.z = fmaf(f, o[s].z, num.z);
+    num.w = fmaf(f, o[s].w, num.w);
   }
-  bf16_t* out = reinterpret_cast<bf16_t*>(a.ol) + (size_t)vec * RP;
-  for (int d = threadIdx.x; d < RP; d += 64) {
-    float num = 0.f;
-    for (int s = 0; s < g.splits; ++s)
-      num = fmaf(exp2f(p[s * (RP + 2) + RP] - top), p[s * (RP + 2) + d], num);
-    out[d] = f32_to_bf16(num / den);
-  }
+  const float inv = 1.0f / den;
+  *reinterpret_cast<uint2*>(reinterpret_cast<bf16_t*>(a.ol) + (size_t)vec * RP + d) =
+      make_uint2(pack_bf16x2(num.x * inv, num.y * inv),
+                 pack_bf16x2(num.z * inv, num.w * inv));
 }
 
 static int tile_groups(int H) { return H > 16 ? 2 : 1; }
@@ -363,14 +387,14 @@ using namespace t5d;
 
 extern "C" int t5d_latent_pad(int rank) {
   if (rank <= 0 || rank > 1024) return -1;
-  for (int p = 64; p <= 512; p *= 2)
+  for (int p = 128; p <= 512; p *= 2)
     if (rank <= p) return p;
   return (rank + 63) / 64 * 64;
 }
 
 extern "C" int64_t t5d_latent_workspace_bytes(int rank) {
   const int rp = t5d_latent_pad(rank);
-  return rp < 0 ? -1 : (int64_t)kMaxParts * 32 * (rp + 2) * 4;
+  return rp < 0 ? -1 : (int64_t)kMaxParts * 32 * (rp + 4) * 4;
 }
 
 #define T5D_TRY(call)        \
@@ -476,12 +500,20 @@ extern "C" int t5d_latent_attention_run(void* stream, const t5d_latent_attention
 #define T5D_LT(DT_, HG_)                                                       \
   if (g.RP == 32 * DT_ && HG == HG_)                                           \
     hipLaunchKernelGGL((latent_tile_kernel<DT_, HG_>), grid, block, 0, s, g)
-    T5D_LT(2, 1); T5D_LT(4, 1); T5D_LT(8, 1); T5D_LT(16, 1);
-    T5D_LT(2, 2); T5D_LT(4, 2); T5D_LT(8, 2); T5D_LT(16, 2);
+    T5D_LT(4, 1); T5D_LT(8, 1); T5D_LT(16, 1);
+    T5D_LT(4, 2); T5D_LT(8, 2); T5D_LT(16, 2);
 #undef T5D_LT
     T5D_CHECK_LAUNCH("latent attention (tile)");
     if (g.splits > 1) {
-      hipLaunchKernelGGL(latent_merge_kernel, dim3(b->M * a->H), dim3(64), 0, s, g);
+      const dim3 mgrid(b->M * a->H), mblock(g.RP / 4);
+      if (g.splits == 2)
+        hipLaunchKernelGGL(latent_merge_kernel<2>, mgrid, mblock, 0, s, g);
+      else if (g.splits == 4)
+        hipLaunchKernelGGL(latent_merge_kernel<4>, mgrid, mblock, 0, s, g);
+      else if (g.splits == 8)
+        hipLaunchKernelGGL(latent_merge_kernel<8>, mgrid, mblock, 0, s, g);
+      else
+        hipLaunchKernelGGL(latent_merge_kernel<16>, mgrid, mblock, 0, s, g);
       T5D_CHECK_LAUNCH("latent attention (merge)");
     }
   } else {

@@ -188,23 +188,6 @@ stream_norm_kernel(StreamNormArgs g) {
 }
 
 // ---- several streams ----------------------------------------------------------------
-// Every stream of a token starts as its scaled embedding.
-template <typename T>
-__global__ void __launch_bounds__(256)
-embed_streams_kernel(const T* __restrict__ table, const int32_t* __restrict__ ids,
-                     float scale, float* __restrict__ out, int d, int ld,
-                     int streams, int V, const int32_t* gate) {
-  T5D_GATED(gate);
-  const int m = blockIdx.x;
-  int id = ids[m];
-  id = id < 0 ? 0 : (id >= V ? V - 1 : id);
-  const T* row = table + (size_t)id * ld;
-  for (int i = threadIdx.x; i < ld; i += 256) {
-    const float v = i < d ? to_f32<T>(row[i]) * scale : 0.f;
-    for (int s = 0; s < streams; ++s) out[((size_t)m * streams + s) * ld + i] = v;
-  }
-}
-
 template <typename T>
 __device__ __forceinline__ float4 load4(const T* p) {
   if constexpr (sizeof(T) == 4) {
@@ -223,6 +206,27 @@ __device__ __forceinline__ void fma4(float4& acc, float w, const float4& v) {
 }
 __device__ __forceinline__ float dot4(const float4& a, const float4& b) {
   return fmaf(a.x, b.x, fmaf(a.y, b.y, fmaf(a.z, b.z, a.w * b.w)));
+}
+
+// Every stream of a token starts as its scaled embedding.  (Columns d .. ld - 1 of
+// the table are zero.)
+template <typename T>
+__global__ void __launch_bounds__(256)
+embed_streams_kernel(const T* __restrict__ table, const int32_t* __restrict__ ids,
+                     float scale, float* __restrict__ out, int ld, int streams,
+                     int V, const int32_t* gate) {
+  T5D_GATED(gate);
+  const int m = blockIdx.x;
+  int id = ids[m];
+  id = id < 0 ? 0 : (id >= V ? V - 1 : id);
+  const T* row = table + (size_t)id * ld;
+  float* dst = out + (size_t)m * streams * ld;
+  for (int c = 4 * threadIdx.x; c < ld; c += 1024) {
+    const float4 e = load4<T>(row + c);
+    const float4 v = make_float4(e.x * scale, e.y * scale, e.z * scale, e.w * scale);
+    for (int s = 0; s < streams; ++s)
+      *reinterpret_cast<float4*>(dst + (size_t)s * ld + c) = v;
+  }
 }
 
 struct HyperArgs {
@@ -416,18 +420,19 @@ extern "C" int t5d_embed_streams(void* stream, int dtype, const void* table,
                                  int d, int ld, int streams, int V) {
   T5D_REQUIRE(dtype == T5D_F32 || dtype == T5D_BF16, T5D_EINVAL,
               "t5d_embed_streams: dtype %d", dtype);
-  T5D_REQUIRE(table && ids && out && M > 0 && d > 0 && ld >= d && V > 0 &&
-                  streams > 0,
+  T5D_REQUIRE(table && ids && out && M > 0 && d > 0 && ld >= d && ld % 4 == 0 &&
+                  V > 0 && streams > 0 &&
+                  (((uintptr_t)table | (uintptr_t)out) % 16) == 0,
               T5D_EINVAL, "t5d_embed_streams: M=%d d=%d ld=%d streams=%d V=%d", M, d,
               ld, streams, V);
   if (dtype == T5D_F32)
     hipLaunchKernelGGL(embed_streams_kernel<float>, dim3(M), dim3(256), 0,
-                       as_stream(stream), (const float*)table, ids, scale, out, d, ld,
+                       as_stream(stream), (const float*)table, ids, scale, out, ld,
                        streams, V, tls_gate);
   else
     hipLaunchKernelGGL(embed_streams_kernel<bf16_t>, dim3(M), dim3(256), 0,
-                       as_stream(stream), (const bf16_t*)table, ids, scale, out, d,
-                       ld, streams, V, tls_gate);
+                       as_stream(stream), (const bf16_t*)table, ids, scale, out, ld,
+                       streams, V, tls_gate);
   T5D_CHECK_LAUNCH("t5d_embed_streams");
   return T5D_OK;
 }

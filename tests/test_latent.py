@@ -138,7 +138,7 @@ def test_spans_cover_what_the_queries_see():
 def test_sizes_and_argument_checks():
   lib = _lib.load()
   assert [lib.t5d_latent_pad(n) for n in (1, 65, 256, 257, 513, 1024, 1025)] == [
-      64, 128, 256, 512, 576, 1024, -1]
+      128, 128, 256, 512, 576, 1024, -1]
   assert lib.t5d_grouped_tile_rows(_lib.F32, 1000, 2) == 8
   assert [lib.t5d_grouped_tile_rows(_lib.BF16, n, 4) for n in
           (3, 64, 65, 256, 257)] == [16, 16, 64, 64, 256]
